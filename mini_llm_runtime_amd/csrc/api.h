@@ -169,7 +169,7 @@ int mlr_paged_attention_simple(const void* q, int64_t q_stride, const void* key_
                                int block_size, int num_pages, float scale, int window, int chunk,
                                const float* sinks, const void* pooled_keys, const void* pooled_values,
                                const int* pooled_table, int pooled_width, int pooled_pages, int pool,
-                               const float* score_bias, hipStream_t stream);
+                               const float* score_bias, float softcap, hipStream_t stream);
 
 // x (float32 [rows, hidden], in place) += weight * y * rsqrt(mean(y^2) + eps), y [rows, hidden] float32
 // or `dtype`, or `slices` float32 partial sums [slices, rows, hidden].  Then mode 1: out = next_weight * x *
@@ -180,6 +180,9 @@ int mlr_add_normed(float* x, const void* y, int y_is_f32, int slices, const void
 
 // out[m, i] = g * sigmoid(alpha * g) * (u + 1), g = min(sums[m, i], limit), u = clamp(sums[m, inter + i],
 // -limit, limit).
+// The stream rounded to bfloat16; gelu(gate) * up of float32 sums [rows, 2 * inter].
+int mlr_round(const float* x, void* out, int64_t count, hipStream_t stream);
+int mlr_glu_gelu(const float* sums, void* out, int dtype, int rows, int inter, hipStream_t stream);
 int mlr_glu_clamped(const void* sums, int sums_is_f32, void* out, int dtype, int rows, int inter, float limit,
                     float alpha, hipStream_t stream);
 
@@ -273,9 +276,10 @@ int mlr_streams_step(float* x, int streams, int tokens, int width, const int* ro
                      hipStream_t stream);
 int mlr_head_norm_rope_write(const float* projected, int width, void* q_out, float* gate, const float* cos,
                              const float* sin, int rotary_dims, float eps, const int* slots, void* key_pages,
-                             void* value_pages, float* v_keep, const float* v_first, const float* lambda, int dtype,
-                             int tokens, int heads, int kv_heads, int dim, int vdim, int kernel_dim, int block_size,
-                             int num_pages, hipStream_t stream);
+                             void* value_pages, float* v_keep, const float* v_first, const float* lambda,
+                             const void* q_weight, const void* k_weight, int weight_is_f32, int dtype, int tokens,
+                             int heads, int kv_heads, int dim, int vdim, int kernel_dim, int block_size, int num_pages,
+                             hipStream_t stream);
 int mlr_matrix_memory_scan(const float* projected, int width, int q_off, int k_off, int v_off, int i_off, int f_off,
                            float* state, int state_rows, const int* read_rows, const int* write_rows, const int* cu_q,
                            const int* q_starts, float cap, float q_scale, float* out, int entries, int heads, int dim,
@@ -304,6 +308,23 @@ int mlr_sample(const float* logits, const float* temperature, const float* unifo
 int64_t mlr_sample_static_capacity();
 int mlr_sample_static(const float* logits, const float* temperature, const float* uniform, int* tokens,
                       int rows, int vocab, hipStream_t stream);
+
+// Recurrences with one decay per head and token behind a short convolution (decay_mixers.hip; the kernels' comments
+// say what each computes).  mlr_decay_scan with `scratch` (mlr_decay_scan_scratch floats, where that is not 0) goes 64
+// tokens at a time on the matrix cores, without it token by token.
+int mlr_conv_gates(const float* projected, int width, int column, const float* taps, const float* bias, float* state,
+                   int state_rows, const int* read_rows, const int* write_rows, const int* token_entry, const int* cu_q,
+                   const int* q_starts, float* out, float* gates, int channels, int n_taps, int unit_heads, int unit_dim,
+                   int scaled_heads, float unit_scale, const float* rate, const float* dt_bias, int heads,
+                   int step_column, int write_column, int tokens, hipStream_t stream);
+int64_t mlr_decay_scan_scratch(int tokens, int entries, int heads, int key_heads, int dim, int vdim, int delta);
+int mlr_decay_scan(const float* x, int channels, int q_off, int k_off, int v_off, const float* gates, float* state,
+                   int state_rows, const int* read_rows, const int* write_rows, const int* cu_q, const int* q_starts,
+                   const float* skip, float* out, int entries, int heads, int key_heads, int dim, int vdim, int tokens,
+                   int delta, float* scratch, int64_t scratch_floats, hipStream_t stream);
+int mlr_gate_group_norm(const float* y, const float* projected, int width, int gate_column, void* out, int dtype,
+                        int tokens, int inner, int groups, float eps, const void* weight, int weight_is_f32,
+                        hipStream_t stream);
 
 // Routed experts (moe.hip).  mlr_moe_route: per token, from the router's float32 logits [tokens,
 // experts]: s = sigmoid(z) (score_kind 0) or softmax(z) over all experts (1), choice scores c = s + correction (float32 [experts], or null); the

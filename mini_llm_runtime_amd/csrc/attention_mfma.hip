@@ -101,6 +101,13 @@ __device__ __forceinline__ float join_sink(const float* __restrict__ sinks, int 
   return keep;
 }
 
+// softcap * tanh(s * scale / softcap) in base 2, for scores s as they leave the product: k1 = 2 log2(e) * scale /
+// softcap, k2 = softcap * log2(e).  tanh(x) = 1 - 2 / (1 + exp(2 x)): 2^inf and 2^-inf give the limits by themselves.
+__device__ __forceinline__ void cap_scores(f32x4_t& s, float k1, float k2) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) s[i] = fmaf(__builtin_amdgcn_rcpf(1.0f + fast_exp2(s[i] * k1)), -2.0f * k2, k2);
+}
+
 // ---- decode ---------------------------------------------------------------------------------
 constexpr int kDecodeWaves = D > 128 ? 2 : 4;  // bounded by the LDS the merge needs
 constexpr int kPartialStride = D + 2;  // numerator[D], max, denominator
@@ -177,7 +184,7 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void attn_decode_kernel(
     const int* __restrict__ cu_q, const int* __restrict__ context_lens, bf16* __restrict__ out,
     float* __restrict__ partial, int heads, int kv_heads, int head_tiles, int block_size, int num_pages,
     float scale, int window, int chunk, int part, int splits, const float* __restrict__ sinks, int keep_partial,
-    const float* __restrict__ score_bias) {
+    const float* __restrict__ score_bias, float softcap) {
   __shared__ float sm_acc[kDecodeWaves][16][D];
   __shared__ float sm_m[kDecodeWaves][16];
   __shared__ float sm_l[kDecodeWaves][16];
@@ -226,7 +233,10 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void attn_decode_kernel(
   // tiles past the end would be loaded all the same) and only then starts on the first.
   // Per tile: scores of both halves, ONE softmax update, one 32-key value product per 16 dims.
   constexpr int kStride = kDecodeWaves * 32;
-  const float scale2 = scale * 1.44269504088896340736f;
+  // softcap: the scores are capped as they leave the product and then are in base 2 already
+  const float cap1 = softcap > 0.f ? 2.0f * 1.44269504088896340736f * scale / softcap : 0.f;
+  const float cap2 = softcap * 1.44269504088896340736f;
+  const float scale2 = softcap > 0.f ? 1.0f : scale * 1.44269504088896340736f;
   // score_bias: no softmax.  A visible key weighs sigmoid(score * scale + bias of the head) whatever the other
   // keys are; the state's maximum stays 0 (so every merge weighs all shares alike) and nothing is divided.
   const bool gated = score_bias != nullptr;
@@ -252,6 +262,7 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void attn_decode_kernel(
 #pragma unroll
       for (int half = 0; half < 2; ++half) {
         sc[half] = score_tile(cur.k[half], qo);
+        if (softcap > 0.f) cap_scores(sc[half], cap1, cap2);
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int key = ts + half * 16 + quarter * 4 + i;
@@ -505,7 +516,7 @@ __global__ __launch_bounds__(256 * kKeyGroups) void attn_prefill_kernel(
     const int* __restrict__ tiles, const int* __restrict__ cu_q, const int* __restrict__ context_lens,
     bf16* __restrict__ out, int num_tiles, int heads, int kv_heads, int bs_shift, int num_pages, float scale,
     int window, int chunk, float* __restrict__ partial, const float* __restrict__ sinks, int keep_partial,
-    const float* __restrict__ score_bias) {
+    const float* __restrict__ score_bias, float softcap) {
   // gridDim.y > 1: the keys of every tile are cut into that many runs, one workgroup each, which
   // leave their unnormalised results in `partial` for attn_prefill_merge (few tiles behind a long
   // context would otherwise be as many long chains on a few compute units).
@@ -590,7 +601,9 @@ __global__ __launch_bounds__(256 * kKeyGroups) void attn_prefill_kernel(
   const int w_min_pos = pos0 + q0 + wave * kWaveQ;
   const int w_max_first = first_visible_key(pos0 + q0 + wave * kWaveQ + kWaveQ - 1, window, chunk);
   // softmax in base 2: exp(x) = exp2(x * log2(e))
-  const float scale2 = scale * 1.44269504088896340736f;
+  const float cap1 = softcap > 0.f ? 2.0f * 1.44269504088896340736f * scale / softcap : 0.f;  // see attn_decode_kernel
+  const float cap2 = softcap * 1.44269504088896340736f;
+  const float scale2 = softcap > 0.f ? 1.0f : scale * 1.44269504088896340736f;
   const bool gated = score_bias != nullptr;  // keys that weigh by themselves, see attn_decode_kernel
   const float bias2 = gated ? score_bias[head] * 1.44269504088896340736f : 0.f;
 
@@ -745,6 +758,13 @@ __global__ __launch_bounds__(256 * kKeyGroups) void attn_prefill_kernel(
 #pragma unroll
         for (int dt = 0; dt < kDimTiles; ++dt) ahead[dt] = value_operand(dt, 0);
         __builtin_amdgcn_sched_barrier(0);
+      }
+      if (softcap > 0.f) {
+        asm volatile("" ::: "memory");
+#pragma unroll
+        for (int b = 0; b < QB; ++b)
+#pragma unroll
+          for (int sub = 0; sub < kSubTiles; ++sub) cap_scores(s[b][sub], cap1, cap2);
       }
       if (!full) {
         // a branch of its own: folded into selects, these comparisons would run for every tile
@@ -992,7 +1012,8 @@ int mlr_attention_decode(const void* q, int64_t q_stride, const void* key_pages,
                          const int* block_table, int table_width, const int* cu_q, const int* context_lens,
                          void* out, float* partial, int entries, int heads, int kv_heads, int block_size,
                          int num_pages, float scale, int window, int chunk, int part, int splits, int merge,
-                         const float* sinks, const float* extra, const float* score_bias, hipStream_t stream) {
+                         const float* sinks, const float* extra, const float* score_bias, float softcap,
+                         hipStream_t stream) {
   MLR_REQUIRE(q && key_pages && value_pages && block_table && cu_q && context_lens && out, "null pointer");
   MLR_REQUIRE(score_bias == nullptr || (sinks == nullptr && extra == nullptr && merge),
               "keys weighed one by one have no sink and no share made elsewhere, and are merged here");
@@ -1009,6 +1030,8 @@ int mlr_attention_decode(const void* q, int64_t q_stride, const void* key_pages,
               "operands must be 16-byte aligned");
   MLR_REQUIRE(scale > 0.f && scale < INFINITY && window >= 0 && chunk >= 0 && !(window > 0 && chunk > 0),
               "bad scale, window or chunk");
+  MLR_REQUIRE(softcap >= 0.f && softcap < INFINITY && (softcap == 0.f || (score_bias == nullptr && extra == nullptr)),
+              "capped scores go with a softmax over the tokens' own keys");
   const int keep_partial = extra != nullptr;
   const int group = heads / kv_heads;
   const int head_tiles = (group + 15) / 16;
@@ -1022,7 +1045,8 @@ int mlr_attention_decode(const void* q, int64_t q_stride, const void* key_pages,
 #define MLR_DECODE(depth)                                                                                       \
   attn_decode_kernel<depth><<<grid, kDecodeWaves * kWave, 0, stream>>>(                                         \
       qp, q_stride, kp, vp, block_table, table_width, cu_q, context_lens, op, partial, heads, kv_heads,         \
-      head_tiles, block_size, num_pages, scale, window, chunk, part, splits, sinks, keep_partial, score_bias)
+      head_tiles, block_size, num_pages, scale, window, chunk, part, splits, sinks, keep_partial, score_bias,   \
+      softcap)
   bool launched = false;
   if constexpr (kMaxDecodeDepth >= 4) {
     if (tiles_per_wave >= 4) {
@@ -1085,7 +1109,7 @@ int mlr_attention_prefill(const void* q, int64_t q_stride, const void* key_pages
                           const int* cu_q, const int* context_lens, void* out, int heads, int kv_heads,
                           int block_size, int num_pages, float scale, int window, int chunk, int splits,
                           float* partial, const float* sinks, const float* extra, const float* score_bias,
-                          hipStream_t stream) {
+                          float softcap, hipStream_t stream) {
   MLR_REQUIRE(splits >= 1 && splits <= 64, "splits must lie within 1..64");
   MLR_REQUIRE(score_bias == nullptr || (sinks == nullptr && extra == nullptr),
               "keys weighed one by one have no sink and no share made elsewhere");
@@ -1106,6 +1130,8 @@ int mlr_attention_prefill(const void* q, int64_t q_stride, const void* key_pages
               "operands must be 16-byte aligned");
   MLR_REQUIRE(scale > 0.f && scale < INFINITY && window >= 0 && chunk >= 0 && !(window > 0 && chunk > 0),
               "bad scale, window or chunk");
+  MLR_REQUIRE(softcap >= 0.f && softcap < INFINITY && (softcap == 0.f || (score_bias == nullptr && extra == nullptr)),
+              "capped scores go with a softmax over the tokens' own keys");
   MLR_REQUIRE(static_cast<int64_t>(num_tiles) * heads < (1ll << 31), "too many tiles for one launch");
   static bool configured = false;
   if (!configured) {
@@ -1133,13 +1159,13 @@ int mlr_attention_prefill(const void* q, int64_t q_stride, const void* key_pages
           static_cast<const bf16*>(q), q_stride, static_cast<const bf16*>(key_pages),                         \
           static_cast<const bf16*>(value_pages), block_table, table_width, tiles, cu_q, context_lens,         \
           static_cast<bf16*>(out), num_tiles, heads, kv_heads, bs_shift, num_pages, scale, window, chunk, partial,  \
-          (splits > 1 || keep_partial) ? nullptr : sinks, keep_partial, score_bias);  \
+          (splits > 1 || keep_partial) ? nullptr : sinks, keep_partial, score_bias, softcap);  \
     else                                                                                                      \
       attn_prefill_kernel<qb, false><<<grid, 256 * kKeyGroups, kPrefillLds, stream>>>(                        \
           static_cast<const bf16*>(q), q_stride, static_cast<const bf16*>(key_pages),                         \
           static_cast<const bf16*>(value_pages), block_table, table_width, tiles, cu_q, context_lens,         \
           static_cast<bf16*>(out), num_tiles, heads, kv_heads, bs_shift, num_pages, scale, window, chunk, partial,  \
-          (splits > 1 || keep_partial) ? nullptr : sinks, keep_partial, score_bias);  \
+          (splits > 1 || keep_partial) ? nullptr : sinks, keep_partial, score_bias, softcap);  \
   } while (0)
   if constexpr (D <= 128) {
     if (wide)

@@ -24,7 +24,7 @@ __global__ __launch_bounds__(64) void paged_attention_simple_kernel(
     int heads, int kv_heads, int head_dim, int block_size, int num_pages, float scale, int window, int chunk,
     const float* __restrict__ sinks, const T* __restrict__ pooled_keys, const T* __restrict__ pooled_values,
     const int* __restrict__ pooled_table, int pooled_width, int pooled_pages, int pool,
-    const float* __restrict__ score_bias) {
+    const float* __restrict__ score_bias, float softcap) {
   __shared__ float qs[MAXD];
   __shared__ float ps[kWave];
   __shared__ int64_t offs[kWave];
@@ -88,7 +88,7 @@ __global__ __launch_bounds__(64) void paged_attention_simple_kernel(
           const T* kp = kpages + off;
           float dot = 0.f;
           for (int i = 0; i < head_dim; ++i) dot = fmaf(qs[i], to_f32(kp[i]), dot);
-          s = dot;
+          s = softcap > 0.f ? softcap * tanhf(dot / softcap) : dot;
         }
       }
       float pr, alpha;
@@ -152,7 +152,7 @@ extern "C" int mlr_paged_attention_simple(const void* q, int64_t q_stride, const
                                           int block_size, int num_pages, float scale, int window, int chunk,
                                           const float* sinks, const void* pooled_keys, const void* pooled_values,
                                           const int* pooled_table, int pooled_width, int pooled_pages, int pool,
-                                          const float* score_bias, hipStream_t stream) {
+                                          const float* score_bias, float softcap, hipStream_t stream) {
   MLR_REQUIRE(q && key_pages && value_pages && block_table && token_entry && positions && out, "null pointer");
   MLR_REQUIRE(tokens > 0 && entries > 0 && heads > 0 && kv_heads > 0, "sizes must be > 0");
   MLR_REQUIRE(heads % kv_heads == 0, "query heads must be a multiple of KV heads");
@@ -167,13 +167,15 @@ extern "C" int mlr_paged_attention_simple(const void* q, int64_t q_stride, const
               "pooled entries need a window, their pages and their table");
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
   MLR_REQUIRE(score_bias == nullptr || (sinks == nullptr && pool == 0), "keys weighed one by one have no sink and no pooled entries");
+  MLR_REQUIRE(softcap >= 0.f && softcap < INFINITY && (softcap == 0.f || (score_bias == nullptr && pool == 0)),
+              "capped scores go with a softmax over the tokens' own keys");
   dim3 grid(tokens, heads);
 #define MLR_SIMPLE(T, MAXD)                                                                                      \
   paged_attention_simple_kernel<T, MAXD><<<grid, kWave, 0, stream>>>(                                            \
       static_cast<const T*>(q), q_stride, static_cast<const T*>(key_pages), static_cast<const T*>(value_pages),   \
       block_table, table_width, token_entry, positions, static_cast<T*>(out), entries, heads, kv_heads, head_dim, \
       block_size, num_pages, scale, window, chunk, sinks, static_cast<const T*>(pooled_keys),                    \
-      static_cast<const T*>(pooled_values), pooled_table, pooled_width, pooled_pages, pool, score_bias)
+      static_cast<const T*>(pooled_values), pooled_table, pooled_width, pooled_pages, pool, score_bias, softcap)
   if (head_dim > 256) {
     if (dtype == kF32)
       MLR_SIMPLE(float, kMaxHeadDim);
@@ -188,14 +190,14 @@ extern "C" int mlr_paged_attention_simple(const void* q, int64_t q_stride, const
         static_cast<const float*>(value_pages), block_table, table_width, token_entry, positions,
         static_cast<float*>(out), entries, heads, kv_heads, head_dim, block_size, num_pages, scale, window, chunk,
         sinks, static_cast<const float*>(pooled_keys), static_cast<const float*>(pooled_values), pooled_table,
-        pooled_width, pooled_pages, pool, score_bias);
+        pooled_width, pooled_pages, pool, score_bias, softcap);
   else
     paged_attention_simple_kernel<bf16, 256><<<grid, kWave, 0, stream>>>(
         static_cast<const bf16*>(q), q_stride, static_cast<const bf16*>(key_pages),
         static_cast<const bf16*>(value_pages), block_table, table_width, token_entry, positions,
         static_cast<bf16*>(out), entries, heads, kv_heads, head_dim, block_size, num_pages, scale, window, chunk,
         sinks, static_cast<const bf16*>(pooled_keys), static_cast<const bf16*>(pooled_values), pooled_table,
-        pooled_width, pooled_pages, pool, score_bias);
+        pooled_width, pooled_pages, pool, score_bias, softcap);
   MLR_LAUNCH_CHECK();
   return 0;
 }

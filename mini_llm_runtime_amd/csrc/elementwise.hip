@@ -201,6 +201,33 @@ __global__ __launch_bounds__(256) void silu_mul_kernel(const T* __restrict__ gat
   out[i] = from_f32<T>(s * u);
 }
 
+// The 32-bit stream rounded to bfloat16, for sublayers that read it un-normed.
+__global__ __launch_bounds__(256) void round_kernel(const float* __restrict__ x, bf16* __restrict__ out, int64_t n) {
+  const int64_t i = (static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x) * 4;
+  if (i + 3 < n) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(x + i);
+    uint2 packed;
+    packed.x = pack_bf16x2(v[0], v[1]);
+    packed.y = pack_bf16x2(v[2], v[3]);
+    *reinterpret_cast<uint2*>(out + i) = packed;
+  } else {
+    for (int64_t j = i; j < n; ++j) out[j] = f32_to_bf16(x[j]);
+  }
+}
+
+// gelu(gate) * up of float32 sums [rows, 2 * inter] (gate sums, then up sums), the tanh form of the GELU.
+template <typename T>
+__global__ __launch_bounds__(256) void glu_gelu_kernel(const float* __restrict__ sums, T* __restrict__ out, int rows,
+                                                       int inter) {
+  const int64_t i = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+  if (i >= static_cast<int64_t>(rows) * inter) return;
+  const int64_t m = i / inter;
+  const int64_t c = i - m * inter;
+  const float g = sums[m * 2 * inter + c];
+  const float u = sums[m * 2 * inter + inter + c];
+  out[i] = from_f32<T>(0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u);
+}
+
 // ---- rotary tables -------------------------------------------------------------------
 // qwen_model_runner.py:45-57: angle = position * inv_freq[j]; here the product and
 // its cosine and sine are evaluated in float64 and rounded once to float32.
@@ -518,6 +545,28 @@ int mlr_gather_rows(const void* src, const int* rows, void* out, int count, int6
   MLR_REQUIRE(row_bytes > 0 && row_bytes % 4 == 0, "rows must be a multiple of 4 bytes wide");
   gather_rows_kernel<<<dim3(count, planes), 256, 0, stream>>>(static_cast<const uint32_t*>(src), rows,
                                                 static_cast<uint32_t*>(out), row_bytes / 4, src_rows);
+  MLR_LAUNCH_CHECK();
+  return 0;
+}
+
+int mlr_round(const float* x, void* out, int64_t count, hipStream_t stream) {
+  MLR_REQUIRE(x && out, "null pointer");
+  MLR_REQUIRE(count > 0 && (count + 1023) / 1024 < (1ll << 31), "bad element count");
+  round_kernel<<<static_cast<unsigned>((count + 1023) / 1024), 256, 0, stream>>>(x, static_cast<bf16*>(out), count);
+  MLR_LAUNCH_CHECK();
+  return 0;
+}
+
+int mlr_glu_gelu(const float* sums, void* out, int dtype, int rows, int inter, hipStream_t stream) {
+  MLR_REQUIRE(sums && out, "null pointer");
+  MLR_REQUIRE(rows > 0 && inter > 0, "sizes must be > 0");
+  MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
+  const int64_t blocks = (static_cast<int64_t>(rows) * inter + 255) / 256;
+  MLR_REQUIRE(blocks < (1ll << 31), "too many elements");
+  if (dtype == kF32)
+    glu_gelu_kernel<float><<<static_cast<unsigned>(blocks), 256, 0, stream>>>(sums, static_cast<float*>(out), rows, inter);
+  else
+    glu_gelu_kernel<bf16><<<static_cast<unsigned>(blocks), 256, 0, stream>>>(sums, static_cast<bf16*>(out), rows, inter);
   MLR_LAUNCH_CHECK();
   return 0;
 }

@@ -40,8 +40,9 @@ constexpr int kEpNone = 0;
 constexpr int kEpSwiglu = 1;
 constexpr int kEpRelu2 = 2;
 constexpr int kEpSigmoid = 3;
-constexpr int kEpGeluTanh = 4;
-constexpr int kEpClampedGlu = 5;  // 0.5 v (1 + tanh(sqrt(2 / pi) (v + 0.044715 v^3)))
+constexpr int kEpGeluTanh = 4;  // 0.5 v (1 + tanh(sqrt(2 / pi) (v + 0.044715 v^3)))
+constexpr int kEpClampedGlu = 5;
+constexpr int kEpGeglu = 6;  // woven as for kEpSwiglu (and the bias with it): stores gelu(gate) * up, the GELU of kEpGeluTanh
 
 // The scaling factors of rows m0 .. m0 + count - 1 into `scales` (LDS), by all wavefronts of the
 // workgroup (a whole number of them): wavefront w takes the rows w, w + waves, ..., its lanes the
@@ -116,6 +117,11 @@ __device__ __forceinline__ void row_scales_finish(const GemmEpilogue& ep, const 
 }
 
 __device__ __forceinline__ float silu(float g) { return g / (1.0f + __expf(-g)); }
+// 0.5 (1 + tanh(u)) = 1 / (1 + exp(-2 u))
+__device__ __forceinline__ float gelu_tanh(float v) {
+  const float u = 0.7978845608028654f * (v + 0.044715f * v * v * v);
+  return v / (1.0f + __expf(-2.0f * u));
+}
 
 // Store four consecutive output features n..n+3 of token m (n is a multiple of 4).
 // ACTIVATIONS false leaves the element-wise activations and the multiplier out: for the one kernel
@@ -126,7 +132,7 @@ __device__ __forceinline__ void store4(const GemmEpilogue& ep, int64_t m, int n,
                                        float v2, float v3) {
   float v[4] = {v0, v1, v2, v3};
   bool paired = ep.swiglu == kEpSwiglu;
-  if constexpr (ACTIVATIONS) paired = paired || ep.swiglu == kEpClampedGlu;
+  if constexpr (ACTIVATIONS) paired = paired || ep.swiglu == kEpClampedGlu || ep.swiglu == kEpGeglu;
   if (paired) {
     // n..n+3 = gate 2j, gate 2j+1, up 2j, up 2j+1 with j = n / 4; N is a multiple of 4
     const int64_t at = m * (N / 2) + n / 2;
@@ -139,10 +145,15 @@ __device__ __forceinline__ void store4(const GemmEpilogue& ep, int64_t m, int n,
 #pragma unroll
         for (int i = 0; i < 4; ++i) v[i] += load_as_f32(ep.bias, n + i, ep.bias_is_f32);
       }
-      const float g0 = fminf(v[0], ep.glu_limit), g1 = fminf(v[1], ep.glu_limit);
-      const float u0 = fminf(fmaxf(v[2], -ep.glu_limit), ep.glu_limit), u1 = fminf(fmaxf(v[3], -ep.glu_limit), ep.glu_limit);
-      a = g0 / (1.0f + __expf(-ep.glu_alpha * g0)) * (u0 + 1.0f);
-      b = g1 / (1.0f + __expf(-ep.glu_alpha * g1)) * (u1 + 1.0f);
+      if (ep.swiglu == kEpGeglu) {
+        a = gelu_tanh(v[0]) * v[2];
+        b = gelu_tanh(v[1]) * v[3];
+      } else {
+        const float g0 = fminf(v[0], ep.glu_limit), g1 = fminf(v[1], ep.glu_limit);
+        const float u0 = fminf(fmaxf(v[2], -ep.glu_limit), ep.glu_limit), u1 = fminf(fmaxf(v[3], -ep.glu_limit), ep.glu_limit);
+        a = g0 / (1.0f + __expf(-ep.glu_alpha * g0)) * (u0 + 1.0f);
+        b = g1 / (1.0f + __expf(-ep.glu_alpha * g1)) * (u1 + 1.0f);
+      }
     }
     if (ep.out_is_f32) {
       float* y = static_cast<float*>(ep.y) + at;
@@ -173,11 +184,7 @@ __device__ __forceinline__ void store4(const GemmEpilogue& ep, int64_t m, int n,
       for (int i = 0; i < 4; ++i) v[i] = 1.0f / (1.0f + __expf(-v[i]));
     } else if (ep.swiglu == kEpGeluTanh) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        // 0.5 (1 + tanh(u)) = 1 / (1 + exp(-2 u))
-        const float u = 0.7978845608028654f * (v[i] + 0.044715f * v[i] * v[i] * v[i]);
-        v[i] = v[i] / (1.0f + __expf(-2.0f * u));
-      }
+      for (int i = 0; i < 4; ++i) v[i] = gelu_tanh(v[i]);
     }
     if (ep.multiply != nullptr) {
       const bf16* other = static_cast<const bf16*>(ep.multiply) +

@@ -1134,15 +1134,16 @@ int mlr_gemm_bf16_kernel(int m, int n, int k, int slices) { return choose_kernel
 // bias), and `multiply` (bfloat16 [m, n], or null) is multiplied into the activated sums; with
 // `multiply_rows` (int32 [m]) row i takes row multiply_rows[i] of `multiply` (a table [rows, n]).
 // `swiglu` 5: rows (and bias) woven as for 1, y [m, n / 2] = g * sigmoid(glu_alpha g) * (u + 1) with
-// g = min(gate, glu_limit), u = clamp(up, -glu_limit, glu_limit).
+// g = min(gate, glu_limit), u = clamp(up, -glu_limit, glu_limit); 6: woven likewise, y = gelu(gate) * up (tanh form).
 int mlr_gemm_bf16(const void* x, const void* w, const void* bias, int bias_is_f32, void* y, int out_is_f32,
                   int swiglu, int slices, int kernel, int m, int n, int k, const float* row_sumsq, int sumsq_parts,
                   float norm_eps, const void* multiply, const int* multiply_rows, float glu_limit, float glu_alpha,
                   hipStream_t stream) {
   MLR_REQUIRE(x && w && y, "null pointer");
-  MLR_REQUIRE(swiglu >= kEpNone && swiglu <= kEpClampedGlu, "unknown epilogue");
+  MLR_REQUIRE(swiglu >= kEpNone && swiglu <= kEpGeglu, "unknown epilogue");
   MLR_REQUIRE(swiglu != kEpClampedGlu || (n % 4 == 0 && multiply == nullptr && glu_limit > 0.f),
               "the clamped gating needs n % 4 == 0, a limit > 0 and no multiplier");
+  MLR_REQUIRE(swiglu != kEpGeglu || (n % 4 == 0 && multiply == nullptr), "the GELU gating needs n % 4 == 0 and no multiplier");
   MLR_REQUIRE(multiply == nullptr || (swiglu != kEpSwiglu && slices == 1), "a multiplier goes with whole, unpaired sums");
   MLR_REQUIRE(slices == 1 || swiglu == kEpNone, "partial sums take no activation");
   MLR_REQUIRE(m > 0 && n > 0 && k > 0, "sizes must be > 0");

@@ -68,8 +68,9 @@ __global__ __launch_bounds__(256) void gemm_simple_kernel(const T* __restrict__ 
   for (int i = 0; i < 4; ++i) {
     const int64_t gm = m0 + tm * 4 + i;
     if (gm >= M) continue;
-    if (swiglu == 5) {
-      // columns as for swiglu 1, the bias woven with them: g sigmoid(alpha g) (u + 1), both halves clamped
+    if (swiglu == 5 || swiglu == 6) {
+      // columns as for swiglu 1, the bias woven with them: g sigmoid(alpha g) (u + 1), both halves clamped, or (6)
+      // gelu(g) u
       const int64_t gn = n0 + tn * 4;
       if (gn >= N) continue;
       const int64_t at = gm * (N / 2) + gn / 2;
@@ -80,9 +81,14 @@ __global__ __launch_bounds__(256) void gemm_simple_kernel(const T* __restrict__ 
           g += load_as_f32(bias, gn + j, bias_is_f32);
           u += load_as_f32(bias, gn + j + 2, bias_is_f32);
         }
-        g = fminf(g, glu_limit);
-        u = fminf(fmaxf(u, -glu_limit), glu_limit);
-        const float v = g / (1.0f + expf(-glu_alpha * g)) * (u + 1.0f);
+        float v;
+        if (swiglu == 6) {
+          v = 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
+        } else {
+          g = fminf(g, glu_limit);
+          u = fminf(fmaxf(u, -glu_limit), glu_limit);
+          v = g / (1.0f + expf(-glu_alpha * g)) * (u + 1.0f);
+        }
         if (out_is_f32)
           static_cast<float*>(y)[at + j] = v;
         else
@@ -143,11 +149,12 @@ extern "C" int mlr_gemm_simple(const void* x, const void* w, const void* bias, i
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
   MLR_REQUIRE(dtype == kBF16 || (out_is_f32 && (bias == nullptr || bias_is_f32)),
               "a float32 product has float32 bias and output");
-  MLR_REQUIRE(swiglu >= 0 && swiglu <= 5, "unknown epilogue");
+  MLR_REQUIRE(swiglu >= 0 && swiglu <= 6, "unknown epilogue");
   MLR_REQUIRE(swiglu != 1 || (n % 4 == 0 && bias == nullptr && multiply == nullptr),
               "swiglu needs n % 4 == 0, no bias and no multiplier");
   MLR_REQUIRE(swiglu != 5 || (n % 4 == 0 && multiply == nullptr && glu_limit > 0.f),
               "the clamped gating needs n % 4 == 0, a limit > 0 and no multiplier");
+  MLR_REQUIRE(swiglu != 6 || (n % 4 == 0 && multiply == nullptr), "the GELU gating needs n % 4 == 0 and no multiplier");
   dim3 grid((n + kTN - 1) / kTN, (m + kTM - 1) / kTM);
   MLR_REQUIRE(grid.y < 65536u, "too many rows for one launch");
   if (dtype == kF32)

@@ -197,13 +197,16 @@ __global__ __launch_bounds__(256) void streams_fill_kernel(const float* __restri
 //    kv_heads * vdim]; (v_first) v = (1 - lambda) v + lambda v_first[t]; values to [page, kv_head, D, offset];
 //  * gate[t, head] = sigmoid(logit).
 // One wavefront per head; a negative slot stores nothing.
+// q_weight given (and k_weight [dim], with keys): a head is divided by its root mean square and multiplied by that
+// weight BEFORE it turns, and the values are stored as they are.  kv_heads 0: the rows hold queries only.
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
     const float* __restrict__ p, int width, T* __restrict__ q_out, float* __restrict__ gate,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rdims, float eps,
     const int* __restrict__ slots, T* __restrict__ key_pages, T* __restrict__ value_pages, float* __restrict__ v_keep,
-    const float* __restrict__ v_first, const float* __restrict__ lambda_p, int heads, int kv_heads, int dim, int vdim,
-    int D, int block_size, int num_pages) {
+    const float* __restrict__ v_first, const float* __restrict__ lambda_p, const void* __restrict__ q_weight,
+    const void* __restrict__ k_weight, int weight_is_f32, int heads, int kv_heads, int dim, int vdim, int D, int block_size,
+    int num_pages) {
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x % kWave;
   const int wave = threadIdx.x / kWave;
@@ -211,7 +214,7 @@ __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
   const int half = rdims / 2;
   const float* cs = cos_t != nullptr ? cos_t + t * half : nullptr;
   const float* sn = sin_t != nullptr ? sin_t + t * half : nullptr;
-  const int slot = slots[t];
+  const int slot = kv_heads > 0 ? slots[t] : -1;
   const int page = slot >= 0 ? slot / block_size : -1;
   const int off = slot >= 0 ? slot - page * block_size : 0;
   const bool store = page >= 0 && page < num_pages;
@@ -223,6 +226,32 @@ __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
     const int h = is_q ? job : (is_k ? job - heads : job - heads - kv_heads);
     const int n = (is_q || is_k) ? dim : vdim;
     const float* src = row + (is_q ? h * dim : (is_k ? heads * dim + h * dim : (heads + kv_heads) * dim + h * vdim));
+    if (q_weight != nullptr) {
+      float inv = 1.0f;
+      if (is_q || is_k) {
+        float ss = 0.f;
+        for (int j = lane; j < n; j += kWave) ss += src[j] * src[j];
+        inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(n) + eps);
+      }
+      const void* w = is_q ? q_weight : k_weight;
+      auto normed = [&](int j) { return src[j] * inv * load_as_f32(w, j, weight_is_f32); };
+      auto turned = [&](int j) {
+        if (j >= rdims || cs == nullptr) return normed(j);
+        return j < half ? normed(j) * cs[j] - normed(j + half) * sn[j]
+                        : normed(j) * cs[j - half] + normed(j - half) * sn[j - half];
+      };
+      if (is_q) {
+        T* dst = q_out + (t * heads + h) * D;
+        for (int j = lane; j < D; j += kWave) dst[j] = from_f32<T>(j < n ? turned(j) : 0.f);
+      } else if (store && is_k) {
+        T* dst = key_pages + ((static_cast<int64_t>(page) * kv_heads + h) * block_size + off) * D;
+        for (int j = lane; j < D; j += kWave) dst[j] = from_f32<T>(j < n ? turned(j) : 0.f);
+      } else if (store) {
+        T* dst = value_pages + (static_cast<int64_t>(page) * kv_heads + h) * D * block_size + off;
+        for (int j = lane; j < D; j += kWave) dst[static_cast<int64_t>(j) * block_size] = from_f32<T>(j < n ? src[j] : 0.f);
+      }
+      continue;
+    }
     auto value = [&](int j) {
       if (!(is_q || is_k) || j >= rdims || cs == nullptr) return src[j];
       return j < half ? src[j] * cs[j] - src[j + half] * sn[j] : src[j] * cs[j - half] + src[j - half] * sn[j - half];
@@ -572,28 +601,30 @@ int mlr_streams_step(float* x, int streams, int tokens, int width, const int* ro
 
 int mlr_head_norm_rope_write(const float* projected, int width, void* q_out, float* gate, const float* cos,
                              const float* sin, int rotary_dims, float eps, const int* slots, void* key_pages,
-                             void* value_pages, float* v_keep, const float* v_first, const float* lambda, int dtype,
-                             int tokens, int heads, int kv_heads, int dim, int vdim, int kernel_dim, int block_size,
+                             void* value_pages, float* v_keep, const float* v_first, const float* lambda, const void* q_weight,
+                             const void* k_weight, int weight_is_f32, int dtype, int tokens, int heads, int kv_heads, int dim, int vdim, int kernel_dim, int block_size,
                              int num_pages, hipStream_t stream) {
-  MLR_REQUIRE(projected && q_out && slots && key_pages && value_pages, "null pointer");
-  MLR_REQUIRE(tokens > 0 && heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0, "sizes must be > 0");
+  MLR_REQUIRE(projected && q_out && (kv_heads == 0 || (slots && key_pages && value_pages)), "null pointer");
+  MLR_REQUIRE(tokens > 0 && heads > 0 && kv_heads >= 0 && dim > 0 && vdim > 0, "sizes must be > 0");
+  MLR_REQUIRE(q_weight == nullptr || ((kv_heads == 0 || k_weight) && !v_keep && !v_first),
+              "weighted head norms come for queries and keys and leave the values as they are");
   MLR_REQUIRE(kernel_dim >= dim && kernel_dim >= vdim, "the kernels' head size must hold keys and values");
   MLR_REQUIRE(rotary_dims >= 0 && rotary_dims % 2 == 0 && rotary_dims <= dim, "rotary_dims must be even and within dim");
   MLR_REQUIRE(rotary_dims == 0 || (cos && sin), "a rotation needs cos and sin tables");
   MLR_REQUIRE(width >= (heads + kv_heads) * dim + kv_heads * vdim + (gate ? heads : 0), "the projected rows are too narrow");
   MLR_REQUIRE(v_first == nullptr || lambda, "mixing values in needs its weight");
-  MLR_REQUIRE(block_size > 0 && num_pages > 0, "page sizes must be > 0");
+  MLR_REQUIRE(kv_heads == 0 || (block_size > 0 && num_pages > 0), "page sizes must be > 0");
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
   if (dtype == kF32)
     head_norm_rope_write_kernel<float><<<tokens, 256, 0, stream>>>(
         projected, width, static_cast<float*>(q_out), gate, cos, sin, rotary_dims, eps, slots,
-        static_cast<float*>(key_pages), static_cast<float*>(value_pages), v_keep, v_first, lambda, heads, kv_heads, dim,
-        vdim, kernel_dim, block_size, num_pages);
+        static_cast<float*>(key_pages), static_cast<float*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight,
+        weight_is_f32, heads, kv_heads, dim, vdim, kernel_dim, block_size, num_pages);
   else
     head_norm_rope_write_kernel<bf16><<<tokens, 256, 0, stream>>>(
         projected, width, static_cast<bf16*>(q_out), gate, cos, sin, rotary_dims, eps, slots,
-        static_cast<bf16*>(key_pages), static_cast<bf16*>(value_pages), v_keep, v_first, lambda, heads, kv_heads, dim,
-        vdim, kernel_dim, block_size, num_pages);
+        static_cast<bf16*>(key_pages), static_cast<bf16*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight,
+        weight_is_f32, heads, kv_heads, dim, vdim, kernel_dim, block_size, num_pages);
   MLR_LAUNCH_CHECK();
   return 0;
 }

@@ -68,6 +68,7 @@ CORE = Module(
         "mixers.hip",
         "side_mixers.hip",
         "stream_mixers.hip",
+        "decay_mixers.hip",
         "sampling.hip",
     ),
 )

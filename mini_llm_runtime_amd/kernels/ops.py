@@ -30,6 +30,18 @@ _SIGNATURES = {
     "mlr_version": ([], _I),
     "mlr_embedding": ([_VP, _I, _VP, _VP, _I, _I, _I, _I, _VP], _I),
     "mlr_add_normed": ([_VP, _VP, _I, _I, _VP, _I, _F, _VP, _I, _F, _I, _VP, _I, _I, _I, _VP], _I),
+    "mlr_round": ([_VP, _VP, _I64, _VP], _I),
+    "mlr_glu_gelu": ([_VP, _VP, _I, _I, _I, _VP], _I),
+    "mlr_conv_gates": (
+        [_VP, _I, _I, _VP, _VP, _VP, _I, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _VP, _VP, _I, _I, _I, _I,
+         _VP],
+        _I,
+    ),
+    "mlr_decay_scan": (
+        [_VP, _I, _I, _I, _I, _VP, _VP, _I, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _VP, _I64, _VP], _I,
+    ),
+    "mlr_decay_scan_scratch": ([_I, _I, _I, _I, _I, _I, _I], _I64),
+    "mlr_gate_group_norm": ([_VP, _VP, _I, _I, _VP, _I, _I, _I, _I, _F, _VP, _I, _VP], _I),
     "mlr_glu_clamped": ([_VP, _I, _VP, _I, _I, _I, _F, _F, _VP], _I),
     "mlr_latent_prepare": (
         [_VP, _I, _VP, _VP, _VP, _VP, _VP, _I, _VP, _I, _F, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _VP,
@@ -39,7 +51,9 @@ _SIGNATURES = {
     "mlr_streams_fill": ([_VP, _VP, _I, _I, _I, _VP], _I),
     "mlr_streams_step": ([_VP, _I, _I, _I, _VP, _I, _VP, _I, _I, _VP, _VP, _VP, _VP, _I, _F, _VP, _VP, _I, _VP], _I),
     "mlr_head_norm_rope_write": (
-        [_VP, _I, _VP, _VP, _VP, _VP, _I, _F, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _I, _VP], _I,
+        [_VP, _I, _VP, _VP, _VP, _VP, _I, _F, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I,
+         _VP],
+        _I,
     ),
     "mlr_matrix_memory_scan": (
         [_VP, _I, _I, _I, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _F, _F, _VP, _I, _I, _I, _I, _I, _VP, _VP, _VP], _I,
@@ -99,7 +113,7 @@ _SIGNATURES = {
     "mlr_gemm_merge_fused_bf16": ([_VP, _VP, _I, _I, _I, _I, _I, _VP, _VP, _I, _VP, _I, _I, _I, _I, _VP], _I),
     "mlr_paged_attention_simple": (
         [_VP, _I64, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _VP, _VP, _VP, _VP,
-         _I, _I, _I, _VP, _VP],
+         _I, _I, _I, _VP, _F, _VP],
         _I,
     ),
     "mlr_sample": ([_VP, _VP, _VP, _VP, _VP, _I, _I, _VP], _I),
@@ -109,19 +123,21 @@ _SIGNATURES = {
     "mlr_attention_wide_tile": ([], _I),
     "mlr_attention_decode_scratch": ([_I, _I, _I], _I64),
     "mlr_attention_decode": (
-        [_VP, _I64, _VP, _VP, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _VP, _VP, _VP, _VP],
+        [_VP, _I64, _VP, _VP, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _VP, _VP, _VP, _F,
+         _VP],
         _I,
     ),
     "mlr_attention_decode_merge": ([_VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _VP, _VP], _I),
     "mlr_attention_prefill_scratch": ([_I, _I, _I, _I], _I64),
     "mlr_attention_prefill": (
-        [_VP, _I64, _VP, _VP, _VP, _I, _VP, _I, _I, _VP, _VP, _VP, _I, _I, _I, _I, _F, _I, _I, _I, _VP, _VP, _VP, _VP, _VP],
+        [_VP, _I64, _VP, _VP, _VP, _I, _VP, _I, _I, _VP, _VP, _VP, _I, _I, _I, _I, _F, _I, _I, _I, _VP, _VP, _VP, _VP, _F,
+         _VP],
         _I,
     ),
 }
 
 # what `linear` may do to its sums before it stores them (the entry points' `swiglu` argument)
-_EPILOGUES = {None: 0, "swiglu": 1, "relu2": 2, "sigmoid": 3, "gelu_tanh": 4, "clamped_glu": 5}
+_EPILOGUES = {None: 0, "swiglu": 1, "relu2": 2, "sigmoid": 3, "gelu_tanh": 4, "clamped_glu": 5, "geglu": 6}
 
 from .plans import PAGED_ATTENTION, QUERY_TILE, WIDE_QUERY_TILE, attention_plan, query_tiles  # noqa: F401
 
@@ -509,12 +525,15 @@ class HipOps:
         multiply: Optional[torch.Tensor] = None,
         clamped_glu: Optional[tuple[float, float]] = None,
         multiply_rows: Optional[torch.Tensor] = None,
+        geglu: bool = False,
     ) -> torch.Tensor:
         """x [M, K] times weight [N, K] transposed, plus bias [N]; F.linear semantics.
 
         clamped_glu: (limit, alpha).  The rows of `weight` (and the bias with them) are woven as for `swiglu`
         (gate 2j, gate 2j+1, up 2j, up 2j+1) and the result is g * sigmoid(alpha g) * (u + 1), [M, N / 2], with
         g = min(gate, limit) and u = clamp(up, -limit, limit): the pairing's other gating, with a bias.
+
+        geglu: rows and bias woven likewise; the result is gelu(gate) * up, [M, N / 2], with the tanh form of the GELU.
 
         activation: "relu2" (max(v, 0)^2) or "sigmoid", applied to the sums (after the bias) in the
         product's epilogue, in 32-bit, before the one rounding to the output's dtype.
@@ -540,7 +559,7 @@ class HipOps:
         """
         if kernel not in ("auto", "fma"):
             raise KernelError("kernel must be 'auto' or 'fma'")
-        if activation not in _EPILOGUES or activation in ("swiglu", "clamped_glu"):
+        if activation not in _EPILOGUES or activation in ("swiglu", "clamped_glu", "geglu"):
             raise KernelError(f"unknown activation {activation!r}")
         glu_limit = glu_alpha = 0.0
         if clamped_glu is not None:
@@ -550,11 +569,18 @@ class HipOps:
             if not glu_limit > 0:
                 raise KernelError("the clamped gating needs a limit > 0")
             x = self.settle(x)  # no fused prologue knows this pairing
+        if geglu:
+            if (
+                swiglu or clamped_glu is not None or activation is not None or multiply is not None or partial_sums or for_stream
+                or slices not in (None, 1)
+            ):
+                raise KernelError("the GELU gating goes with whole sums and nothing else")
+            x = self.settle(x)
         if (activation is not None or multiply is not None) and (swiglu or partial_sums or for_stream or slices not in (None, 1)):
             raise KernelError("an activation or a multiplier goes with whole sums: no SwiGLU pairing, no slices of k")
         epilogue = 1 if swiglu else _EPILOGUES[activation]
-        if clamped_glu is not None:
-            epilogue = _EPILOGUES["clamped_glu"]
+        if clamped_glu is not None or geglu:
+            epilogue = _EPILOGUES["geglu" if geglu else "clamped_glu"]
             swiglu = True  # for the shape of the result; the bias check below is the pairing-without-bias one
         if for_stream:
             partial_sums = True
@@ -583,7 +609,7 @@ class HipOps:
         n = weight.shape[0]
         if bias is not None:
             self._check(bias, "linear bias", (torch.float32, self.dtype), (n,))
-        if swiglu and (n % 4 or (bias is not None and clamped_glu is None)):
+        if swiglu and (n % 4 or (bias is not None and clamped_glu is None and not geglu)):
             raise KernelError("a SwiGLU product needs a multiple of 4 rows and no bias")
         out_dtype = out_dtype or self.dtype
         if out_dtype not in (torch.float32, self.dtype):
@@ -673,6 +699,25 @@ class HipOps:
             int(slices > 1 or out_dtype == torch.float32), slices, m, n, self._stream(),
         )
         return y
+
+    def rounded(self, x: torch.Tensor) -> torch.Tensor:
+        """The residual stream x (float32) in the engine's dtype; x itself where that is float32."""
+        self._check(x, "residual stream", torch.float32)
+        if self.dtype == torch.float32:
+            return x
+        out = self._empty(x.shape, self.dtype)
+        self._call("mlr_round", self._ptr(x), self._ptr(out), x.numel(), self._stream())
+        return out
+
+    def glu_gelu(self, sums: torch.Tensor) -> torch.Tensor:
+        """sums float32 [rows, 2 * inter] (gate sums, then up sums) -> gelu(gate) * up [rows, inter] (tanh form)."""
+        self._check(sums, "gate and up sums", torch.float32, (None, None))
+        rows, width = sums.shape
+        if width % 2:
+            raise KernelError("gate and up sums must have an even width")
+        out = self._empty((rows, width // 2), self.dtype)
+        self._call("mlr_glu_gelu", self._ptr(sums), self._ptr(out), self.code, rows, width // 2, self._stream())
+        return out
 
     def silu_mul(self, gate_up: torch.Tensor) -> torch.Tensor:
         self._check(gate_up, "gate_up", self.dtype, (None, None))
@@ -909,8 +954,11 @@ class HipOps:
         sinks: Optional[torch.Tensor] = None,
         pooled: Optional[tuple] = None,
         score_bias: Optional[torch.Tensor] = None,
+        softcap: Optional[float] = None,
     ):
         """Causal attention of the step's tokens over their requests' pages.
+
+        softcap: the scaled score s becomes softcap * tanh(s / softcap) before the softmax.
 
         score_bias: float32 [num_heads]; no softmax then: a visible key weighs sigmoid(score * scale +
         score_bias[head]) whatever the other keys are, and the weights are not normalised.
@@ -964,6 +1012,12 @@ class HipOps:
             self._check(score_bias, "score bias", torch.float32, (num_heads,))
             if sinks is not None or pooled is not None:
                 raise KernelError("keys weighed one by one have no sink and no pooled entries")
+        cap = float(softcap or 0.0)
+        if softcap is not None:
+            if not cap > 0:
+                raise KernelError("a soft cap must be > 0")
+            if score_bias is not None or pooled is not None:
+                raise KernelError("capped scores go with a softmax over the tokens' own keys")
         out = self._empty((tokens, num_heads * head_dim), self.dtype)
         width = block_table.shape[1]
         pooled_keys = pooled_values = pooled_table = None
@@ -1002,7 +1056,7 @@ class HipOps:
                 self._ptr(out), self.code, tokens, entries, num_heads, num_kv_heads, head_dim, block_size,
                 num_pages, float(scale), int(window or 0), chunk, self._ptr(sinks), self._ptr(pooled_keys),
                 self._ptr(pooled_values), self._ptr(pooled_table), pooled_width, pooled_pages, pool,
-                self._ptr(score_bias), self._stream(),
+                self._ptr(score_bias), cap, self._stream(),
             )
             return out
         self._check(ctx.cu_q, "cu_q", torch.int32, (entries + 1,))
@@ -1045,7 +1099,7 @@ class HipOps:
                 self._ptr(block_table), width, self._ptr(ctx.cu_q), self._ptr(ctx.context_lens), self._ptr(out),
                 self._ptr(partial), entries, num_heads, num_kv_heads, block_size, num_pages, float(scale),
                 int(window or 0), chunk, part, splits, int(not leave_unmerged), self._ptr(sinks), self._ptr(share),
-                self._ptr(score_bias), self._stream(), lib=lib,
+                self._ptr(score_bias), cap, self._stream(), lib=lib,
             )
             if leave_unmerged:
                 return PendingMerge(
@@ -1083,7 +1137,7 @@ class HipOps:
                 self._ptr(block_table), width, self._ptr(tiles), num_tiles, wide, self._ptr(ctx.cu_q),
                 self._ptr(ctx.context_lens), self._ptr(out), num_heads, num_kv_heads, block_size, num_pages,
                 float(scale), int(window or 0), chunk, key_runs, self._ptr(partial), self._ptr(sinks), self._ptr(share),
-                self._ptr(score_bias), self._stream(), lib=lib,
+                self._ptr(score_bias), cap, self._stream(), lib=lib,
             )
         return out
 
@@ -1605,6 +1659,7 @@ class HipOps:
         keep_values: bool = False,
         first_values: Optional[torch.Tensor] = None,
         mix_weight: Optional[torch.Tensor] = None,
+        weights: Optional[tuple] = None,
     ):
         """From the float32 sums of an attention layer's input product ([T, heads * head_dim + kv_heads * head_dim +
         kv_heads * value_dim (+ heads)]: queries, keys, values, gate logits) to what the attention kernels take.
@@ -1612,7 +1667,10 @@ class HipOps:
         by its root mean square over head_dim; every value head by its own over value_dim (eps inside the roots,
         no weights).  With `first_values` (float32 [T, kv_heads * value_dim]) and `mix_weight` (float32 [1]) the
         values become (1 - w) v + w first_values.  Queries go to [T, heads * kernel_dim], keys and values into
-        the pages at `slot_mapping`, all zero beyond their own widths.  Returns (queries, sigmoid of the gate
+        the pages at `slot_mapping`, all zero beyond their own widths.  weights: (query norm weight, key norm weight),
+        [head_dim] each; a head is then normed and multiplied by its weight BEFORE the rotation, and values are stored as
+        they are.  kv_heads 0: the rows hold queries only (keys and values are another layer's), nothing is stored.
+        Returns (queries, sigmoid of the gate
         logits as float32 [T, heads] or None, the normed values before mixing as float32 if `keep_values`)."""
         self._check(projected, "projected input", torch.float32, (None, None))
         tokens, width = projected.shape
@@ -1622,8 +1680,24 @@ class HipOps:
             cos, sin, rotary = rotation
             self._check(cos, "rotary cos", torch.float32, (tokens, rotary // 2))
             self._check(sin, "rotary sin", torch.float32, (tokens, rotary // 2))
-        num_pages = self._check_pages(key_pages, value_pages, kv_heads, kernel_dim, block_size)
-        self._check(slot_mapping, "slot mapping", torch.int32, (tokens,))
+        num_pages = 0
+        if kv_heads:
+            num_pages = self._check_pages(key_pages, value_pages, kv_heads, kernel_dim, block_size)
+            self._check(slot_mapping, "slot mapping", torch.int32, (tokens,))
+        else:
+            slot_mapping = key_pages = value_pages = None
+            if keep_values or first_values is not None:
+                raise KernelError("rows that hold queries only have no values to keep or mix")
+        q_weight = k_weight = None
+        if weights is not None:
+            q_weight, k_weight = weights
+            self._check(q_weight, "query norm weight", (torch.float32, self.dtype), (head_dim,))
+            if kv_heads:
+                self._check(k_weight, "key norm weight", q_weight.dtype, (head_dim,))
+            else:
+                k_weight = None
+            if keep_values or first_values is not None:
+                raise KernelError("weighted head norms leave the values as they are")
         if width < (heads + kv_heads) * head_dim + kv_heads * value_dim + (heads if gated else 0):
             raise KernelError("the projected rows are too narrow")
         if first_values is not None:
@@ -1636,7 +1710,8 @@ class HipOps:
             "mlr_head_norm_rope_write", self._ptr(projected), width, self._ptr(q), self._ptr(gate), self._ptr(cos),
             self._ptr(sin), int(rotary), float(eps), self._ptr(slot_mapping), self._ptr(key_pages),
             self._ptr(value_pages), self._ptr(kept), self._ptr(first_values),
-            self._ptr(mix_weight if first_values is not None else None), self.code, tokens, heads, kv_heads, head_dim,
+            self._ptr(mix_weight if first_values is not None else None), self._ptr(q_weight), self._ptr(k_weight),
+            int(q_weight is not None and q_weight.dtype == torch.float32), self.code, tokens, heads, kv_heads, head_dim,
             value_dim, kernel_dim, block_size, num_pages, self._stream(),
         )
         return q, gate, kept
@@ -1692,6 +1767,153 @@ class HipOps:
             state.shape[0], self._ptr(read_rows), self._ptr(write_rows), self._ptr(ctx.cu_q), self._ptr(ctx.q_starts),
             float(cap), float(q_scale), self._ptr(out), entries, heads, head_dim, value_dim, tokens, self._ptr(runs),
             self._ptr(gates), self._stream(),
+        )
+        return out
+
+    # ---- recurrences behind a short convolution, one decay per head and token ----------------------------------
+    def conv_gates(
+        self,
+        projected: torch.Tensor,
+        taps: torch.Tensor,
+        bias: Optional[torch.Tensor],
+        carried: Any,
+        ctx: Any,
+        *,
+        column: int,
+        heads: int,
+        rate: torch.Tensor,
+        dt_bias: torch.Tensor,
+        step_column: int,
+        write_column: Optional[int] = None,
+        unit_heads: int = 0,
+        unit_dim: int = 0,
+        scaled_heads: int = 0,
+        unit_scale: float = 1.0,
+    ) -> tuple[torch.Tensor, torch.Tensor]:
+        """What a recurrence reads, from its input product's float32 sums `projected` [T, width].  The columns column ..
+        column + C (C = taps.shape[1]) pass a causal convolution over time per channel, sum_j taps[j, c] * in_(t -
+        n + 1 + j, c) (+ bias[c]), n = taps.shape[0], and silu.  `carried` (None with one tap) is a state view whose rows
+        [n - 1, C] hold the inputs before the step (zeros where an entry starts its request) and receive the newest
+        ones.  The first unit_heads * unit_dim channels are heads that are then divided by sqrt(sum of squares + 1e-6), the
+        first `scaled_heads` of them times unit_scale.  Per head, with s = softplus(projected[step_column + head] +
+        dt_bias[head]): gates[t, head] = (rate[head] * s, w), the logarithm of the decay and the strength of the
+        write, w = s, or sigmoid(projected[write_column + head]).  Everything 32-bit.  Returns (float32 [T, C], gates float32
+        [T, heads, 2])."""
+        self._check(projected, "projected input", torch.float32, (None, None))
+        tokens, width = projected.shape
+        self._check(taps, "convolution taps", torch.float32, (None, None))
+        n, channels = taps.shape
+        if bias is not None:
+            self._check(bias, "convolution bias", torch.float32, (channels,))
+        entries = ctx.num_entries
+        state = read_rows = write_rows = None
+        rows = 0
+        if n > 1:
+            state, read_rows, write_rows = carried.tensor, carried.read_rows, carried.write_rows
+            self._check(state, "carried inputs", torch.float32, (None, n - 1, channels))
+            rows = state.shape[0]
+            self._check(read_rows, "state rows to read", torch.int32, (entries,))
+            self._check(write_rows, "state rows to write", torch.int32, (entries,))
+        self._check(ctx.token_entry, "token entries", torch.int32, (tokens,))
+        self._check(ctx.cu_q, "cu_q", torch.int32, (entries + 1,))
+        self._check(ctx.q_starts, "q_starts", torch.int32, (entries,))
+        self._check(rate, "decay rates", torch.float32, (heads,))
+        self._check(dt_bias, "step bias", torch.float32, (heads,))
+        if column < 0 or column + channels > width or unit_heads * unit_dim > channels:
+            raise KernelError("the projected rows do not hold the convolution's channels")
+        for at in (step_column, write_column):
+            if at is not None and not 0 <= at <= width - heads:
+                raise KernelError("the projected rows do not hold the gates' sums")
+        out = self._empty((tokens, channels), torch.float32)
+        gates = self._empty((tokens, heads, 2), torch.float32)
+        self._call(
+            "mlr_conv_gates", self._ptr(projected), width, int(column), self._ptr(taps), self._ptr(bias), self._ptr(state),
+            rows, self._ptr(read_rows), self._ptr(write_rows), self._ptr(ctx.token_entry), self._ptr(ctx.cu_q),
+            self._ptr(ctx.q_starts), self._ptr(out), self._ptr(gates), channels, n, int(unit_heads), int(unit_dim),
+            int(scaled_heads), float(unit_scale), self._ptr(rate), self._ptr(dt_bias), heads, int(step_column),
+            -1 if write_column is None else int(write_column), tokens, self._stream(),
+        )
+        return out, gates
+
+    DECAY_CHUNKS_FROM = 64  # tokens more than entries from which the scan goes by chunks instead of token by token
+
+    def decay_scan(
+        self,
+        mixed: torch.Tensor,
+        gates: torch.Tensor,
+        state: torch.Tensor,
+        read_rows: torch.Tensor,
+        write_rows: torch.Tensor,
+        ctx: Any,
+        *,
+        heads: int,
+        key_heads: int,
+        head_dim: int,
+        value_dim: int,
+        offsets: Sequence[int],
+        delta: bool = False,
+        skip: Optional[torch.Tensor] = None,
+        chunked: Optional[bool] = None,
+    ) -> torch.Tensor:
+        """The step's tokens, every entry's in order, through a state S per head with one decay per head and token: with
+        (a, w) = gates[t, head], S <- exp(a) S, then u = w v, or with `delta` u = w (v - S^T k), then S <- S + k
+        u^T and o = S^T q (+ skip[head] * v).  `mixed` (float32 [T, C]) holds q and k (key_heads * head_dim each; head h
+        reads key head h // (heads // key_heads)) and v (heads * value_dim) from the columns `offsets` = (q, k, v) on.
+        State rows as for `retention_scan`.  Everything 32-bit.  Returns o, float32 [T, heads * value_dim].  Steps with few
+        tokens an entry walk them one by one with the state in registers; others go 64 tokens at a time on the
+        matrix cores in true 32-bit (`chunked` forces one way): that reorders 32-bit sums only."""
+        self._check(mixed, "recurrence input", torch.float32, (None, None))
+        tokens, channels = mixed.shape
+        entries = ctx.num_entries
+        if key_heads <= 0 or heads % key_heads:
+            raise KernelError("heads must be a multiple of key heads")
+        self._check(gates, "decays and write strengths", torch.float32, (tokens, heads, 2))
+        self._check(state, "recurrent state", torch.float32, (None, heads, head_dim, value_dim))
+        self._check(read_rows, "state rows to read", torch.int32, (entries,))
+        self._check(write_rows, "state rows to write", torch.int32, (entries,))
+        self._check(ctx.cu_q, "cu_q", torch.int32, (entries + 1,))
+        self._check(ctx.q_starts, "q_starts", torch.int32, (entries,))
+        if skip is not None:
+            self._check(skip, "skip weights", torch.float32, (heads,))
+        q_off, k_off, v_off = (int(o) for o in offsets)
+        if min(q_off, k_off, v_off) < 0 or max(q_off, k_off) + key_heads * head_dim > channels or v_off + heads * value_dim > channels:
+            raise KernelError("the rows do not hold what the offsets name")
+        out = self._empty((tokens, heads * value_dim), torch.float32)
+        if chunked is None:
+            chunked = tokens >= entries + self.DECAY_CHUNKS_FROM
+        scratch, floats = None, 0
+        if chunked:
+            floats = int(self.lib.mlr_decay_scan_scratch(tokens, entries, heads, key_heads, head_dim, value_dim, int(bool(delta))))
+            if floats:
+                scratch = self._empty((floats,), torch.float32)
+        self._call(
+            "mlr_decay_scan", self._ptr(mixed), channels, q_off, k_off, v_off, self._ptr(gates), self._ptr(state),
+            state.shape[0], self._ptr(read_rows), self._ptr(write_rows), self._ptr(ctx.cu_q), self._ptr(ctx.q_starts),
+            self._ptr(skip), self._ptr(out), entries, heads, key_heads, head_dim, value_dim, tokens, int(bool(delta)),
+            self._ptr(scratch), floats, self._stream(),
+        )
+        return out
+
+    def gate_group_norm(
+        self, y: torch.Tensor, projected: torch.Tensor, *, gate_column: int, groups: int, eps: float, norm_weight: torch.Tensor
+    ) -> torch.Tensor:
+        """y (float32 [T, N]) times silu of columns gate_column .. gate_column + N of `projected`, then every one of `groups`
+        equal parts of a row divided by its own root mean square (eps inside the root), times norm_weight [N]; in the
+        engine's dtype."""
+        self._check(projected, "projected input", torch.float32, (None, None))
+        tokens, width = projected.shape
+        self._check(y, "heads", torch.float32, (tokens, None))
+        inner = y.shape[1]
+        if gate_column < 0 or gate_column + inner > width:
+            raise KernelError("the projected rows do not hold the gate")
+        if groups <= 0 or inner % groups:
+            raise KernelError("the parts of a row must be equal")
+        self._check(norm_weight, "norm weight", (torch.float32, self.dtype), (inner,))
+        out = self._empty((tokens, inner), self.dtype)
+        self._call(
+            "mlr_gate_group_norm", self._ptr(y), self._ptr(projected), width, int(gate_column), self._ptr(out), self.code,
+            tokens, inner, int(groups), float(eps), self._ptr(norm_weight), int(norm_weight.dtype == torch.float32),
+            self._stream(),
         )
         return out
 

@@ -46,6 +46,14 @@ class GQAAttention(Mixer):
     output_gate: out = Wo (A * sigmoid(Wg h)), A the attended heads side by side [T, heads * value_dim],
         * the Hadamard product, h the input that q, k and v are made from too.  The Wg product runs
         behind the attention kernel and multiplies in its epilogue.
+    qk_norm_eps: every query head and key head is divided by its root mean square over head_dim (this eps inside the
+        root) and multiplied by a weight [head_dim] that all query heads, or all key heads, share, before its
+        position is encoded (which must be a rotation or nothing).  The input product then keeps its 32-bit sums, one
+        kernel norms, rotates and stores, and heads whose size is no multiple of 16 are padded there to one that is.
+    softcap: score <- softcap * tanh(score / softcap), after the scale.
+    unit_sink: the softmax's denominator is one larger (a key of score 0 without a value).
+    reads_cache: the layer has no key and value projections; it reads the pages another site owns (an execution
+        order entry with `reads_cache_of`).  Goes with `qk_norm_eps`.
     """
 
     replayable = True
@@ -65,6 +73,10 @@ class GQAAttention(Mixer):
         chunk: Optional[int] = None,
         value_dim: Optional[int] = None,
         output_gate: bool = False,
+        qk_norm_eps: Optional[float] = None,
+        softcap: Optional[float] = None,
+        unit_sink: bool = False,
+        reads_cache: bool = False,
     ) -> None:
         if num_heads <= 0 or num_kv_heads <= 0 or num_heads % num_kv_heads:
             raise ValueError("num_heads must be a positive multiple of num_kv_heads")
@@ -74,6 +86,12 @@ class GQAAttention(Mixer):
             raise ValueError("a mixer has a window or a chunked mask, not both")
         if chunk is not None and chunk <= 0:
             raise ValueError("chunk must be > 0")
+        if softcap is not None and not softcap > 0:
+            raise ValueError("softcap must be > 0")
+        if qk_norm_eps is None and reads_cache:
+            raise ValueError("queries without keys of their own go with per-head norms")
+        if qk_norm_eps is not None and (qkv_bias or not qk_norm_eps >= 0):
+            raise ValueError("per-head norms have an eps >= 0 and go with projections without biases")
         self.hidden_size = int(hidden_size)
         self.num_heads = int(num_heads)
         self.num_kv_heads = int(num_kv_heads)
@@ -81,7 +99,7 @@ class GQAAttention(Mixer):
         self.value_dim = self.head_dim if value_dim is None else int(value_dim)
         # the one head size that kernels and pages see
         self.kernel_dim = self.head_dim
-        if self.value_dim != self.head_dim:
+        if self.value_dim != self.head_dim or qk_norm_eps is not None:
             self.kernel_dim = -(-max(self.head_dim, self.value_dim) // 16) * 16
         check_attention_sizes(num_heads, num_kv_heads, self.kernel_dim)  # refused here, not at the first step
         self.chunk = None if chunk is None else int(chunk)
@@ -92,9 +110,18 @@ class GQAAttention(Mixer):
         self.o_bias = bool(o_bias)
         self.window = None if window is None else int(window)
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(head_dim)
+        self.qk_norm_eps = None if qk_norm_eps is None else float(qk_norm_eps)
+        self.softcap = None if softcap is None else float(softcap)
+        self.unit_sink = bool(unit_sink)
+        self.reads_cache = bool(reads_cache)
         self.position: Optional[PositionEncoding] = (
             build_part("position", position) if position is not None else None
         )
+        if self.qk_norm_eps is not None and getattr(self.position, "rotary_dim", 0) > self.head_dim:
+            raise ValueError("the rotation covers more dimensions than a head has")
+        self.q_norm_weight: Optional[torch.Tensor] = None
+        self.k_norm_weight: Optional[torch.Tensor] = None
+        self.sinks: Optional[torch.Tensor] = None
         self.qkv_weight: Optional[torch.Tensor] = None
         self.qkv_bias_vec: Optional[torch.Tensor] = None
         self.o_weight: Optional[torch.Tensor] = None
@@ -119,7 +146,7 @@ class GQAAttention(Mixer):
         return self.num_heads * self.value_dim
 
     def param_specs(self) -> dict[str, ParamSpec]:
-        width = self.q_size + self.kv_size + self.v_size
+        width = self.q_size + (0 if self.reads_cache else self.kv_size + self.v_size)
         specs = {
             "qkv_weight": ParamSpec((width, self.hidden_size)),
             "o_weight": ParamSpec((self.hidden_size, self.out_size)),
@@ -130,11 +157,17 @@ class GQAAttention(Mixer):
             specs["o_bias_vec"] = ParamSpec((self.hidden_size,), keep_stored_precision=True)
         if self.output_gate:
             specs["gate_weight"] = ParamSpec((self.out_size, self.hidden_size))
+        if self.qk_norm_eps is not None:
+            specs["q_norm_weight"] = ParamSpec((self.head_dim,), init="one_plus_normal", keep_stored_precision=True)
+            if not self.reads_cache:
+                specs["k_norm_weight"] = ParamSpec((self.head_dim,), init="one_plus_normal", keep_stored_precision=True)
         return specs
 
     def bind(self, params, *, dtype: torch.dtype, device: torch.device) -> None:
         super().bind(params, dtype=dtype, device=device)
         D = self.kernel_dim
+        if self.unit_sink:
+            self.sinks = torch.zeros(self.num_heads, dtype=torch.float32, device=device)  # exp(0) = 1
         if D == self.head_dim == self.value_dim:
             return
         # heads of two widths: every head at the common size D, the added rows and columns zero
@@ -151,12 +184,14 @@ class GQAAttention(Mixer):
                  rows(v, self.num_kv_heads, self.value_dim)]
             ).contiguous()
 
-        self.qkv_weight = fused(self.qkv_weight)
+        if self.qk_norm_eps is None:  # the kernel that norms the heads pads queries, keys and values itself
+            self.qkv_weight = fused(self.qkv_weight)
         if self.qkv_bias_vec is not None:
             self.qkv_bias_vec = fused(self.qkv_bias_vec)
         if self.gate_weight is not None:
             self.gate_weight = rows(self.gate_weight, self.num_heads, self.value_dim).contiguous()
-        self.o_weight = rows(self.o_weight.t().contiguous(), self.num_heads, self.value_dim).t().contiguous()
+        if D != self.value_dim:
+            self.o_weight = rows(self.o_weight.t().contiguous(), self.num_heads, self.value_dim).t().contiguous()
 
     def children(self) -> dict[str, Part]:
         return {"position": self.position} if self.position is not None else {}
@@ -179,7 +214,28 @@ class GQAAttention(Mixer):
             block_size=cache.block_size,
             write=cache.writable,
         )
-        if self.position is not None and rotation is None:
+        if self.qk_norm_eps is not None:
+            if cache.writable == self.reads_cache:
+                raise RuntimeError("an attention layer reads another site's pages exactly if it is said to")
+            if self.position is not None and rotation is None:
+                raise RuntimeError("per-head norms go with a rotation or no position encoding")
+            own = self.num_kv_heads if cache.writable else 0
+            qkv, _, _ = ops.head_norm_rope_write(
+                ops.linear(h, self.qkv_weight, None, out_dtype=torch.float32),  # norms read it unrounded
+                heads=self.num_heads,
+                kv_heads=own,
+                head_dim=self.head_dim,
+                value_dim=self.value_dim,
+                kernel_dim=self.kernel_dim,
+                eps=self.qk_norm_eps,
+                rotation=rotation,
+                slot_mapping=cache.slot_mapping if own else None,
+                key_pages=cache.key if own else None,
+                value_pages=cache.value if own else None,
+                block_size=cache.block_size,
+                weights=(self.q_norm_weight, self.k_norm_weight),
+            )
+        elif self.position is not None and rotation is None:
             # a position encoding with a rule of its own: it sees the queries and keys between
             # the product and the cache write
             qkv = ops.linear(h, self.qkv_weight, self.qkv_bias_vec)
@@ -211,6 +267,8 @@ class GQAAttention(Mixer):
             defer_merge=not self.output_gate,  # the output product is the only reader
             plan=ctx.plan(getattr(ops, "ATTENTION_PLAN", None)),
             **({"chunk": self.chunk} if self.chunk is not None else {}),
+            **({"sinks": self.sinks} if self.unit_sink else {}),
+            **({"softcap": self.softcap} if self.softcap is not None else {}),
         )
         if self.output_gate:
             attended = ops.linear(h, self.gate_weight, None, activation="sigmoid", multiply=attended)

@@ -123,6 +123,59 @@ class SandwichNormBlock(Block):
         return x, owed
 
 
+@register_part("block", "post_norm")
+class PostNormBlock(Block):
+    """Norms on the sublayers' outputs only; the sublayers read the stream itself:
+
+        x += norm_mixer_out(mixer(x));  x += norm_ff_out(feed_forward(x)).
+
+    A sublayer reads the 32-bit stream rounded to the engine's dtype; its output y enters the stream as w * y *
+    rsqrt(mean(y^2) + eps), computed in 32-bit.  Each such addition is one kernel with the rounding of the
+    stream that the next sublayer reads; the last one is handed to the next block as a `NormedDelta`.  A layer may
+    have no feed-forward.
+    """
+
+    replayable = True
+
+    def __init__(self, mixer: Mixer, feed_forward: Optional[FeedForward], norms: Mapping[str, Norm]) -> None:
+        needed = ["mixer_out"] + (["ff_out"] if feed_forward is not None else [])
+        missing = [n for n in needed if n not in norms]
+        if missing:
+            raise ValueError(f"post_norm block needs the norms {needed}, missing {missing}")
+        self.mixer = mixer
+        self.feed_forward = feed_forward
+        self.norm_mixer_out = norms["mixer_out"]
+        self.norm_ff_out = norms["ff_out"] if feed_forward is not None else None
+        for norm in (self.norm_mixer_out, self.norm_ff_out):
+            if norm is not None and not hasattr(norm, "eps"):
+                raise ValueError("post_norm takes RMS norms (a weight and an eps)")
+
+    def children(self) -> dict[str, Part]:
+        parts: dict[str, Part] = {"mixer": self.mixer, "norm_mixer_out": self.norm_mixer_out}
+        if self.feed_forward is not None:
+            parts.update(feed_forward=self.feed_forward, norm_ff_out=self.norm_ff_out)
+        return parts
+
+    def forward(
+        self, ctx: StepContext, x: torch.Tensor, delta, site: int
+    ) -> tuple[torch.Tensor, Optional[NormedDelta]]:
+        ops = ctx.ops
+        if delta is None:
+            h = ops.rounded(x)
+        elif isinstance(delta, NormedDelta):
+            h = ops.add_normed(x, delta.y, delta.weight, delta.eps, cast=True)
+        else:  # the layer before hands its output on as it is
+            ops.add_(x, delta)
+            h = ops.rounded(x)
+        mixed = self.mixer.forward(ctx, h, site)
+        owed = NormedDelta(mixed, self.norm_mixer_out.weight, self.norm_mixer_out.eps)
+        if self.feed_forward is None:
+            return x, owed
+        h = ops.add_normed(x, owed.y, owed.weight, owed.eps, cast=True)
+        out = self.feed_forward.forward(ctx, h)
+        return x, NormedDelta(out, self.norm_ff_out.weight, self.norm_ff_out.eps)
+
+
 @register_part("block", "parallel")
 class ParallelBlock(Block):
     """One norm, both sublayers read it, both results enter the stream together:

@@ -105,6 +105,46 @@ class ClampedGLU(FeedForward):
         return ops.linear(hidden, self.down_weight, self.down_bias, for_stream=True)
 
 
+@register_part("feed_forward", "geglu")
+class GeGLU(FeedForward):
+    """Dense gated feed-forward with biases on all three products and the tanh form of the GELU:
+
+        y = Wdown (gelu(Wgate x + bgate) * (Wup x + bup)) + bdown,   gelu(z) = z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))).
+
+    Gate and up are one product over rows (and biases) woven in pairs as in `ClampedGLU`, the gating is that product's
+    epilogue, on its 32-bit sums; an odd intermediate size is not woven and gated by a kernel of its own.
+    """
+
+    replayable = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int) -> None:
+        if hidden_size <= 0 or intermediate_size <= 0:
+            raise ValueError("GeGLU sizes must be > 0")
+        self.hidden_size = int(hidden_size)
+        self.intermediate_size = int(intermediate_size)
+        self.woven = self.intermediate_size % 2 == 0
+        self.gate_up_weight: Optional[torch.Tensor] = None
+        self.gate_up_bias: Optional[torch.Tensor] = None
+        self.down_weight: Optional[torch.Tensor] = None
+        self.down_bias: Optional[torch.Tensor] = None
+
+    def param_specs(self) -> dict[str, ParamSpec]:
+        return {
+            "gate_up_weight": ParamSpec((2 * self.intermediate_size, self.hidden_size)),
+            "gate_up_bias": ParamSpec((2 * self.intermediate_size,), keep_stored_precision=True),
+            "down_weight": ParamSpec((self.hidden_size, self.intermediate_size)),
+            "down_bias": ParamSpec((self.hidden_size,), keep_stored_precision=True),
+        }
+
+    def forward(self, ctx: StepContext, h: torch.Tensor) -> torch.Tensor:
+        ops = ctx.ops
+        if self.woven:
+            hidden = ops.linear(h, self.gate_up_weight, self.gate_up_bias, geglu=True)
+        else:
+            hidden = ops.glu_gelu(ops.linear(h, self.gate_up_weight, self.gate_up_bias, out_dtype=torch.float32))
+        return ops.linear(hidden, self.down_weight, self.down_bias, for_stream=True)
+
+
 ACTIVATIONS = ("relu2", "sigmoid")  # what `ops.linear(..., activation=)` applies to its sums
 EXPERT_ACTIVATIONS = ACTIVATIONS + ("swiglu",)  # an expert may also be gated: down(silu(gate(x)) * up(x))
 

@@ -79,7 +79,7 @@ class TorchOps:
     # matrix products ---------------------------------------------------------------------
     def linear(
         self, x, weight, bias=None, out_dtype=None, kernel="auto", swiglu=False, partial_sums=False, for_stream=False,
-        activation=None, multiply=None, clamped_glu=None, multiply_rows=None,
+        activation=None, multiply=None, clamped_glu=None, multiply_rows=None, geglu=False,
     ):
         self._count("linear")
         y = x.float() @ weight.float().t()
@@ -101,11 +101,27 @@ class TorchOps:
             gate = quads[..., :2].clamp(max=limit)
             up = quads[..., 2:].clamp(-limit, limit)
             y = (gate * torch.sigmoid(alpha * gate) * (up + 1.0)).reshape(y.shape[0], -1)
+        if geglu:  # rows and bias woven likewise
+            quads = y.view(y.shape[0], -1, 4)
+            y = (self._gelu(quads[..., :2]) * quads[..., 2:]).reshape(y.shape[0], -1)
         if swiglu:  # rows of weight: gate 2j, gate 2j+1, up 2j, up 2j+1
             quads = y.view(y.shape[0], -1, 4)
             gate, up = quads[..., :2], quads[..., 2:]
             y = (gate * torch.sigmoid(gate) * up).reshape(y.shape[0], -1)
         return y.to(out_dtype or self.dtype)
+
+    @staticmethod
+    def _gelu(z):
+        return 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z**3)))
+
+    def rounded(self, x):
+        self._count("rounded")
+        return x if self.dtype == torch.float32 else x.to(self.dtype)
+
+    def glu_gelu(self, sums):
+        self._count("glu_gelu")
+        inter = sums.shape[1] // 2
+        return (self._gelu(sums[:, :inter].float()) * sums[:, inter:].float()).to(self.dtype)
 
     def silu_mul(self, gate_up):
         inter = gate_up.shape[1] // 2
@@ -365,7 +381,7 @@ class TorchOps:
 
     def paged_attention(
         self, qkv, key_pages, value_pages, block_table, ctx, *, num_heads, num_kv_heads, head_dim, block_size, scale, window,
-        defer_merge=False, plan=None, chunk=None, sinks=None, pooled=None, score_bias=None,
+        defer_merge=False, plan=None, chunk=None, sinks=None, pooled=None, score_bias=None, softcap=None,
     ):
         self._count("paged_attention")
         tokens = qkv.shape[0]
@@ -394,6 +410,8 @@ class TorchOps:
             k = k.repeat_interleave(group, dim=1)
             v = v.repeat_interleave(group, dim=1)
             s = torch.einsum("hd,nhd->hn", q[t], k) * scale
+            if softcap is not None:
+                s = softcap * torch.tanh(s / softcap)
             if score_bias is not None:  # no softmax: every key weighs by itself
                 w = torch.sigmoid(s + score_bias.float()[:, None])
             elif sinks is not None:  # one more term of the denominator, with no key and no value
@@ -430,7 +448,7 @@ class TorchOps:
 
     def head_norm_rope_write(
         self, projected, *, heads, kv_heads, head_dim, value_dim, kernel_dim, eps, rotation, slot_mapping, key_pages,
-        value_pages, block_size, gated=False, keep_values=False, first_values=None, mix_weight=None,
+        value_pages, block_size, gated=False, keep_values=False, first_values=None, mix_weight=None, weights=None,
     ):
         self._count("head_norm_rope_write")
         tokens = projected.shape[0]
@@ -441,9 +459,18 @@ class TorchOps:
         def unit(x):
             return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
 
-        q = unit(self._rotate(p[:, :a].view(tokens, heads, head_dim), rotation))
-        k = unit(self._rotate(p[:, a:b].view(tokens, kv_heads, head_dim), rotation))
-        v = unit(p[:, b:c].view(tokens, kv_heads, value_dim))
+        if weights is not None:  # norm and weight before the rotation, values as they are
+            q = self._rotate(unit(p[:, :a].view(tokens, heads, head_dim)) * weights[0].float(), rotation)
+            if kv_heads == 0:
+                q_out = torch.zeros(tokens, heads, kernel_dim)
+                q_out[..., :head_dim] = q
+                return q_out.view(tokens, heads * kernel_dim).to(self.dtype), None, None
+            k = self._rotate(unit(p[:, a:b].view(tokens, kv_heads, head_dim)) * weights[1].float(), rotation)
+            v = p[:, b:c].view(tokens, kv_heads, value_dim)
+        else:
+            q = unit(self._rotate(p[:, :a].view(tokens, heads, head_dim), rotation))
+            k = unit(self._rotate(p[:, a:b].view(tokens, kv_heads, head_dim), rotation))
+            v = unit(p[:, b:c].view(tokens, kv_heads, value_dim))
         kept = v.reshape(tokens, kv_heads * value_dim).clone() if keep_values else None
         if first_values is not None:
             w = mix_weight.float()[0]
@@ -493,6 +520,69 @@ class TorchOps:
                 out[t] = torch.einsum("hdv,hd->hv", C, q[t]) / below[:, None]
             state[int(write_rows[r])] = torch.cat([C.reshape(heads, cells), n, m[:, None]], dim=1)
         return out.view(tokens, heads * value_dim)
+
+    # recurrences behind a short convolution ---------------------------------------------------------
+    def conv_gates(
+        self, projected, taps, bias, carried, ctx, *, column, heads, rate, dt_bias, step_column, write_column=None,
+        unit_heads=0, unit_dim=0, scaled_heads=0, unit_scale=1.0,
+    ):
+        self._count("conv_gates")
+        n, channels = taps.shape
+        p = projected.float()
+        x = p[:, column : column + channels]
+        out = torch.zeros_like(x)
+        for r in range(ctx.num_entries):
+            a, b = int(ctx.cu_q[r]), int(ctx.cu_q[r + 1])
+            before = torch.zeros(n - 1, channels)
+            if n > 1 and int(ctx.q_starts[r]) > 0:
+                before = carried.tensor[int(carried.read_rows[r])].float().clone()
+            seq = torch.cat([before, x[a:b]])
+            y = sum(taps[j] * seq[j : j + (b - a)] for j in range(n))
+            y = y if bias is None else y + bias
+            out[a:b] = y * torch.sigmoid(y)
+            if n > 1:
+                carried.tensor[int(carried.write_rows[r])] = seq[seq.shape[0] - (n - 1) :]
+        if unit_heads:
+            u = out[:, : unit_heads * unit_dim].view(-1, unit_heads, unit_dim)
+            u = u * torch.rsqrt(u.pow(2).sum(-1, keepdim=True) + 1e-6)
+            u[:, :scaled_heads] *= unit_scale
+            out[:, : unit_heads * unit_dim] = u.reshape(-1, unit_heads * unit_dim)
+        s = torch.nn.functional.softplus(p[:, step_column : step_column + heads] + dt_bias)
+        w = s if write_column is None else torch.sigmoid(p[:, write_column : write_column + heads])
+        return out, torch.stack([rate * s, w], dim=-1)
+
+    def decay_scan(
+        self, mixed, gates, state, read_rows, write_rows, ctx, *, heads, key_heads, head_dim, value_dim, offsets,
+        delta=False, skip=None, chunked=None,
+    ):
+        self._count("decay_scan")
+        tokens = mixed.shape[0]
+        qa, ka, va = offsets
+        group = heads // key_heads
+        q = mixed[:, qa : qa + key_heads * head_dim].view(tokens, key_heads, head_dim).repeat_interleave(group, 1)
+        k = mixed[:, ka : ka + key_heads * head_dim].view(tokens, key_heads, head_dim).repeat_interleave(group, 1)
+        v = mixed[:, va : va + heads * value_dim].view(tokens, heads, value_dim)
+        out = torch.zeros(tokens, heads, value_dim)
+        for r in range(ctx.num_entries):
+            a, b = int(ctx.cu_q[r]), int(ctx.cu_q[r + 1])
+            s = state[int(read_rows[r])].float().clone() if int(ctx.q_starts[r]) > 0 else torch.zeros_like(state[0])
+            for t in range(a, b):
+                s = torch.exp(gates[t, :, 0])[:, None, None] * s
+                u = v[t] - torch.einsum("hdv,hd->hv", s, k[t]) if delta else v[t]
+                s = s + k[t][:, :, None] * (gates[t, :, 1, None] * u)[:, None, :]
+                out[t] = torch.einsum("hdv,hd->hv", s, q[t])
+            state[int(write_rows[r])] = s
+        if skip is not None:
+            out = out + skip[:, None] * v
+        return out.view(tokens, heads * value_dim)
+
+    def gate_group_norm(self, y, projected, *, gate_column, groups, eps, norm_weight):
+        self._count("gate_group_norm")
+        tokens, inner = y.shape
+        z = projected[:, gate_column : gate_column + inner].float()
+        x = (y.float() * z * torch.sigmoid(z)).view(tokens, groups, inner // groups)
+        x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+        return (x.view(tokens, inner) * norm_weight.float()).to(self.dtype)
 
     # routed experts ------------------------------------------------------------------------------
     def route_experts(self, logits, correction, *, top, groups, keep_groups, scale, scores="sigmoid", normalise=False):
