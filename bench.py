@@ -50,6 +50,9 @@ per key channel, a short convolution before the mixer, a looped span of layers) 
 The points named `streams-*` (`PEPULIX_POINTS`; not among the default points) run the Pepulix decoder (four residual
 streams; layers of latent attention with a query latent, matrix memories and attention with sigmoid weights in turn;
 dense feed-forwards with biases and a mixture of gated experts) beside that Qwen2 twin.
+The points named `delta-*` (`ROFETAR_POINTS`; not among the default points) run the Rofetar decoder (norms on the
+sublayers' outputs; layers of a gated delta rule, attention with capped scores, a state-space recurrence and attention
+that reads the other attention's keys in turn) beside that Qwen2 twin.
 `reference`: the reference's own published measurements, run here at their parameters with the
 0.5B shape (random weights and token ids of the published lengths; its figures are of an RTX 3060
 laptop GPU in float16 and stand beside for scale): the burst of 8 short requests under continuous and
@@ -109,7 +112,7 @@ def parse_args() -> argparse.Namespace:
     p.add_argument("--no-prefill", action="store_true", help="skip the prefill measurement")
     p.add_argument("--seed", type=int, default=0)
     p.add_argument("--workload", default="decode", choices=("decode", "burst", "chunked", "library", "reference", "designs"))
-    p.add_argument("--design-only", default="", choices=("", "fedolorn", "qwen2", "bubitar", "vobisun", "pepulix"), help="run one of the two designs of the `designs` workload (for profiles)")
+    p.add_argument("--design-only", default="", choices=("", "fedolorn", "qwen2", "bubitar", "vobisun", "pepulix", "rofetar"), help="run one of the two designs of the `designs` workload (for profiles)")
     p.add_argument("--design-points", default="", help="names of the `designs` workload's points to run, comma separated (default: all)")
     p.add_argument("--no-large", action="store_true", help="leave out the 7B and 32B points of the default run")
     p.add_argument("--samples", action="store_true", help="print every raw sample, not only their summary")
@@ -806,6 +809,25 @@ class Bench:
                 pairs = sum(min(t + 1, a.window) + max(0, t - a.window + 1) // a.pool for t in range(tokens))
                 flops += 2 * tokens * per_token + 2 * a.heads * (a.dim + a.vdim) * pairs
             return flops
+        if getattr(config, "architecture", "") == "Rofetar":
+            # per layer: the mixer's products, its (query, visible key) pairs or its state's update and read (the delta
+            # rule reads the state twice), and a gated feed-forward of three matrices
+            for layer in config.layers:
+                a, m = layer.mixer, layer.mlp
+                per_token, per_pair = a.heads * a.vdim * width, 0
+                if a.kind == "attention":
+                    per_token += width * (a.heads * a.dim + (0 if a.kv_from is not None else a.kv_heads * (a.dim + a.vdim)))
+                    per_pair = a.heads * (a.dim + a.vdim)
+                elif a.kind == "mamba2":
+                    per_token += width * (2 * a.heads * a.vdim + 2 * a.groups * a.state + a.heads)
+                    per_token += 2 * a.heads * a.state * a.vdim + a.conv * (a.heads * a.vdim + 2 * a.groups * a.state)
+                else:
+                    per_token += width * (2 * a.kv_heads * a.dim + 2 * a.heads * a.vdim + 2 * a.heads)
+                    per_token += 3 * a.heads * a.dim * a.vdim + a.conv * (2 * a.kv_heads * a.dim + a.heads * a.vdim)
+                if m is not None:
+                    per_token += 3 * width * m.ff
+                flops += 2 * tokens * per_token + 2 * per_pair * (tokens * (tokens + 1) // 2)
+            return flops
         if getattr(config, "architecture", "") == "Pepulix":
             # per layer: the mixer's products (latent attention as the kernels run it: the query's two products,
             # the query through Wuk^T, scores and values over rows of kv_rank + rot_dim and kv_rank, the attended
@@ -1043,7 +1065,48 @@ def pepulix_configs(name: str) -> dict:
     return {"pepulix": pepulix, "qwen2": qwen2}
 
 
+# The Rofetar decoder beside the Qwen2 decoder: the same width, query and key/value heads, head size, feed-forward
+# width, layers and vocabulary.  The layers take turns: a gated delta rule (as many heads of dim x dim, half as many
+# key heads), attention with capped scores, a state-space recurrence (as many heads, values of twice the head size,
+# a state of 128 rows in two groups), attention that reads the keys and values of the attention before it.
+ROFETAR_POINTS = {
+    # name: (width, heads, kv heads, head size, feed-forward width, layers run)
+    "delta-0.5b": (896, 14, 2, 64, 4864, 12),
+    "delta-7b": (3584, 28, 4, 128, 18944, 4),
+}
+
+
+def rofetar_configs(name: str) -> dict:
+    width, heads, kv_heads, dim, inter, layers = ROFETAR_POINTS[name]
+    attention = {
+        "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim**-0.5, "softcap": 30.0,
+        "rot": {"base": 1000000.0, "dims": dim, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}},
+    }
+    listed = []
+    for i in range(layers):
+        if i % 4 == 0:
+            kind, mixer = "delta", {"heads": heads, "kv_heads": heads // 2, "dim": dim, "vdim": dim, "conv": 4}
+        elif i % 4 == 2:
+            kind = "mamba2"
+            mixer = {"heads": heads, "vdim": 2 * dim, "state": 128, "groups": 2, "conv": 4, "norm_groups": 2}
+        else:
+            kind, mixer = "attention", dict(attention)
+            if i % 4 == 3:
+                mixer["kv_from"] = i - 2
+        listed.append({"type": kind, "mixer": mixer, "mlp": {"kind": "dense", "ff": inter}})
+    rofetar = {"architecture": "Rofetar", "vocab": DESIGN_VOCAB, "width": width, "norm": {"eps": 1e-5}, "layers": listed}
+    qwen2 = {
+        "architectures": ["Qwen2ForCausalLM"], "model_type": "qwen2", "vocab_size": DESIGN_VOCAB, "hidden_size": width,
+        "intermediate_size": inter, "num_hidden_layers": layers, "num_attention_heads": heads,
+        "num_key_value_heads": kv_heads, "head_dim": dim, "max_position_embeddings": 32768, "rms_norm_eps": 1e-5,
+        "rope_theta": 1000000.0, "hidden_act": "silu", "tie_word_embeddings": True,
+    }
+    return {"rofetar": rofetar, "qwen2": qwen2}
+
+
 def design_configs(name: str) -> dict:
+    if name in ROFETAR_POINTS:
+        return rofetar_configs(name)
     if name in PEPULIX_POINTS:
         return pepulix_configs(name)
     if name in BUBITAR_POINTS:

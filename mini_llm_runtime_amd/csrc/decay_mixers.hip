@@ -245,6 +245,574 @@ __global__ __launch_bounds__(256) void decay_walk_kernel(
   }
 }
 
+// ---- the scan, 64 tokens at a time on the matrix cores ----------------------------------------------------------
+// In true 32-bit: v_mfma_f32_16x16x4_f32 takes and sums float32.  Within a chunk of n tokens (local index i, j; what is
+// beyond n is zero) with S the state before it, A_i = a_0 + .. + a_i (summed in float64: only differences of it are
+// used, and they may be small beside it) and e(i, j) = exp(A_i - A_j):
+//     DELTA: u solves u_i + sum_{j<i} w_i e(i, j) (k_i . k_j) u_j = w_i v_i - w_i exp(A_i) S^T k_i, i.e. with L the strictly
+//     lower triangular matrix of the sum, U = U0 - X S for (I + L) [X | U0] = [w exp(A) K | w V];    else u_i = w_i v_i;
+//     o_i = exp(A_i) S^T q_i + sum_{j<=i} e(i, j) (q_i . k_j) u_j,     S' = exp(A_n) S + sum_j e(n, j) k_j u_j^T.
+// decay_local_kernel, all chunks of all entries at once: the parts that do not need S (DELTA: X and U0 by block forward
+// substitution; else the chunk's share of S').  The walk over an entry's chunks: delta_carry_kernel (two products a
+// chunk) or plain_carry_kernel (element by element); both leave the state BEFORE every chunk.  decay_apply_kernel, all chunks at
+// once again, makes the outputs.
+// Lane layouts of the product D[16x16] += A[16x4] B[4x16]: lane l holds A[l % 16][l / 16], B[l / 16][l % 16] and
+// D[4 (l / 16) + e][l % 16], e = 0..3.  A sum over 16 values of k is four such products, and any order of k will do if
+// both operands keep it: product e takes k = 4 (l / 16) + e.  So operands are read as four consecutive k (16 bytes) a
+// lane, and a D tile is, register by register, the B operand of the next product over its rows.
+constexpr int kChunk = 64;
+constexpr int kMatLd = kChunk + 8;  // row of a 64 x 64 matrix in LDS: 32 bytes modulo 64 keeps 16-byte reads of 16 rows off each other's banks
+
+__device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
+__host__ __device__ __forceinline__ int chunks_of(int tokens) { return (tokens + kChunk - 1) / kChunk; }
+
+// Which entry chunk number `chunk` (counted through the entries in order) belongs to, its first token and its tokens.
+__device__ inline bool find_chunk(const int* __restrict__ cu_q, int entries, int chunk, int& entry, int& place, int& t0, int& n) {
+  for (int e = 0; e < entries; ++e) {
+    const int have = chunks_of(cu_q[e + 1] - cu_q[e]);
+    if (chunk < have) {
+      entry = e;
+      place = chunk;
+      t0 = cu_q[e] + chunk * kChunk;
+      n = min(kChunk, cu_q[e + 1] - t0);
+      return true;
+    }
+    chunk -= have;
+  }
+  return false;
+}
+
+// The chunk's A_i (float64) and w_i into LDS, by the first wavefront.
+__device__ __forceinline__ void chunk_gates(const float* __restrict__ gates, int heads, int h, int t0, int n, double* As, float* ws) {
+  if (threadIdx.x < kChunk) {
+    const int i = threadIdx.x;
+    const float* g = gates + (static_cast<int64_t>(t0 + min(i, n - 1)) * heads + h) * 2;
+    double a = i < n ? static_cast<double>(g[0]) : 0.0;
+#pragma unroll
+    for (int d = 1; d < kChunk; d *= 2) {
+      const double before = __shfl_up(a, d, kWave);
+      if (i >= d) a += before;
+    }
+    As[i] = a;
+    ws[i] = i < n ? g[1] : 0.f;
+  }
+}
+
+// Rows of one head of the chunk (columns `at` .. of x), zero beyond n and dim, into LDS rows of LD floats.
+template <int DP, int LD>
+__device__ __forceinline__ void chunk_rows(const float* __restrict__ x, int channels, int at, int t0, int n, int dim, float* rows) {
+  constexpr int kEach = kChunk * DP / 256;
+  float v[kEach];
+#pragma unroll
+  for (int u = 0; u < kEach; ++u) {
+    const int idx = threadIdx.x + u * 256;
+    const int i = idx / DP, d = idx % DP;
+    v[u] = x[static_cast<int64_t>(t0 + min(i, n - 1)) * channels + at + min(d, dim - 1)];
+  }
+#pragma unroll
+  for (int u = 0; u < kEach; ++u) {
+    const int idx = threadIdx.x + u * 256;
+    const int i = idx / DP, d = idx % DP;
+    rows[i * LD + d] = (i < n && d < dim) ? v[u] : 0.f;
+  }
+}
+
+// The lower triangle of 4 x 4 blocks of 16 x 16, diagonal included, as a list: block b is (row, column).
+__device__ __forceinline__ void triangle_block(int b, int& row, int& column) {
+  row = b < 1 ? 0 : b < 3 ? 1 : b < 6 ? 2 : 3;
+  column = b - row * (row + 1) / 2;
+}
+
+// rows a[16 bi ..] times rows b[16 bj ..] transposed, both [64][LD] in LDS: a D tile.
+template <int DP, int LD>
+__device__ __forceinline__ f32x4 rows_product(const float* a, const float* b, int bi, int bj, int r16, int quad) {
+  f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+  for (int g = 0; g < DP / 16; ++g) {
+    const f32x4 av = *reinterpret_cast<const f32x4*>(&a[(16 * bi + r16) * LD + 16 * g + 4 * quad]);
+    const f32x4 bv = *reinterpret_cast<const f32x4*>(&b[(16 * bj + r16) * LD + 16 * g + 4 * quad]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) acc[e % 2] = mfma_f32(av[e], bv[e], acc[e % 2]);
+  }
+  return acc[0] + acc[1];
+}
+
+// Where a scan's scratch memory holds what, per chunk and head (offsets in floats): the state before the chunk [DP, vpad]; for
+// the delta rule X [64, DP], K [64, DP] (zero padded), U [64, vpad] (U0, then U) and e(n, j) [64]; exp(A_n).
+struct ChunkScratch {
+  float *state, *x, *k, *u, *last, *decay;
+  int dp, vpad;
+};
+__host__ __device__ inline int64_t scratch_floats_per_chunk(int dp, int vpad, int delta) {
+  return static_cast<int64_t>(dp) * vpad + (delta ? 2 * kChunk * dp + kChunk * vpad + kChunk : 0) + 1;
+}
+inline ChunkScratch chunk_scratch(float* base, int64_t cells, int dp, int vpad, int delta) {
+  ChunkScratch s;
+  s.dp = dp;
+  s.vpad = vpad;
+  s.state = base;
+  float* at = base + cells * dp * vpad;
+  s.x = at;
+  if (delta) at += cells * kChunk * dp;
+  s.k = at;
+  if (delta) at += cells * kChunk * dp;
+  s.u = at;
+  if (delta) at += cells * kChunk * vpad;
+  s.last = at;
+  if (delta) at += cells * kChunk;
+  s.decay = at;
+  return s;
+}
+
+template <int DP, bool DELTA>
+__global__ __launch_bounds__(256) void decay_local_kernel(const float* __restrict__ x, int channels, int k_off, int v_off,
+                                                          const float* __restrict__ gates, const int* __restrict__ cu_q,
+                                                          int entries, int heads, int key_heads, int dim, int vdim,
+                                                          ChunkScratch out) {
+  constexpr int LD = DELTA ? DP + 8 : DP + 4;  // DELTA reads four k of a row at a time, else single elements of rows 4 apart
+  __shared__ __attribute__((aligned(16))) float Ks[kChunk * LD];
+  __shared__ __attribute__((aligned(16))) float Ls[DELTA ? kChunk * kMatLd : 4];      // -L
+  __shared__ __attribute__((aligned(16))) float Ti[DELTA ? 4 * 16 * 24 : 4];         // inverses of I + L's diagonal blocks
+  __shared__ double As[kChunk];
+  __shared__ float ws[kChunk];
+  int entry, place, t0, n;
+  if (!find_chunk(cu_q, entries, blockIdx.x, entry, place, t0, n)) return;  // the grid is sized for the most chunks
+  const int h = blockIdx.y;
+  const int kh = h / (heads / key_heads);
+  const int tid = threadIdx.x;
+  const int lane = tid % kWave;
+  const int w = __builtin_amdgcn_readfirstlane(tid / kWave);
+  const int r16 = lane % 16;
+  const int quad = lane / 16;
+  const int64_t cell = static_cast<int64_t>(blockIdx.x) * heads + h;
+  const int vpad = out.vpad;
+  chunk_gates(gates, heads, h, t0, n, As, ws);
+  chunk_rows<DP, LD>(x, channels, k_off + kh * dim, t0, n, dim, Ks);
+  __syncthreads();
+  const double a_last = As[kChunk - 1];
+  if (tid == 0) out.decay[cell] = expf(static_cast<float>(a_last));
+
+  // values of a strip of 16 columns, rows 16 b + 4 quad + e
+  auto values = [&](int strip, f32x4 (&v)[4]) {
+    const int c = strip * 16 + r16;
+#pragma unroll
+    for (int b = 0; b < 4; ++b)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int row = 16 * b + 4 * quad + e;
+        v[b][e] = x[static_cast<int64_t>(t0 + min(row, n - 1)) * channels + v_off + static_cast<int64_t>(h) * vdim + min(c, vdim - 1)];
+      }
+#pragma unroll
+    for (int b = 0; b < 4; ++b)
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (!(16 * b + 4 * quad + e < n && c < vdim)) v[b][e] = 0.f;
+  };
+
+  if constexpr (DELTA) {
+    if (tid < kChunk) out.last[cell * kChunk + tid] = expf(static_cast<float>(a_last - As[tid]));
+    for (int b = w; b < 10; b += 4) {
+      int bi, bj;
+      triangle_block(b, bi, bj);
+      const f32x4 dot = rows_product<DP, LD>(Ks, Ks, bi, bj, r16, quad);
+      const int j = 16 * bj + r16;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int i = 16 * bi + 4 * quad + e;
+        Ls[i * kMatLd + j] = j < i ? -ws[i] * expf(static_cast<float>(As[i] - As[j])) * dot[e] : 0.f;
+      }
+    }
+    // K as the carry kernel reads it
+    for (int idx = tid; idx < kChunk * DP; idx += 256) out.k[cell * kChunk * DP + idx] = Ks[idx / DP * LD + idx % DP];
+    __syncthreads();
+    {
+      // column r16 of the inverse of diagonal block w, by forward substitution (every 16 lanes the same)
+      float t[16];
+      const float* block = &Ls[16 * w * kMatLd + 16 * w];
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        float acc = i == r16 ? 1.0f : 0.f;
+#pragma unroll
+        for (int j = 0; j < i; ++j) acc = fmaf(block[i * kMatLd + j], t[j], acc);
+        t[i] = acc;
+      }
+      if (quad == 0)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) Ti[(16 * w + i) * 24 + r16] = t[i];
+    }
+    __syncthreads();
+    const int strips = DP / 16 + vpad / 16;
+    for (int s = w; s < strips; s += 4) {
+      f32x4 r[4];
+      if (s < DP / 16) {
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const int row = 16 * b + 4 * quad + e;
+            r[b][e] = ws[row] * expf(static_cast<float>(As[row])) * Ks[row * LD + 16 * s + r16];
+          }
+      } else {
+        values(s - DP / 16, r);
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) r[b][e] *= ws[16 * b + 4 * quad + e];
+      }
+      f32x4 solved[4];
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+        f32x4 acc = r[b];
+#pragma unroll
+        for (int k = 0; k < b; ++k) {
+          const f32x4 l = *reinterpret_cast<const f32x4*>(&Ls[(16 * b + r16) * kMatLd + 16 * k + 4 * quad]);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) acc = mfma_f32(l[e], solved[k][e], acc);
+        }
+        const f32x4 t = *reinterpret_cast<const f32x4*>(&Ti[(16 * b + r16) * 24 + 4 * quad]);
+        f32x4 y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y = mfma_f32(t[e], acc[e], y);
+        solved[b] = y;
+      }
+      float* dst = s < DP / 16 ? out.x + cell * kChunk * DP + 16 * s : out.u + cell * kChunk * vpad + 16 * (s - DP / 16);
+      const int stride = s < DP / 16 ? DP : vpad;
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) dst[static_cast<int64_t>(16 * b + 4 * quad + e) * stride + r16] = solved[b][e];
+    }
+  } else {
+    float factor[16];
+#pragma unroll
+    for (int b = 0; b < 4; ++b)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int row = 16 * b + 4 * quad + e;
+        factor[4 * b + e] = ws[row] * expf(static_cast<float>(a_last - As[row]));
+      }
+    for (int s = w; s < vpad / 16; s += 4) {
+      f32x4 v[4];
+      values(s, v);
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[b][e] *= factor[4 * b + e];
+      float* dst = out.state + cell * DP * vpad + 16 * s + r16;
+#pragma unroll
+      for (int dt = 0; dt < DP / 16; ++dt) {
+        f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            acc[e % 2] = mfma_f32(Ks[(16 * b + 4 * quad + e) * LD + 16 * dt + r16], v[b][e], acc[e % 2]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) dst[static_cast<int64_t>(16 * dt + 4 * quad + e) * vpad] = acc[0][e] + acc[1][e];
+      }
+    }
+  }
+}
+
+// S' = exp(A_n) S + (the chunk's share), element by element; leaves the state before every chunk where its share was.
+__global__ __launch_bounds__(256) void plain_carry_kernel(float* __restrict__ state, const int* __restrict__ read_rows,
+                                                          const int* __restrict__ write_rows, const int* __restrict__ cu_q,
+                                                          const int* __restrict__ q_starts, int heads, int dim, int vdim,
+                                                          ChunkScratch s) {
+  const int entry = blockIdx.x;
+  const int h = blockIdx.y;
+  const int idx = blockIdx.z * 256 + threadIdx.x;
+  if (idx >= s.dp * s.vpad) return;
+  const int d = idx / s.vpad;
+  const int v = idx - d * s.vpad;
+  const bool real = d < dim && v < vdim;
+  const int count = chunks_of(cu_q[entry + 1] - cu_q[entry]);
+  int first = 0;
+  for (int e = 0; e < entry; ++e) first += chunks_of(cu_q[e + 1] - cu_q[e]);
+  const int64_t head_state = static_cast<int64_t>(dim) * vdim;
+  float value = 0.f;
+  if (real && q_starts[entry] > 0)
+    value = state[(static_cast<int64_t>(read_rows[entry]) * heads + h) * head_state + static_cast<int64_t>(d) * vdim + v];
+  const int64_t cells = static_cast<int64_t>(s.dp) * s.vpad;
+  float* at = s.state + (static_cast<int64_t>(first) * heads + h) * cells + idx;
+  const float* decay = s.decay + static_cast<int64_t>(first) * heads + h;
+  for (int c0 = 0; c0 < count; c0 += 8) {  // eight chunks' loads on their way at a time
+    float add[8], keep[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      const int64_t c = min(c0 + k, count - 1);
+      add[k] = at[c * heads * cells];
+      keep[k] = decay[c * heads];
+    }
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      if (c0 + k < count) {
+        at[static_cast<int64_t>(c0 + k) * heads * cells] = value;
+        value = fmaf(keep[k], value, add[k]);
+      }
+    }
+  }
+  if (real)
+    state[(static_cast<int64_t>(write_rows[entry]) * heads + h) * head_state + static_cast<int64_t>(d) * vdim + v] = value;
+}
+
+// The delta rule's walk over an entry's chunks for 16 value columns of one head: U = U0 - X S, S' = exp(A_n) S + K^T (e(n, .) U).
+// Wavefront w owns the rows 16 w .. of U and every fourth 16-row tile of S (in registers, a D tile each); both go
+// through LDS as B operands.  The next chunk's X, K and U0 are on their way meanwhile.
+template <int DP>
+__global__ __launch_bounds__(256) void delta_carry_kernel(float* __restrict__ state, const int* __restrict__ read_rows,
+                                                          const int* __restrict__ write_rows, const int* __restrict__ cu_q,
+                                                          const int* __restrict__ q_starts, int heads, int dim, int vdim,
+                                                          ChunkScratch s) {
+  constexpr int kTiles = DP / 16;
+  constexpr int kOwn = (kTiles + 3) / 4;  // tiles of S a wavefront owns at most
+  __shared__ __attribute__((aligned(16))) f32x4 Sb[kTiles][kWave];
+  __shared__ __attribute__((aligned(16))) f32x4 Ub[4][kWave];
+  const int entry = blockIdx.z;
+  const int h = blockIdx.y;
+  const int tid = threadIdx.x;
+  const int lane = tid % kWave;
+  const int w = __builtin_amdgcn_readfirstlane(tid / kWave);
+  const int r16 = lane % 16;
+  const int quad = lane / 16;
+  const int col = blockIdx.x * 16 + r16;
+  const int vpad = s.vpad;
+  const int count = chunks_of(cu_q[entry + 1] - cu_q[entry]);
+  int first = 0;
+  for (int e = 0; e < entry; ++e) first += chunks_of(cu_q[e + 1] - cu_q[e]);
+  const int64_t head_state = static_cast<int64_t>(dim) * vdim;
+
+  f32x4 S[kOwn];
+  const bool fresh = q_starts[entry] == 0;
+  const float* src = state + (static_cast<int64_t>(read_rows[entry]) * heads + h) * head_state;
+#pragma unroll
+  for (int o = 0; o < kOwn; ++o)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int d = 16 * (w + 4 * o) + 4 * quad + e;
+      S[o][e] = (!fresh && d < dim && col < vdim) ? src[static_cast<int64_t>(d) * vdim + col] : 0.f;
+    }
+
+  f32x4 xa[kTiles], u0, last;
+  float ka[kOwn][16];
+  float keep;
+  auto fetch = [&](int c) {
+    const int64_t cell = static_cast<int64_t>(first + c) * heads + h;
+    const float* xr = s.x + (cell * kChunk + 16 * w + r16) * DP + 4 * quad;
+#pragma unroll
+    for (int g = 0; g < kTiles; ++g) xa[g] = *reinterpret_cast<const f32x4*>(xr + 16 * g);
+    const float* kr = s.k + (cell * kChunk + 4 * quad) * DP + r16;
+#pragma unroll
+    for (int o = 0; o < kOwn; ++o) {
+      const int tile = min(w + 4 * o, kTiles - 1);
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ka[o][4 * b + e] = kr[(16 * b + e) * DP + 16 * tile];
+    }
+    const float* ur = s.u + (cell * kChunk + 16 * w + 4 * quad) * vpad + blockIdx.x * 16 + r16;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) u0[e] = ur[e * vpad];
+    last = *reinterpret_cast<const f32x4*>(s.last + cell * kChunk + 16 * w + 4 * quad);
+    keep = s.decay[cell];
+  };
+  fetch(0);
+  for (int c = 0; c < count; ++c) {
+    const int64_t cell = static_cast<int64_t>(first + c) * heads + h;
+    float* before = s.state + cell * DP * vpad + blockIdx.x * 16 + r16;
+#pragma unroll
+    for (int o = 0; o < kOwn; ++o) {
+      const int tile = w + 4 * o;
+      if (tile < kTiles) {
+        Sb[tile][lane] = S[o];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) before[static_cast<int64_t>(16 * tile + 4 * quad + e) * vpad] = S[o][e];
+      }
+    }
+    __syncthreads();
+    f32x4 held[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+    for (int g = 0; g < kTiles; ++g) {
+      const f32x4 sb = Sb[g][lane];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) held[e % 2] = mfma_f32(xa[g][e], sb[e], held[e % 2]);
+    }
+    const f32x4 u = u0 - (held[0] + held[1]);
+    float* ur = s.u + (cell * kChunk + 16 * w + 4 * quad) * vpad + blockIdx.x * 16 + r16;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ur[e * vpad] = u[e];
+    Ub[w][lane] = u * last;
+    const float decay = keep;
+    float kb[kOwn][16];
+#pragma unroll
+    for (int o = 0; o < kOwn; ++o)
+#pragma unroll
+      for (int b = 0; b < 16; ++b) kb[o][b] = ka[o][b];
+    if (c + 1 < count) fetch(c + 1);
+    __syncthreads();
+    f32x4 ub[4];
+#pragma unroll
+    for (int b = 0; b < 4; ++b) ub[b] = Ub[b][lane];
+#pragma unroll
+    for (int o = 0; o < kOwn; ++o) {
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+      S[o] *= decay;
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+#pragma unroll
+        for (int e = 0; e < 4; e += 2) {
+          S[o] = mfma_f32(kb[o][4 * b + e], ub[b][e], S[o]);
+          acc = mfma_f32(kb[o][4 * b + e + 1], ub[b][e + 1], acc);
+        }
+      }
+      S[o] += acc;
+    }
+  }
+  float* dst = state + (static_cast<int64_t>(write_rows[entry]) * heads + h) * head_state;
+#pragma unroll
+  for (int o = 0; o < kOwn; ++o)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int d = 16 * (w + 4 * o) + 4 * quad + e;
+      if (d < dim && col < vdim) dst[static_cast<int64_t>(d) * vdim + col] = S[o][e];
+    }
+}
+
+// The outputs of a chunk: o_i = exp(A_i) S^T q_i + sum_{j<=i} e(i, j) (q_i . k_j) u_j (+ skip v_i).  The scores take the
+// place of the keys in LDS; a wavefront then owns every fourth strip of 16 value columns, whose state and u it
+// reads once for all 64 rows.
+template <int DP, bool DELTA>
+__global__ __launch_bounds__(256) void decay_apply_kernel(const float* __restrict__ x, int channels, int q_off, int k_off,
+                                                          int v_off, const float* __restrict__ gates,
+                                                          const int* __restrict__ cu_q, const int* __restrict__ q_starts,
+                                                          const float* __restrict__ skip, float* __restrict__ out,
+                                                          int entries, int heads, int key_heads, int dim, int vdim,
+                                                          ChunkScratch s) {
+  constexpr int LD = DP + 8;
+  extern __shared__ __attribute__((aligned(16))) float apply_lds[];
+  float* const Qs = apply_lds;            // [64][LD]
+  float* const Ks = Qs + kChunk * LD;     // [64][LD], then the scores [64][kMatLd]
+  float* const Ps = Ks;
+  __shared__ double As[kChunk];
+  __shared__ float ws[kChunk];
+  int entry, place, t0, n;
+  if (!find_chunk(cu_q, entries, blockIdx.x, entry, place, t0, n)) return;
+  const int h = blockIdx.y;
+  const int kh = h / (heads / key_heads);
+  const int tid = threadIdx.x;
+  const int lane = tid % kWave;
+  const int w = __builtin_amdgcn_readfirstlane(tid / kWave);
+  const int r16 = lane % 16;
+  const int quad = lane / 16;
+  const int64_t cell = static_cast<int64_t>(blockIdx.x) * heads + h;
+  const int vpad = s.vpad;
+  chunk_gates(gates, heads, h, t0, n, As, ws);
+  chunk_rows<DP, LD>(x, channels, q_off + kh * dim, t0, n, dim, Qs);
+  chunk_rows<DP, LD>(x, channels, k_off + kh * dim, t0, n, dim, Ks);
+  __syncthreads();
+  f32x4 dots[3];
+#pragma unroll
+  for (int u = 0; u < 3; ++u) {
+    const int b = w + 4 * u;
+    if (b < 10) {
+      int bi, bj;
+      triangle_block(b, bi, bj);
+      dots[u] = rows_product<DP, LD>(Qs, Ks, bi, bj, r16, quad);
+    }
+  }
+  __syncthreads();  // the keys are done with
+#pragma unroll
+  for (int u = 0; u < 3; ++u) {
+    const int b = w + 4 * u;
+    if (b < 10) {
+      int bi, bj;
+      triangle_block(b, bi, bj);
+      const int j = 16 * bj + r16;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int i = 16 * bi + 4 * quad + e;
+        Ps[i * kMatLd + j] = j <= i ? expf(static_cast<float>(As[i] - As[j])) * (DELTA ? 1.0f : ws[j]) * dots[u][e] : 0.f;
+      }
+    }
+  }
+  __syncthreads();
+  const bool carried = !(place == 0 && q_starts[entry] == 0);  // else the state before the chunk is zero
+  const float d_skip = skip != nullptr ? skip[h] : 0.f;
+  for (int strip = w; strip < vpad / 16; strip += 4) {
+    const int c = strip * 16 + r16;
+    f32x4 u[4];
+    if constexpr (DELTA) {
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) u[b][e] = s.u[(cell * kChunk + 16 * b + 4 * quad + e) * vpad + c];
+    } else {
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          u[b][e] = x[static_cast<int64_t>(t0 + min(16 * b + 4 * quad + e, n - 1)) * channels + v_off +
+                      static_cast<int64_t>(h) * vdim + min(c, vdim - 1)];
+    }
+    f32x4 o[4];
+#pragma unroll
+    for (int b = 0; b < 4; ++b) o[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (carried) {
+      const float* before = s.state + cell * DP * vpad + c;
+      constexpr int kHalf = DP / 16 > 4 ? 4 : DP / 16;  // tiles of the state in registers at a time
+#pragma unroll
+      for (int g0 = 0; g0 < DP / 16; g0 += kHalf) {
+        f32x4 sb[kHalf];
+#pragma unroll
+        for (int g = 0; g < kHalf; ++g)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) sb[g][e] = before[static_cast<int64_t>(16 * (g0 + g) + 4 * quad + e) * vpad];
+#pragma unroll
+        for (int g = 0; g < kHalf; ++g) {
+          f32x4 q[4];
+#pragma unroll
+          for (int b = 0; b < 4; ++b)
+            q[b] = *reinterpret_cast<const f32x4*>(&Qs[(16 * b + r16) * LD + 16 * (g0 + g) + 4 * quad]);
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int b = 0; b < 4; ++b) o[b] = mfma_f32(q[b][e], sb[g][e], o[b]);
+        }
+      }
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[b][e] *= expf(static_cast<float>(As[16 * b + 4 * quad + e]));
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      f32x4 p[4];
+#pragma unroll
+      for (int b = k; b < 4; ++b) p[b] = *reinterpret_cast<const f32x4*>(&Ps[(16 * b + r16) * kMatLd + 16 * k + 4 * quad]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int b = k; b < 4; ++b) o[b] = mfma_f32(p[b][e], u[k][e], o[b]);
+    }
+    if (c < vdim) {
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int i = 16 * b + 4 * quad + e;
+          if (i < n) {
+            float v = o[b][e];
+            if (!DELTA && skip != nullptr) v = fmaf(d_skip, u[b][e], v);
+            out[(static_cast<int64_t>(t0 + i) * heads + h) * vdim + c] = v;
+          }
+        }
+    }
+  }
+}
+
 // ---- gate, then norm in equal parts of a row -----------------------------------------------------------------
 // out[t, i] = y silu(z) / sqrt(mean over the element's part of (y silu(z))^2 + eps) * weight[i], z = p[t, gate_column + i].
 // One workgroup per (token, part).
@@ -324,7 +892,14 @@ int mlr_conv_gates(const float* projected, int width, int column, const float* t
   return 0;
 }
 
-int64_t mlr_decay_scan_scratch(int tokens, int entries, int heads, int key_heads, int dim, int vdim, int delta) { return 0; }
+static int padded_rows(int dim) { return dim <= 32 ? 32 : dim <= 64 ? 64 : 128; }
+
+// Floats of scratch memory that mlr_decay_scan needs to go by chunks (0: it will not go that way).
+int64_t mlr_decay_scan_scratch(int tokens, int entries, int heads, int key_heads, int dim, int vdim, int delta) {
+  if (tokens <= 0 || entries <= 0 || heads <= 0 || key_heads <= 0 || dim <= 0 || vdim <= 0 || dim > 128) return 0;
+  const int64_t cells = (static_cast<int64_t>(tokens) / kChunk + entries) * heads;
+  return cells * scratch_floats_per_chunk(padded_rows(dim), (vdim + 15) / 16 * 16, delta);
+}
 
 int mlr_decay_scan(const float* x, int channels, int q_off, int k_off, int v_off, const float* gates, float* state,
                    int state_rows, const int* read_rows, const int* write_rows, const int* cu_q, const int* q_starts,
@@ -338,6 +913,59 @@ int mlr_decay_scan(const float* x, int channels, int q_off, int k_off, int v_off
   MLR_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && q_off + key_heads * dim <= channels &&
                   k_off + key_heads * dim <= channels && v_off + heads * vdim <= channels,
               "the rows do not hold what the offsets name");
+  MLR_REQUIRE(skip == nullptr || !delta, "the delta rule's scan adds no skip");
+  const int64_t needed = mlr_decay_scan_scratch(tokens, entries, heads, key_heads, dim, vdim, delta);
+  if (scratch != nullptr && needed > 0) {
+    MLR_REQUIRE(scratch_floats >= needed, "the scratch memory is too small");
+    MLR_REQUIRE(entries < 65536, "too many entries for one launch");
+    const int chunks = tokens / kChunk + entries;
+    const int dp = padded_rows(dim), vpad = (vdim + 15) / 16 * 16;
+    const ChunkScratch s = chunk_scratch(scratch, static_cast<int64_t>(chunks) * heads, dp, vpad, delta);
+#define MLR_CHUNKS(DP, DELTA)                                                                                          \
+  do {                                                                                                               \
+    constexpr int kLds = 2 * kChunk * (DP + 8) * 4;                                                                  \
+    constexpr int kApplyLds = kLds > (kChunk * (DP + 8) + kChunk * kMatLd) * 4 ? kLds : (kChunk * (DP + 8) + kChunk * kMatLd) * 4; \
+    static bool configured = false;                                                                                  \
+    if (!configured) {                                                                                               \
+      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(decay_apply_kernel<DP, DELTA>),          \
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, kApplyLds);               \
+      if (e != hipSuccess) {                                                                                         \
+        set_error(std::string("mlr_decay_scan: cannot raise the LDS limit: ") + hipGetErrorString(e));               \
+        return -1;                                                                                                   \
+      }                                                                                                              \
+      configured = true;                                                                                             \
+    }                                                                                                                \
+    decay_local_kernel<DP, DELTA><<<dim3(chunks, heads), 256, 0, stream>>>(x, channels, k_off, v_off, gates, cu_q,    \
+                                                                           entries, heads, key_heads, dim, vdim, s); \
+    MLR_LAUNCH_CHECK();                                                                                              \
+    if constexpr (DELTA)                                                                                             \
+      delta_carry_kernel<DP><<<dim3(vpad / 16, heads, entries), 256, 0, stream>>>(state, read_rows, write_rows, cu_q, \
+                                                                                  q_starts, heads, dim, vdim, s);    \
+    else                                                                                                             \
+      plain_carry_kernel<<<dim3(entries, heads, (dp * vpad + 255) / 256), 256, 0, stream>>>(                         \
+          state, read_rows, write_rows, cu_q, q_starts, heads, dim, vdim, s);                                        \
+    MLR_LAUNCH_CHECK();                                                                                              \
+    decay_apply_kernel<DP, DELTA><<<dim3(chunks, heads), 256, kApplyLds, stream>>>(                                   \
+        x, channels, q_off, k_off, v_off, gates, cu_q, q_starts, skip, out, entries, heads, key_heads, dim, vdim, s); \
+    MLR_LAUNCH_CHECK();                                                                                              \
+  } while (0)
+#define MLR_CHUNKS_SIZED(DELTA) \
+  do {                          \
+    if (dp == 32)               \
+      MLR_CHUNKS(32, DELTA);    \
+    else if (dp == 64)          \
+      MLR_CHUNKS(64, DELTA);    \
+    else                        \
+      MLR_CHUNKS(128, DELTA);   \
+  } while (0)
+    if (delta)
+      MLR_CHUNKS_SIZED(true);
+    else
+      MLR_CHUNKS_SIZED(false);
+#undef MLR_CHUNKS_SIZED
+#undef MLR_CHUNKS
+    return 0;
+  }
 #define MLR_WALK(R, DELTA)                                                                                        \
   decay_walk_kernel<R, DELTA><<<dim3(entries, heads, (vdim + 63) / 64), 256, 0, stream>>>(                         \
       x, channels, q_off, k_off, v_off, gates, state, read_rows, write_rows, cu_q, q_starts, skip, out, heads,    \
