@@ -561,25 +561,40 @@ __global__ __launch_bounds__(256) void plain_carry_kernel(float* __restrict__ st
 
 // The delta rule's walk over an entry's chunks for 16 value columns of one head: U = U0 - X S, S' = exp(A_n) S + K^T (e(n, .) U).
 // Wavefront w owns the rows 16 w .. of U and every fourth 16-row tile of S (in registers, a D tile each); both go
-// through LDS as B operands.  The next chunk's X, K and U0 are on their way meanwhile.
+// through LDS as B operands.  A chunk's X, K and U0 are asked for a whole chunk ahead.  All strips of a head read the
+// same X and K: workgroup b runs on accelerator die b % 8, so a head's strips are dealt to one die and share its L2.
+template <int DP>
+struct CarryOperands {
+  f32x4 x[DP / 16], u0, last;
+  float k[(DP / 16 + 3) / 4][16];
+  float keep;
+};
+
+constexpr int kDies = 8;
+
 template <int DP>
 __global__ __launch_bounds__(256) void delta_carry_kernel(float* __restrict__ state, const int* __restrict__ read_rows,
                                                           const int* __restrict__ write_rows, const int* __restrict__ cu_q,
-                                                          const int* __restrict__ q_starts, int heads, int dim, int vdim,
-                                                          ChunkScratch s) {
+                                                          const int* __restrict__ q_starts, int entries, int heads, int dim,
+                                                          int vdim, ChunkScratch s) {
   constexpr int kTiles = DP / 16;
   constexpr int kOwn = (kTiles + 3) / 4;  // tiles of S a wavefront owns at most
   __shared__ __attribute__((aligned(16))) f32x4 Sb[kTiles][kWave];
   __shared__ __attribute__((aligned(16))) f32x4 Ub[4][kWave];
-  const int entry = blockIdx.z;
-  const int h = blockIdx.y;
+  const int vpad = s.vpad;
+  const int strips = vpad / 16;
+  const int slot = blockIdx.x / kDies;
+  const int unit = slot / strips * kDies + blockIdx.x % kDies;  // (entry, head)
+  const int strip = slot % strips;
+  if (unit >= entries * heads) return;
+  const int entry = unit / heads;
+  const int h = unit - entry * heads;
   const int tid = threadIdx.x;
   const int lane = tid % kWave;
   const int w = __builtin_amdgcn_readfirstlane(tid / kWave);
   const int r16 = lane % 16;
   const int quad = lane / 16;
-  const int col = blockIdx.x * 16 + r16;
-  const int vpad = s.vpad;
+  const int col = strip * 16 + r16;
   const int count = chunks_of(cu_q[entry + 1] - cu_q[entry]);
   int first = 0;
   for (int e = 0; e < entry; ++e) first += chunks_of(cu_q[e + 1] - cu_q[e]);
@@ -596,14 +611,16 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(float* __restrict__ st
       S[o][e] = (!fresh && d < dim && col < vdim) ? src[static_cast<int64_t>(d) * vdim + col] : 0.f;
     }
 
-  f32x4 xa[kTiles], u0, last;
-  float ka[kOwn][16];
-  float keep;
-  auto fetch = [&](int c) {
+  auto fetch = [&](CarryOperands<DP>& op, int c) {
     const int64_t cell = static_cast<int64_t>(first + c) * heads + h;
     const float* xr = s.x + (cell * kChunk + 16 * w + r16) * DP + 4 * quad;
 #pragma unroll
-    for (int g = 0; g < kTiles; ++g) xa[g] = *reinterpret_cast<const f32x4*>(xr + 16 * g);
+    for (int g = 0; g < kTiles; ++g) op.x[g] = *reinterpret_cast<const f32x4*>(xr + 16 * g);
+    const float* ur = s.u + (cell * kChunk + 16 * w + 4 * quad) * vpad + col;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) op.u0[e] = ur[e * vpad];
+    op.last = *reinterpret_cast<const f32x4*>(s.last + cell * kChunk + 16 * w + 4 * quad);
+    op.keep = s.decay[cell];
     const float* kr = s.k + (cell * kChunk + 4 * quad) * DP + r16;
 #pragma unroll
     for (int o = 0; o < kOwn; ++o) {
@@ -611,65 +628,65 @@ __global__ __launch_bounds__(256) void delta_carry_kernel(float* __restrict__ st
 #pragma unroll
       for (int b = 0; b < 4; ++b)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) ka[o][4 * b + e] = kr[(16 * b + e) * DP + 16 * tile];
+        for (int e = 0; e < 4; ++e) op.k[o][4 * b + e] = kr[(16 * b + e) * DP + 16 * tile];
     }
-    const float* ur = s.u + (cell * kChunk + 16 * w + 4 * quad) * vpad + blockIdx.x * 16 + r16;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) u0[e] = ur[e * vpad];
-    last = *reinterpret_cast<const f32x4*>(s.last + cell * kChunk + 16 * w + 4 * quad);
-    keep = s.decay[cell];
   };
-  fetch(0);
-  for (int c = 0; c < count; ++c) {
+  auto step = [&](const CarryOperands<DP>& op, CarryOperands<DP>& next, int c) {
     const int64_t cell = static_cast<int64_t>(first + c) * heads + h;
-    float* before = s.state + cell * DP * vpad + blockIdx.x * 16 + r16;
+    float* before = s.state + cell * DP * vpad + col;
 #pragma unroll
     for (int o = 0; o < kOwn; ++o) {
       const int tile = w + 4 * o;
-      if (tile < kTiles) {
-        Sb[tile][lane] = S[o];
-#pragma unroll
-        for (int e = 0; e < 4; ++e) before[static_cast<int64_t>(16 * tile + 4 * quad + e) * vpad] = S[o][e];
-      }
+      if (kTiles % 4 == 0 || tile < kTiles) Sb[tile][lane] = S[o];
     }
     __syncthreads();
+    // asked for without a condition (past the end: the last chunk again): a load inside a conditional block would make the
+    // compiler wait for every load on its way where the block ends
+    fetch(next, min(c + 1, count - 1));
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int o = 0; o < kOwn; ++o) {
+      const int tile = w + 4 * o;
+      if (kTiles % 4 == 0 || tile < kTiles)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) before[static_cast<int64_t>(16 * tile + 4 * quad + e) * vpad] = S[o][e];
+    }
     f32x4 held[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
     for (int g = 0; g < kTiles; ++g) {
       const f32x4 sb = Sb[g][lane];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) held[e % 2] = mfma_f32(xa[g][e], sb[e], held[e % 2]);
+      for (int e = 0; e < 4; ++e) held[e % 2] = mfma_f32(op.x[g][e], sb[e], held[e % 2]);
     }
-    const f32x4 u = u0 - (held[0] + held[1]);
-    float* ur = s.u + (cell * kChunk + 16 * w + 4 * quad) * vpad + blockIdx.x * 16 + r16;
+    const f32x4 u = op.u0 - (held[0] + held[1]);
+    Ub[w][lane] = u * op.last;
+    __syncthreads();
+    float* ur = s.u + (cell * kChunk + 16 * w + 4 * quad) * vpad + col;
 #pragma unroll
     for (int e = 0; e < 4; ++e) ur[e * vpad] = u[e];
-    Ub[w][lane] = u * last;
-    const float decay = keep;
-    float kb[kOwn][16];
-#pragma unroll
-    for (int o = 0; o < kOwn; ++o)
-#pragma unroll
-      for (int b = 0; b < 16; ++b) kb[o][b] = ka[o][b];
-    if (c + 1 < count) fetch(c + 1);
-    __syncthreads();
     f32x4 ub[4];
 #pragma unroll
     for (int b = 0; b < 4; ++b) ub[b] = Ub[b][lane];
 #pragma unroll
     for (int o = 0; o < kOwn; ++o) {
       f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-      S[o] *= decay;
+      S[o] *= op.keep;
 #pragma unroll
       for (int b = 0; b < 4; ++b) {
 #pragma unroll
         for (int e = 0; e < 4; e += 2) {
-          S[o] = mfma_f32(kb[o][4 * b + e], ub[b][e], S[o]);
-          acc = mfma_f32(kb[o][4 * b + e + 1], ub[b][e + 1], acc);
+          S[o] = mfma_f32(op.k[o][4 * b + e], ub[b][e], S[o]);
+          acc = mfma_f32(op.k[o][4 * b + e + 1], ub[b][e + 1], acc);
         }
       }
       S[o] += acc;
     }
+  };
+  CarryOperands<DP> even, odd;
+  fetch(even, 0);
+  for (int c = 0; c < count; c += 2) {
+    step(even, odd, c);
+    if (c + 1 < count) step(odd, even, c + 1);
   }
   float* dst = state + (static_cast<int64_t>(write_rows[entry]) * heads + h) * head_state;
 #pragma unroll
@@ -741,46 +758,47 @@ __global__ __launch_bounds__(256) void decay_apply_kernel(const float* __restric
   __syncthreads();
   const bool carried = !(place == 0 && q_starts[entry] == 0);  // else the state before the chunk is zero
   const float d_skip = skip != nullptr ? skip[h] : 0.f;
-  for (int strip = w; strip < vpad / 16; strip += 4) {
+  // a strip's u and state, all asked for before the first is used
+  struct Strip {
+    f32x4 u[4], s[DP / 16];
+  };
+  auto fetch = [&](Strip& t, int strip) {
     const int c = strip * 16 + r16;
-    f32x4 u[4];
     if constexpr (DELTA) {
 #pragma unroll
       for (int b = 0; b < 4; ++b)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) u[b][e] = s.u[(cell * kChunk + 16 * b + 4 * quad + e) * vpad + c];
+        for (int e = 0; e < 4; ++e) t.u[b][e] = s.u[(cell * kChunk + 16 * b + 4 * quad + e) * vpad + c];
     } else {
 #pragma unroll
       for (int b = 0; b < 4; ++b)
 #pragma unroll
         for (int e = 0; e < 4; ++e)
-          u[b][e] = x[static_cast<int64_t>(t0 + min(16 * b + 4 * quad + e, n - 1)) * channels + v_off +
-                      static_cast<int64_t>(h) * vdim + min(c, vdim - 1)];
+          t.u[b][e] = x[static_cast<int64_t>(t0 + min(16 * b + 4 * quad + e, n - 1)) * channels + v_off +
+                        static_cast<int64_t>(h) * vdim + min(c, vdim - 1)];
     }
+    const float* before = s.state + cell * DP * vpad + c;  // zeros before a request's first chunk
+#pragma unroll
+    for (int g = 0; g < DP / 16; ++g)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) t.s[g][e] = before[static_cast<int64_t>(16 * g + 4 * quad + e) * vpad];
+    __builtin_amdgcn_sched_barrier(0);  // all asked for here, not each where it is used
+  };
+  auto compute = [&](const Strip& t, int strip) {
+    const int c = strip * 16 + r16;
     f32x4 o[4];
 #pragma unroll
     for (int b = 0; b < 4; ++b) o[b] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (carried) {
-      const float* before = s.state + cell * DP * vpad + c;
-      constexpr int kHalf = DP / 16 > 4 ? 4 : DP / 16;  // tiles of the state in registers at a time
 #pragma unroll
-      for (int g0 = 0; g0 < DP / 16; g0 += kHalf) {
-        f32x4 sb[kHalf];
+      for (int g = 0; g < DP / 16; ++g) {
+        f32x4 q[4];
 #pragma unroll
-        for (int g = 0; g < kHalf; ++g)
+        for (int b = 0; b < 4; ++b) q[b] = *reinterpret_cast<const f32x4*>(&Qs[(16 * b + r16) * LD + 16 * g + 4 * quad]);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) sb[g][e] = before[static_cast<int64_t>(16 * (g0 + g) + 4 * quad + e) * vpad];
+        for (int e = 0; e < 4; ++e)
 #pragma unroll
-        for (int g = 0; g < kHalf; ++g) {
-          f32x4 q[4];
-#pragma unroll
-          for (int b = 0; b < 4; ++b)
-            q[b] = *reinterpret_cast<const f32x4*>(&Qs[(16 * b + r16) * LD + 16 * (g0 + g) + 4 * quad]);
-#pragma unroll
-          for (int e = 0; e < 4; ++e)
-#pragma unroll
-            for (int b = 0; b < 4; ++b) o[b] = mfma_f32(q[b][e], sb[g][e], o[b]);
-        }
+          for (int b = 0; b < 4; ++b) o[b] = mfma_f32(q[b][e], t.s[g][e], o[b]);
       }
 #pragma unroll
       for (int b = 0; b < 4; ++b)
@@ -795,7 +813,7 @@ __global__ __launch_bounds__(256) void decay_apply_kernel(const float* __restric
 #pragma unroll
       for (int e = 0; e < 4; ++e)
 #pragma unroll
-        for (int b = k; b < 4; ++b) o[b] = mfma_f32(p[b][e], u[k][e], o[b]);
+        for (int b = k; b < 4; ++b) o[b] = mfma_f32(p[b][e], t.u[k][e], o[b]);
     }
     if (c < vdim) {
 #pragma unroll
@@ -805,11 +823,16 @@ __global__ __launch_bounds__(256) void decay_apply_kernel(const float* __restric
           const int i = 16 * b + 4 * quad + e;
           if (i < n) {
             float v = o[b][e];
-            if (!DELTA && skip != nullptr) v = fmaf(d_skip, u[b][e], v);
+            if (!DELTA && skip != nullptr) v = fmaf(d_skip, t.u[b][e], v);
             out[(static_cast<int64_t>(t0 + i) * heads + h) * vdim + c] = v;
           }
         }
     }
+  };
+  for (int strip = w; strip < vpad / 16; strip += 4) {
+    Strip t;
+    fetch(t, strip);
+    compute(t, strip);
   }
 }
 
@@ -939,8 +962,8 @@ int mlr_decay_scan(const float* x, int channels, int q_off, int k_off, int v_off
                                                                            entries, heads, key_heads, dim, vdim, s); \
     MLR_LAUNCH_CHECK();                                                                                              \
     if constexpr (DELTA)                                                                                             \
-      delta_carry_kernel<DP><<<dim3(vpad / 16, heads, entries), 256, 0, stream>>>(state, read_rows, write_rows, cu_q, \
-                                                                                  q_starts, heads, dim, vdim, s);    \
+      delta_carry_kernel<DP><<<static_cast<unsigned>((entries * heads + kDies - 1) / kDies * kDies * (vpad / 16)), 256, 0, \
+                               stream>>>(state, read_rows, write_rows, cu_q, q_starts, entries, heads, dim, vdim, s); \
     else                                                                                                             \
       plain_carry_kernel<<<dim3(entries, heads, (dp * vpad + 255) / 256), 256, 0, stream>>>(                         \
           state, read_rows, write_rows, cu_q, q_starts, heads, dim, vdim, s);                                        \

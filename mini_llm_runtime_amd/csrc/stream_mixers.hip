@@ -196,7 +196,8 @@ __global__ __launch_bounds__(256) void streams_fill_kernel(const float* __restri
 //  * every value head divided by its root mean square over vdim; (v_keep) the normed values as float32 [tokens,
 //    kv_heads * vdim]; (v_first) v = (1 - lambda) v + lambda v_first[t]; values to [page, kv_head, D, offset];
 //  * gate[t, head] = sigmoid(logit).
-// One wavefront per head; a negative slot stores nothing.
+// One wavefront per head (four heads a workgroup; the grid's second axis takes the others, as far as it reaches); a
+// negative slot stores nothing.
 // q_weight given (and k_weight [dim], with keys): a head is divided by its root mean square and multiplied by that
 // weight BEFORE it turns, and the values are stored as they are.  kv_heads 0: the rows hold queries only.
 template <typename T>
@@ -220,7 +221,7 @@ __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
   const bool store = page >= 0 && page < num_pages;
   const float lambda = (v_first != nullptr && lambda_p != nullptr) ? lambda_p[0] : 0.f;
   const int jobs = heads + 2 * kv_heads;
-  for (int job = wave; job < jobs; job += 4) {
+  for (int job = blockIdx.y * 4 + wave; job < jobs; job += 4 * gridDim.y) {
     const bool is_q = job < heads;
     const bool is_k = !is_q && job < heads + kv_heads;
     const int h = is_q ? job : (is_k ? job - heads : job - heads - kv_heads);
@@ -283,7 +284,7 @@ __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
       }
     }
   }
-  if (gate != nullptr) {
+  if (gate != nullptr && blockIdx.y == 0) {
     const float* z = row + (heads + kv_heads) * dim + kv_heads * vdim;
     for (int h = threadIdx.x; h < heads; h += 256) gate[t * heads + h] = 1.0f / (1.0f + expf(-z[h]));
   }
@@ -615,13 +616,16 @@ int mlr_head_norm_rope_write(const float* projected, int width, void* q_out, flo
   MLR_REQUIRE(v_first == nullptr || lambda, "mixing values in needs its weight");
   MLR_REQUIRE(kv_heads == 0 || (block_size > 0 && num_pages > 0), "page sizes must be > 0");
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
+  // few tokens: every wavefront one head; many: a workgroup takes a token's heads in turn
+  const dim3 grid(tokens, tokens <= 256 ? (heads + 2 * kv_heads + 3) / 4 : 1);
+  MLR_REQUIRE(grid.y < 65536u, "too many heads for one launch");
   if (dtype == kF32)
-    head_norm_rope_write_kernel<float><<<tokens, 256, 0, stream>>>(
+    head_norm_rope_write_kernel<float><<<grid, 256, 0, stream>>>(
         projected, width, static_cast<float*>(q_out), gate, cos, sin, rotary_dims, eps, slots,
         static_cast<float*>(key_pages), static_cast<float*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight,
         weight_is_f32, heads, kv_heads, dim, vdim, kernel_dim, block_size, num_pages);
   else
-    head_norm_rope_write_kernel<bf16><<<tokens, 256, 0, stream>>>(
+    head_norm_rope_write_kernel<bf16><<<grid, 256, 0, stream>>>(
         projected, width, static_cast<bf16*>(q_out), gate, cos, sin, rotary_dims, eps, slots,
         static_cast<bf16*>(key_pages), static_cast<bf16*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight,
         weight_is_f32, heads, kv_heads, dim, vdim, kernel_dim, block_size, num_pages);

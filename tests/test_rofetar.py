@@ -211,13 +211,13 @@ GPU_CASES = [
 ]
 
 
-def _compare(got, requests, weights, cfg, dtype, f32_bound=3e-4, row_bound=6e-2, together=3e-2):
+def _compare(got, requests, weights, cfg, dtype, f32_bound=3e-4, row_bound=6e-2, together=3e-2, worst_row=4.0):
     """float32: every value within 3e-4 of the logits' size, or within 4 times of what rounding the inputs of the
     products to float32 does to the worst row (a sublayer's output is divided by its own size on its way into the
     stream, so where a head's read-out nearly vanishes any rounding is blown up).  bfloat16: all rows together
     within 3 % (relative L2, the mean over the vocabulary taken off) or twice what rounding alone does; every row
     within 6 %, but for a few (one in twenty, and as many as rounding alone puts beyond 6 %) that may be off by up
-    to 4 times what rounding alone does to the worst row of their request.  A wrong key, page, slot or state
+    to `worst_row` times what rounding alone does to the worst row of their request.  A wrong key, page, slot or state
     changes most rows, by half and more."""
     assert got, "no logits came back"
     w64 = _f64(weights)
@@ -244,7 +244,7 @@ def _compare(got, requests, weights, cfg, dtype, f32_bound=3e-4, row_bound=6e-2,
             rel = float(diff.pow(2).sum().sqrt() / ref[pos].pow(2).sum().sqrt())
             if rel >= row_bound:
                 loose += 1
-                assert rel < 4.0 * max(float(alone.max()), row_bound / 2), f"{rid}:{pos}: relative error {rel:.3e}, rounding alone up to {float(alone.max()):.3e}"
+                assert rel < worst_row * max(float(alone.max()), row_bound / 2), f"{rid}:{pos}: relative error {rel:.3e}, rounding alone up to {float(alone.max()):.3e}"
                 continue
             num += float(diff.pow(2).sum())
             num_alone += float((coarse[pos] - ref[pos]).pow(2).sum())
