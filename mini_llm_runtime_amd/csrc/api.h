@@ -322,6 +322,12 @@ int mlr_decay_scan(const float* x, int channels, int q_off, int k_off, int v_off
                    int state_rows, const int* read_rows, const int* write_rows, const int* cu_q, const int* q_starts,
                    const float* skip, float* out, int entries, int heads, int key_heads, int dim, int vdim, int tokens,
                    int delta, float* scratch, int64_t scratch_floats, hipStream_t stream);
+int mlr_decay_step(const float* projected, int width, int column, const float* taps, const float* bias, float* carried,
+                   int carried_rows, const int* carried_read, const int* carried_write, int channels, int n_taps,
+                   float unit_scale, const float* rate, const float* dt_bias, int step_column, int write_column, int q_off,
+                   int k_off, int v_off, float* state, int state_rows, const int* read_rows, const int* write_rows,
+                   const int* q_starts, const float* skip, float* out, int entries, int heads, int key_heads, int dim,
+                   int vdim, int delta, hipStream_t stream);
 int mlr_gate_group_norm(const float* y, const float* projected, int width, int gate_column, void* out, int dtype,
                         int tokens, int inner, int groups, float eps, const void* weight, int weight_is_f32,
                         hipStream_t stream);

@@ -245,6 +245,173 @@ __global__ __launch_bounds__(256) void decay_walk_kernel(
   }
 }
 
+// ---- one token per entry: convolution, gates and scan in one kernel ---------------------------------------------
+// What conv_gates_kernel and decay_walk_kernel do for a step in which every entry has a single token (entry e is token
+// e), for convolutions of up to kStepTaps taps.  A workgroup owns 64 value columns of one head of one entry and makes
+// the head's q and k and its columns' v itself; the carried inputs of q's and k's channels are written by the first
+// head of those that share them (and its first columns), those of v's channels by their owner.
+constexpr int kStepTaps = 4;
+
+struct StepConv {
+  const float* p;  // [tokens, width]; the convolution's channels start at `column`
+  int width, column, n_taps;
+  const float *taps, *bias;
+  float* carried;  // [rows, n_taps - 1, channels]
+  const int *read_rows, *write_rows;
+  const float *rate, *dt_bias;
+  int step_column, write_column;
+  float unit_scale;  // of q (unit heads only)
+};
+
+template <int R, bool DELTA>  // R: rows of the state a lane holds, dim <= 4 * R; DELTA: unit q and k, else as they are
+__global__ __launch_bounds__(256) void decay_step_kernel(StepConv in, int channels, int q_off, int k_off, int v_off,
+                                                         float* __restrict__ state, const int* __restrict__ read_rows,
+                                                         const int* __restrict__ write_rows,
+                                                         const int* __restrict__ q_starts, const float* __restrict__ skip,
+                                                         float* __restrict__ out, int heads, int key_heads, int dim,
+                                                         int vdim) {
+  constexpr int MAXD = 4 * R;
+  constexpr int kGroup = R + 4;
+  constexpr int kRounds = (2 * MAXD + 255) / 256;
+  __shared__ __attribute__((aligned(16))) float qk[2][4][kGroup];
+  __shared__ float sv[64];
+  __shared__ float sg[2];
+  __shared__ float squares[kRounds][4];
+  const int entry = blockIdx.x;
+  const int h = blockIdx.y;
+  const int group = heads / key_heads;
+  const int kh = h / group;
+  const int tid = threadIdx.x;
+  const int lane = tid % kWave;
+  const int wave = tid / kWave;
+  const int g = lane / 16;
+  const int c_local = wave * 16 + lane % 16;
+  const int col = blockIdx.z * 64 + c_local;
+  const bool col_ok = col < vdim;
+  const bool fresh = q_starts[entry] == 0;
+  const int64_t per_head = static_cast<int64_t>(dim) * vdim;
+  const float* src = state + (static_cast<int64_t>(read_rows[entry]) * heads + h) * per_head;
+  float* dst = state + (static_cast<int64_t>(write_rows[entry]) * heads + h) * per_head;
+  // the state is on its way while the token's q, k and v are made (what is absent reads element 0)
+  float S[R];
+#pragma unroll
+  for (int j = 0; j < R; ++j) {
+    const int r = g * R + j;
+    S[j] = src[(r < dim && col_ok) ? static_cast<int64_t>(r) * vdim + col : 0];
+  }
+  const float* row = in.p + static_cast<int64_t>(entry) * in.width;
+  const int carried = in.n_taps - 1;
+  const bool keeps = carried > 0;
+  const float* old = keeps ? in.carried + static_cast<int64_t>(in.read_rows[entry]) * carried * channels : row;
+  float* kept = keeps ? in.carried + static_cast<int64_t>(in.write_rows[entry]) * carried * channels : nullptr;
+  auto convolved = [&](int c, bool owner) {  // channel c: convolution and activation; `owner` writes its inputs
+    float x[kStepTaps], w[kStepTaps];
+    const float now = row[in.column + c];
+#pragma unroll
+    for (int k = 0; k < kStepTaps - 1; ++k)  // x[k]: the input k + 1 tokens ago
+      x[k] = k < carried && !fresh ? old[static_cast<int64_t>(carried - 1 - k) * channels + c] : 0.f;
+#pragma unroll
+    for (int k = 0; k < kStepTaps; ++k) w[k] = k <= carried ? in.taps[static_cast<int64_t>(carried - k) * channels + c] : 0.f;
+    float acc = in.bias != nullptr ? in.bias[c] : 0.f;
+#pragma unroll
+    for (int k = kStepTaps - 1; k > 0; --k)
+      if (k <= carried) acc = fmaf(w[k], x[k - 1], acc);  // the oldest first, as in conv_gates_kernel
+    acc = fmaf(w[0], now, acc);
+    if (owner && keeps) {
+#pragma unroll
+      for (int k = 0; k < kStepTaps - 1; ++k)
+        if (k < carried) kept[static_cast<int64_t>(carried - 1 - k) * channels + c] = k == 0 ? now : x[k - 1];
+    }
+    return silu_f32(acc);
+  };
+  const bool first = h == kh * group && blockIdx.z == 0;
+  float made[kRounds];
+#pragma unroll
+  for (int u = 0; u < kRounds; ++u) {
+    const int idx = tid + u * 256;
+    const int which = idx / MAXD;  // 0: q, 1: k
+    const int r = idx % MAXD;
+    made[u] = 0.f;
+    if (which < 2 && r < dim) made[u] = convolved((which ? k_off : q_off) + kh * dim + r, first);
+    if constexpr (DELTA) {
+      const float ss = wave_sum(made[u] * made[u]);
+      if (lane == 0) squares[u][wave] = ss;
+    }
+  }
+  if (wave == 3) {
+    const int c = blockIdx.z * 64 + lane;
+    sv[lane] = c < vdim ? convolved(v_off + h * vdim + c, true) : 0.f;
+  }
+  if (tid == 128) {
+    const float s = softplus_f32(row[in.step_column + h] + in.dt_bias[h]);
+    sg[0] = expf(in.rate[h] * s);
+    sg[1] = in.write_column >= 0 ? 1.0f / (1.0f + expf(-row[in.write_column + h])) : s;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int u = 0; u < kRounds; ++u) {
+    const int idx = tid + u * 256;
+    const int which = idx / MAXD;
+    const int r = idx % MAXD;
+    if (which < 2) {
+      float v = made[u];
+      if constexpr (DELTA) {
+        float ss = 0.f;
+#pragma unroll
+        for (int a = 0; a < kRounds; ++a)
+#pragma unroll
+          for (int b = 0; b < 4; ++b)
+            if ((a * 256 + b * 64) / MAXD == which) ss += squares[a][b];
+        v *= (which ? 1.0f : in.unit_scale) / sqrtf(ss + 1e-6f);
+      }
+      qk[which][r / R][r % R] = v;
+    }
+  }
+  __syncthreads();
+#pragma unroll
+  for (int j = 0; j < R; ++j)
+    if (!(g * R + j < dim && col_ok) || fresh) S[j] = 0.f;
+  const float keep = sg[0];
+  const float v = sv[c_local];
+  float u = v;
+  if constexpr (DELTA) {
+    float held = 0.f;
+#pragma unroll
+    for (int j = 0; j < R; j += 4) {
+      const f32x4 k4 = *reinterpret_cast<const f32x4*>(&qk[1][g][j]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[j + e] *= keep;
+        held = fmaf(S[j + e], k4[e], held);
+      }
+    }
+    held += __shfl_xor(held, 16, kWave);
+    held += __shfl_xor(held, 32, kWave);
+    u = v - held;
+  }
+  u *= sg[1];
+  float o = 0.f;
+#pragma unroll
+  for (int j = 0; j < R; j += 4) {
+    const f32x4 k4 = *reinterpret_cast<const f32x4*>(&qk[1][g][j]);
+    const f32x4 q4 = *reinterpret_cast<const f32x4*>(&qk[0][g][j]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      S[j + e] = DELTA ? fmaf(k4[e], u, S[j + e]) : fmaf(keep, S[j + e], k4[e] * u);
+      o = fmaf(S[j + e], q4[e], o);
+    }
+  }
+  o += __shfl_xor(o, 16, kWave);
+  o += __shfl_xor(o, 32, kWave);
+  if (g == 0 && col_ok)
+    out[(static_cast<int64_t>(entry) * heads + h) * vdim + col] = fmaf(skip != nullptr ? skip[h] : 0.f, v, o);
+#pragma unroll
+  for (int j = 0; j < R; ++j) {
+    const int r = g * R + j;
+    if (r < dim && col_ok) dst[static_cast<int64_t>(r) * vdim + col] = S[j];
+  }
+}
+
 // ---- the scan, 64 tokens at a time on the matrix cores ----------------------------------------------------------
 // In true 32-bit: v_mfma_f32_16x16x4_f32 takes and sums float32.  Within a chunk of n tokens (local index i, j; what is
 // beyond n is zero) with S the state before it, A_i = a_0 + .. + a_i (summed in float64: only differences of it are
@@ -1008,6 +1175,51 @@ int mlr_decay_scan(const float* x, int channels, int q_off, int k_off, int v_off
     MLR_WALK_SIZED(false);
 #undef MLR_WALK_SIZED
 #undef MLR_WALK
+  MLR_LAUNCH_CHECK();
+  return 0;
+}
+
+// Convolution, gates and scan of a step of single tokens (entry e is token e) in one kernel: mlr_conv_gates followed by
+// mlr_decay_scan, for up to 4 taps.  With `delta` q and k are unit heads (q times unit_scale), without it there are none.
+int mlr_decay_step(const float* projected, int width, int column, const float* taps, const float* bias, float* carried,
+                   int carried_rows, const int* carried_read, const int* carried_write, int channels, int n_taps,
+                   float unit_scale, const float* rate, const float* dt_bias, int step_column, int write_column, int q_off,
+                   int k_off, int v_off, float* state, int state_rows, const int* read_rows, const int* write_rows,
+                   const int* q_starts, const float* skip, float* out, int entries, int heads, int key_heads, int dim,
+                   int vdim, int delta, hipStream_t stream) {
+  MLR_REQUIRE(projected && taps && rate && dt_bias && state && read_rows && write_rows && q_starts && out, "null pointer");
+  MLR_REQUIRE(n_taps > 0 && n_taps <= kStepTaps, "up to 4 taps");
+  MLR_REQUIRE(n_taps == 1 || (carried && carried_read && carried_write && carried_rows > 0), "several taps carry inputs");
+  MLR_REQUIRE(entries > 0 && heads > 0 && heads < 65536 && key_heads > 0 && heads % key_heads == 0 && vdim > 0 && state_rows > 0,
+              "bad sizes");
+  MLR_REQUIRE(dim > 0 && dim <= 256, "states of up to 256 rows");
+  MLR_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && q_off + key_heads * dim <= channels &&
+                  k_off + key_heads * dim <= channels && v_off + heads * vdim <= channels &&
+                  channels == 2 * key_heads * dim + heads * vdim,
+              "the channels are those of q, k and v");
+  MLR_REQUIRE(column >= 0 && column + channels <= width && step_column >= 0 && step_column + heads <= width &&
+                  (write_column < 0 || write_column + heads <= width),
+              "the projected rows do not hold what the columns name");
+  const StepConv in{projected, width, column, n_taps, taps, bias, carried, carried_read, carried_write, rate, dt_bias,
+                    step_column, write_column, unit_scale};
+#define MLR_STEP(R, DELTA)                                                                                          \
+  decay_step_kernel<R, DELTA><<<dim3(entries, heads, (vdim + 63) / 64), 256, 0, stream>>>(                          \
+      in, channels, q_off, k_off, v_off, state, read_rows, write_rows, q_starts, skip, out, heads, key_heads, dim, vdim)
+#define MLR_STEP_SIZED(DELTA) \
+  do {                        \
+    if (dim <= 64)            \
+      MLR_STEP(16, DELTA);    \
+    else if (dim <= 128)      \
+      MLR_STEP(32, DELTA);    \
+    else                      \
+      MLR_STEP(64, DELTA);    \
+  } while (0)
+  if (delta)
+    MLR_STEP_SIZED(true);
+  else
+    MLR_STEP_SIZED(false);
+#undef MLR_STEP_SIZED
+#undef MLR_STEP
   MLR_LAUNCH_CHECK();
   return 0;
 }

@@ -40,6 +40,11 @@ _SIGNATURES = {
     "mlr_decay_scan": (
         [_VP, _I, _I, _I, _I, _VP, _VP, _I, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _VP, _I64, _VP], _I,
     ),
+    "mlr_decay_step": (
+        [_VP, _I, _I, _VP, _VP, _VP, _I, _VP, _VP, _I, _I, _F, _VP, _VP, _I, _I, _I, _I, _I, _VP, _I, _VP, _VP, _VP, _VP, _VP,
+         _I, _I, _I, _I, _I, _I, _VP],
+        _I,
+    ),
     "mlr_decay_scan_scratch": ([_I, _I, _I, _I, _I, _I, _I], _I64),
     "mlr_gate_group_norm": ([_VP, _VP, _I, _I, _VP, _I, _I, _I, _I, _F, _VP, _I, _VP], _I),
     "mlr_glu_clamped": ([_VP, _I, _VP, _I, _I, _I, _F, _F, _VP], _I),
@@ -1891,6 +1896,89 @@ class HipOps:
             state.shape[0], self._ptr(read_rows), self._ptr(write_rows), self._ptr(ctx.cu_q), self._ptr(ctx.q_starts),
             self._ptr(skip), self._ptr(out), entries, heads, key_heads, head_dim, value_dim, tokens, int(bool(delta)),
             self._ptr(scratch), floats, self._stream(),
+        )
+        return out
+
+    FUSED_STEP_TAPS = 4  # convolutions of up to this many taps run inside the scan of a step of single tokens
+
+    def conv_decay_scan(
+        self,
+        projected: torch.Tensor,
+        taps: torch.Tensor,
+        bias: Optional[torch.Tensor],
+        carried: Any,
+        state: Any,
+        ctx: Any,
+        *,
+        column: int,
+        heads: int,
+        key_heads: int,
+        head_dim: int,
+        value_dim: int,
+        offsets: Sequence[int],
+        rate: torch.Tensor,
+        dt_bias: torch.Tensor,
+        step_column: int,
+        write_column: Optional[int] = None,
+        delta: bool = False,
+        skip: Optional[torch.Tensor] = None,
+        fused: Optional[bool] = None,
+    ) -> torch.Tensor:
+        """A recurrence from its input product's sums to its heads' outputs, float32 [T, heads * value_dim]: `conv_gates`
+        (whose channels are q, k and v at `offsets`; with `delta` q and k are unit heads that lie in front, q times
+        head_dim^-0.5) and `decay_scan` behind it; `carried` and `state` are state views.  A step of single tokens is one kernel
+        (`fused` forces one way)."""
+        n, channels = taps.shape
+        tokens = projected.shape[0]
+        unit = float(head_dim) ** -0.5
+        q_off, k_off, v_off = (int(o) for o in offsets)
+        can = (
+            tokens == ctx.num_entries and n <= self.FUSED_STEP_TAPS and channels == 2 * key_heads * head_dim + heads * value_dim
+        )
+        if fused is None:
+            fused = can
+        elif fused and not can:
+            raise KernelError("the fused step takes single tokens, up to 4 taps and channels that are q, k and v")
+        if not fused:
+            units = {}
+            if delta:
+                if (q_off, k_off) != (0, key_heads * head_dim):
+                    raise KernelError("unit heads lie in front of the channels, q before k")
+                units = dict(unit_heads=2 * key_heads, unit_dim=head_dim, scaled_heads=key_heads, unit_scale=unit)
+            mixed, gates = self.conv_gates(
+                projected, taps, bias, carried, ctx, column=column, heads=heads, rate=rate, dt_bias=dt_bias,
+                step_column=step_column, write_column=write_column, **units,
+            )
+            return self.decay_scan(
+                mixed, gates, state.tensor, state.read_rows, state.write_rows, ctx, heads=heads, key_heads=key_heads,
+                head_dim=head_dim, value_dim=value_dim, offsets=offsets, delta=delta, skip=skip,
+            )
+        self._check(projected, "projected input", torch.float32, (None, None))
+        self._check(taps, "convolution taps", torch.float32, (n, channels))
+        if bias is not None:
+            self._check(bias, "convolution bias", torch.float32, (channels,))
+        held = held_read = held_write = None
+        if n > 1:
+            held, held_read, held_write = carried.tensor, carried.read_rows, carried.write_rows
+            self._check(held, "carried inputs", torch.float32, (None, n - 1, channels))
+            self._check(held_read, "state rows to read", torch.int32, (tokens,))
+            self._check(held_write, "state rows to write", torch.int32, (tokens,))
+        self._check(state.tensor, "recurrent state", torch.float32, (None, heads, head_dim, value_dim))
+        self._check(state.read_rows, "state rows to read", torch.int32, (tokens,))
+        self._check(state.write_rows, "state rows to write", torch.int32, (tokens,))
+        self._check(ctx.q_starts, "q_starts", torch.int32, (tokens,))
+        self._check(rate, "decay rates", torch.float32, (heads,))
+        self._check(dt_bias, "step bias", torch.float32, (heads,))
+        if skip is not None:
+            self._check(skip, "skip weights", torch.float32, (heads,))
+        out = self._empty((tokens, heads * value_dim), torch.float32)
+        self._call(
+            "mlr_decay_step", self._ptr(projected), projected.shape[1], int(column), self._ptr(taps), self._ptr(bias),
+            self._ptr(held), 0 if held is None else held.shape[0], self._ptr(held_read), self._ptr(held_write), channels, n,
+            unit, self._ptr(rate), self._ptr(dt_bias), int(step_column), -1 if write_column is None else int(write_column),
+            q_off, k_off, v_off, self._ptr(state.tensor), state.tensor.shape[0], self._ptr(state.read_rows),
+            self._ptr(state.write_rows), self._ptr(ctx.q_starts), self._ptr(skip), self._ptr(out), tokens, heads, key_heads,
+            head_dim, value_dim, int(bool(delta)), self._stream(),
         )
         return out
 

@@ -29,8 +29,9 @@ class GatedDelta(Mixer):
     the heads side by side are multiplied by silu(Wg h) and projected by Wo.
 
     A request keeps its state and the convolutions' last inputs (two members of the site in the cache manager's state
-    banks), so a prompt can be cut anywhere.  One input product (rows q, k, v, gate, a, b; 32-bit sums); a kernel for the
-    convolutions, activations, unit norms and gates; the scan; a kernel for norm and gate; the output product.
+    banks), so a prompt can be cut anywhere.  One input product (rows q, k, v, gate, a, b; 32-bit sums); convolutions,
+    activations, unit norms and gates, then the scan (one kernel where a step has single tokens only); a kernel for norm
+    and gate; the output product.
     """
 
     replayable = True
@@ -91,15 +92,11 @@ class GatedDelta(Mixer):
         ops = ctx.ops
         state, carried = conv_state_views(ctx, site, self.taps)
         projected = ops.linear(h, self.in_weight, None, out_dtype=torch.float32)  # what enters the recurrence stays 32-bit
-        mixed, gates = ops.conv_gates(
-            projected, self.conv_taps, None, carried, ctx, column=0, heads=self.num_heads, rate=self.rate,
-            dt_bias=self.dt_bias, step_column=self.step_at, write_column=self.write_at, unit_heads=2 * self.num_kv_heads,
-            unit_dim=self.head_dim, scaled_heads=self.num_kv_heads, unit_scale=float(self.head_dim) ** -0.5,
-        )
-        o = ops.decay_scan(
-            mixed, gates, state.tensor, state.read_rows, state.write_rows, ctx, heads=self.num_heads,
+        o = ops.conv_decay_scan(
+            projected, self.conv_taps, None, carried, state, ctx, column=0, heads=self.num_heads,
             key_heads=self.num_kv_heads, head_dim=self.head_dim, value_dim=self.value_dim,
-            offsets=(0, self.k_at, self.v_at), delta=True,
+            offsets=(0, self.k_at, self.v_at), rate=self.rate, dt_bias=self.dt_bias, step_column=self.step_at,
+            write_column=self.write_at, delta=True,
         )
         gated = ops.retention_gate(
             o, projected, heads=self.num_heads, value_dim=self.value_dim, gate_offset=self.gate_at, eps=self.norm_eps,

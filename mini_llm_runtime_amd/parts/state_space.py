@@ -42,8 +42,8 @@ class StateSpace(Mixer):
     root mean square, multiplied by a weight over all of them and projected by Wo.
 
     A request keeps its state and the convolution's last inputs (two members of the site in the cache manager's state
-    banks), so a prompt can be cut anywhere.  One input product with 32-bit sums; a kernel for the convolution, the
-    activation and the decays; the scan; a kernel for gate and norm; the output product.
+    banks), so a prompt can be cut anywhere.  One input product with 32-bit sums; convolution, activation and decays,
+    then the scan (one kernel where a step has single tokens only); a kernel for gate and norm; the output product.
     """
 
     replayable = True
@@ -109,15 +109,12 @@ class StateSpace(Mixer):
         ops = ctx.ops
         state, carried = conv_state_views(ctx, site, self.taps)
         projected = ops.linear(h, self.in_weight, None, out_dtype=torch.float32)  # what enters the recurrence stays 32-bit
-        mixed, gates = ops.conv_gates(
-            projected, self.conv_taps, self.conv_bias, carried, ctx, column=self.inner, heads=self.num_heads, rate=self.rate,
-            dt_bias=self.dt_bias, step_column=self.inner + self.channels,
-        )
-        x_at, b_at = 0, self.inner
-        y = ops.decay_scan(
-            mixed, gates, state.tensor, state.read_rows, state.write_rows, ctx, heads=self.num_heads, key_heads=self.groups,
-            head_dim=self.state_dim, value_dim=self.value_dim, offsets=(b_at + self.groups * self.state_dim, b_at, x_at),
-            skip=self.skip,
+        b_at = self.inner  # the channels: x, B, C
+        y = ops.conv_decay_scan(
+            projected, self.conv_taps, self.conv_bias, carried, state, ctx, column=self.inner, heads=self.num_heads,
+            key_heads=self.groups, head_dim=self.state_dim, value_dim=self.value_dim,
+            offsets=(b_at + self.groups * self.state_dim, b_at, 0), rate=self.rate, dt_bias=self.dt_bias,
+            step_column=self.inner + self.channels, skip=self.skip,
         )
         gated = ops.gate_group_norm(
             y, projected, gate_column=0, groups=self.norm_groups, eps=self.norm_eps, norm_weight=self.norm_weight

@@ -576,6 +576,23 @@ class TorchOps:
             out = out + skip[:, None] * v
         return out.view(tokens, heads * value_dim)
 
+    def conv_decay_scan(
+        self, projected, taps, bias, carried, state, ctx, *, column, heads, key_heads, head_dim, value_dim, offsets, rate,
+        dt_bias, step_column, write_column=None, delta=False, skip=None, fused=None,
+    ):
+        self._count("conv_decay_scan")
+        units = {}
+        if delta:
+            units = dict(unit_heads=2 * key_heads, unit_dim=head_dim, scaled_heads=key_heads, unit_scale=head_dim**-0.5)
+        mixed, gates = self.conv_gates(
+            projected, taps, bias, carried, ctx, column=column, heads=heads, rate=rate, dt_bias=dt_bias,
+            step_column=step_column, write_column=write_column, **units,
+        )
+        return self.decay_scan(
+            mixed, gates, state.tensor, state.read_rows, state.write_rows, ctx, heads=heads, key_heads=key_heads,
+            head_dim=head_dim, value_dim=value_dim, offsets=offsets, delta=delta, skip=skip,
+        )
+
     def gate_group_norm(self, y, projected, *, gate_column, groups, eps, norm_weight):
         self._count("gate_group_norm")
         tokens, inner = y.shape

@@ -421,6 +421,43 @@ def test_scan_and_its_state_rows(heads, key_heads, dim, vdim, delta, chunked):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("delta", [False, True], ids=["plain", "delta"])
+@pytest.mark.parametrize("taps", [1, 2, 4])
+@pytest.mark.parametrize("heads,key_heads,dim,vdim", [(2, 1, 16, 32), (6, 2, 64, 80), (3, 3, 100, 12), (4, 2, 144, 70), (1, 1, 1, 1)])
+def test_single_token_step_in_one_kernel(heads, key_heads, dim, vdim, taps, delta):
+    """Convolution, gates and scan of single tokens in one kernel: as the separate kernels, and as the stand-in; one
+    entry starts its request on rows of NaN."""
+    hip, double = _ops("hip", torch.float32), TorchOps(torch.float32, "cpu")
+    g = torch.Generator().manual_seed(heads * 100 + dim + taps)
+    starts, tokens = [4, 0, 1], 3
+    qk, v = key_heads * dim, heads * vdim
+    channels, column = 2 * qk + v, 6
+    offsets = (0, qk, 2 * qk) if delta else (v + qk, v, 0)
+    projected = torch.randn(tokens, column + channels + 2 * heads + 2, generator=g)
+    conv, bias = torch.randn(taps, channels, generator=g) * 0.5, None if delta else torch.randn(channels, generator=g) * 0.3
+    rate, dt_bias = -torch.rand(heads, generator=g) - 0.1, torch.randn(heads, generator=g)
+    skip = None if delta else torch.randn(heads, generator=g)
+    held = torch.randn(8, max(taps - 1, 1), channels, generator=g)
+    state = torch.randn(8, heads, dim, vdim, generator=g) * 0.5
+    held[5], state[5] = float("nan"), float("nan")
+    read, write = torch.tensor([2, 5, 6], dtype=torch.int32), torch.tensor([3, 4, 7], dtype=torch.int32)
+    results = []
+    for ops, fused in ((double, None), (hip, False), (hip, True)):
+        to = (lambda t: None if t is None else t.cuda()) if ops is hip else (lambda t: None if t is None else t.clone())
+        views = [SimpleNamespace(tensor=to(t), read_rows=to(read), write_rows=to(write)) for t in (held, state)]
+        out = ops.conv_decay_scan(
+            to(projected), to(conv), to(bias), views[0] if taps > 1 else None, views[1], _step_context([1] * tokens, starts, ops),
+            column=column, heads=heads, key_heads=key_heads, head_dim=dim, value_dim=vdim, offsets=offsets, rate=to(rate),
+            dt_bias=to(dt_bias), step_column=column + channels + 1,
+            write_column=column + channels + heads + 2 if delta else None, delta=delta, skip=to(skip), fused=fused,
+        )
+        results.append((out.cpu(), views[0].tensor.cpu(), views[1].tensor.cpu()))
+    for want, apart, one in zip(*results):
+        torch.testing.assert_close(one, want, rtol=2e-5, atol=1e-5, equal_nan=True)
+        torch.testing.assert_close(one, apart, rtol=2e-5, atol=1e-5, equal_nan=True)
+
+
+@pytest.mark.gpu
 def test_delta_scan_with_one_key_over_and_over():
     """The same key every token, writes of full strength, no decay: every write replaces the one before (the
     triangular system of a chunk is as far from the identity as it gets)."""
