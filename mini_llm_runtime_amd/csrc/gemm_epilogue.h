@@ -123,6 +123,21 @@ __device__ __forceinline__ float gelu_tanh(float v) {
   return v / (1.0f + __expf(-2.0f * u));
 }
 
+// kEpGeglu alone: a kernel whose epilogue is fixed when it is compiled stores through this, without the choices of store4.
+__device__ __forceinline__ void store_geglu4(const GemmEpilogue& ep, int64_t m, int n, int N, const float (&sums)[4]) {
+  float v[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = sums[i] + (ep.bias != nullptr ? load_as_f32(ep.bias, n + i, ep.bias_is_f32) : 0.f);
+  const float a = gelu_tanh(v[0]) * v[2], b = gelu_tanh(v[1]) * v[3];
+  const int64_t at = m * (N / 2) + n / 2;
+  if (ep.out_is_f32) {
+    static_cast<float*>(ep.y)[at] = a;
+    static_cast<float*>(ep.y)[at + 1] = b;
+  } else {
+    *reinterpret_cast<uint32_t*>(static_cast<bf16*>(ep.y) + at) = pack_bf16x2(a, b);
+  }
+}
+
 // Store four consecutive output features n..n+3 of token m (n is a multiple of 4).
 // ACTIVATIONS false leaves the element-wise activations and the multiplier out: for the one kernel
 // whose accumulators fill the register file (the 256 x 320 tile), where the longer epilogue made the

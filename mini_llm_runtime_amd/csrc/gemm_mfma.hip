@@ -576,7 +576,8 @@ constexpr int direct_lds_bytes(int tokens, int features, int waves, int bk, int 
   return buffers * (runs + (runs % waves != 0 ? 1 : 0)) * 1024;
 }
 
-template <int KEEP, int WM, int WN, int GM, int GN, int BKT = kBK, int NBUF = 2, bool ONCE = false>
+// FIXED: an epilogue fixed at compile time (kEpGeglu, for the tile that has no room for a choice), or -1.
+template <int KEEP, int WM, int WN, int GM, int GN, int BKT = kBK, int NBUF = 2, bool ONCE = false, int FIXED = -1>
 __global__ __launch_bounds__(64 * GM * GN) void gemm_direct_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
                                                                   GemmEpilogue ep, TileOrder order, int M, int N, int K) {
   constexpr int BM = 32 * WM * GM, BN = 32 * WN * GN, WAVES = GM * GN;
@@ -734,7 +735,11 @@ __global__ __launch_bounds__(64 * GM * GN) void gemm_direct_kernel(const bf16* _
         const int n = n0 + (wn * WN + i) * 32 + g * 8 + h * 4;
         const float v[4] = {acc[i][j][g * 4 + 0] * scale, acc[i][j][g * 4 + 1] * scale, acc[i][j][g * 4 + 2] * scale,
                             acc[i][j][g * 4 + 3] * scale};
-        finish4<(WM * WN < 10)>(ep, slice, slices, m, n, M, N, v);  // ten blocks a wavefront: the registers are full
+        if constexpr (FIXED == kEpGeglu) {
+          if (m < M && n < N) store_geglu4(ep, m, n, N, v);
+        } else {
+          finish4<(WM * WN < 10)>(ep, slice, slices, m, n, M, N, v);  // ten blocks a wavefront: the registers are full
+        }
       }
     }
 }
@@ -1063,6 +1068,11 @@ static int gemm_bf16(const bf16* xb, const bf16* wb, const GemmEpilogue& ep, int
                            configured, xb, wb, ep, m, n, k, slices, stream);
     }
     case 48: {  // 256 tokens x 320 features, eight wavefronts of 64 x 160
+      if (ep.swiglu == kEpGeglu) {
+        static bool configured_geglu = false;
+        return launch_direct(gemm_direct_kernel<1, 2, 5, 4, 2, kBK, 2, false, kEpGeglu>, 256, 320, 512, 4,
+                             direct_lds_bytes(256, 320, 8, 64, 2), configured_geglu, xb, wb, ep, m, n, k, slices, stream);
+      }
       static bool configured = false;
       return launch_direct(gemm_direct_kernel<1, 2, 5, 4, 2>, 256, 320, 512, 4, direct_lds_bytes(256, 320, 8, 64, 2), configured,
                            xb, wb, ep, m, n, k, slices, stream);
@@ -1160,8 +1170,9 @@ int mlr_gemm_bf16(const void* x, const void* w, const void* bias, int bias_is_f3
   GemmEpilogue ep{bias, bias_is_f32, y, out_is_f32, swiglu, row_sumsq, sumsq_parts, norm_eps, multiply, glu_limit, glu_alpha,
                   multiply_rows};
   if (kernel == 0) kernel = choose_kernel(m, n, k, slices);
-  // the 256 x 320 tile has no room for the activations and the multiplier in its epilogue
-  if (kernel == 48 && (swiglu >= kEpRelu2 || multiply != nullptr)) kernel = 45;
+  // the 256 x 320 tile has no room for a choice of activations and the multiplier in its epilogue (the GELU gating has an
+  // instance of its own)
+  if (kernel == 48 && ((swiglu >= kEpRelu2 && swiglu != kEpGeglu) || multiply != nullptr)) kernel = 45;
   if (gemm_bf16(static_cast<const bf16*>(x), static_cast<const bf16*>(w), ep, m, n, k, slices, kernel, stream) != 0)
     return -1;
   MLR_LAUNCH_CHECK();
