@@ -12,7 +12,7 @@ took and leaves the written bytes as invisible garbage.
 
 Beyond the reference: several groups (each with pages and a free list of its
 own), windows (pages that every later query has passed are given back at
-commit), capacity promised by count instead of by pinning pages, and state slots.
+commit, but for those of first tokens that a spec keeps for good), capacity promised by count instead of by pinning pages, and state slots.
 
 What lives in a page, and in which order, is the business of the sites' cache specs
 (`cache/spec.py`): the manager counts pages, rows and tokens and never asks what kind a
@@ -85,11 +85,17 @@ class KVGroup:
         """Pages that hold the entries of a request of `num_tokens` tokens."""
         return blocks_for(self.spec.entries_for(num_tokens), self.block_size)
 
-    def dead_blocks(self, num_tokens: int) -> int:
-        """How many leading pages no query at position >= num_tokens can see."""
+    @property
+    def kept_blocks(self) -> int:
+        """Leading pages of a request that are never given back while it lives."""
+        return blocks_for(int(getattr(self.spec, "keep_first", 0)), self.block_size)
+
+    def dead_blocks(self, num_tokens: int) -> tuple[int, int]:
+        """The pages [from, to) that no query at position >= num_tokens can see."""
         if self.stride != 1:
-            return 0  # entries of several tokens stay
-        return max(0, self.spec.first_live_position(num_tokens) // self.block_size)
+            return 0, 0  # entries of several tokens stay
+        kept = self.kept_blocks
+        return kept, max(kept, self.spec.first_live_position(num_tokens) // self.block_size)
 
     def lifetime_blocks(self, max_tokens: int, max_step_tokens: int) -> int:
         """Most pages a request holds at one time over its life."""
@@ -98,8 +104,8 @@ class KVGroup:
         if span is None:
             return full
         # what the first query of a step may still see (a window, the run of a chunked mask), the
-        # step's own tokens, and one page for the misalignment of the first live position
-        bounded = blocks_for(span + max_step_tokens, self.block_size) + 1
+        # step's own tokens, one page for the misalignment of the first live position, and what is kept for good
+        bounded = blocks_for(span + max_step_tokens, self.block_size) + 1 + self.kept_blocks
         return min(full, bounded)
 
     def storage_bytes(self) -> int:
@@ -521,14 +527,14 @@ class CacheManager:
             request.pending_tokens = 0
             request.state_parity ^= 1
             for i, g in enumerate(self.groups):
-                dead = g.dead_blocks(request.num_tokens)
-                ids = [b for b in request.tables[i][:dead] if b >= 0]
+                first, dead = g.dead_blocks(request.num_tokens)
+                ids = [b for b in request.tables[i][first:dead] if b >= 0]
                 if not ids:
                     continue
                 keep = len(ids) if request.has_reservation else 0
                 g.allocator.free(ids, to_reserved=keep)
                 request.reserved[i] += keep
-                for j in range(dead):
+                for j in range(first, dead):
                     request.tables[i][j] = -1
                 request.tables_changed()
                 passed.setdefault(request.request_id, {})[i] = tuple(ids)

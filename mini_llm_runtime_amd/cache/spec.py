@@ -44,6 +44,8 @@ class PagedSpec(SiteCacheSpec):
     chunk: an integer C likewise keeps only the run of C positions (runs counted from position 0)
     that the next query lies in: a query never sees beyond the start of its own run.
     The manager asks `first_live_position` and `live_span`, never which of the two it is.
+    keep_first: beside a window, the first `keep_first` positions of a request are seen by every later query and
+    kept for good.
 
     tokens_per_entry: 1 keeps something for every token.  An integer P > 1 keeps ONE entry for every
     run of P positions (runs counted from position 0), made when the run's last token comes in: the
@@ -55,13 +57,15 @@ class PagedSpec(SiteCacheSpec):
     window: Optional[int] = None
     chunk: Optional[int] = None
     tokens_per_entry: int = 1
+    keep_first: int = 0
 
     def entries_for(self, num_tokens: int) -> int:
         """Entries that a request of `num_tokens` tokens owns."""
         return num_tokens // self.tokens_per_entry
 
     def first_live_position(self, num_tokens: int) -> int:
-        """The first position that a query at position >= num_tokens may still see."""
+        """The first position, of those that are not kept for good, that a query at position >= num_tokens may still
+        see."""
         if self.window is not None:
             return max(0, num_tokens - self.window + 1)
         if self.chunk is not None:
@@ -166,8 +170,11 @@ class PagedKVSpec(PagedSpec):
     value_head_dim: Optional[int] = None
     chunk: Optional[int] = None
     tokens_per_entry: int = 1
+    keep_first: int = 0
 
     def __post_init__(self) -> None:
+        if self.keep_first < 0 or (self.keep_first and self.window is None):
+            raise ValueError("PagedKVSpec.keep_first must be >= 0 and goes with a window")
         if self.num_kv_heads <= 0 or self.head_dim <= 0:
             raise ValueError("PagedKVSpec sizes must be > 0")
         if self.tokens_per_entry <= 0 or (self.tokens_per_entry > 1 and (self.window or self.chunk)):

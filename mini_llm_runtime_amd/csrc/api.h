@@ -169,14 +169,17 @@ int mlr_paged_attention_simple(const void* q, int64_t q_stride, const void* key_
                                int block_size, int num_pages, float scale, int window, int chunk,
                                const float* sinks, const void* pooled_keys, const void* pooled_values,
                                const int* pooled_table, int pooled_width, int pooled_pages, int pool,
-                               const float* score_bias, float softcap, hipStream_t stream);
+                               const float* score_bias, float softcap, int keep_first, hipStream_t stream);
 
 // x (float32 [rows, hidden], in place) += weight * y * rsqrt(mean(y^2) + eps), y [rows, hidden] float32
 // or `dtype`, or `slices` float32 partial sums [slices, rows, hidden].  Then mode 1: out = next_weight * x *
 // rsqrt(mean(x^2) + next_eps), mode 2: out = x, both in `dtype`; mode 0: no output.
+// y2 (or null): a second output, normed by its own size with weight2; what is added then is scale * the first +
+// scale2 * the second.
 int mlr_add_normed(float* x, const void* y, int y_is_f32, int slices, const void* weight, int weight_is_f32, float eps,
-                   const void* next_weight, int next_is_f32, float next_eps, int mode, void* out, int dtype, int rows,
-                   int hidden, hipStream_t stream);
+                   const void* y2, int y2_is_f32, int slices2, const void* weight2, int weight2_is_f32, float scale,
+                   float scale2, const void* next_weight, int next_is_f32, float next_eps, int mode, void* out, int dtype,
+                   int rows, int hidden, hipStream_t stream);
 
 // out[m, i] = g * sigmoid(alpha * g) * (u + 1), g = min(sums[m, i], limit), u = clamp(sums[m, inter + i],
 // -limit, limit).
@@ -277,7 +280,8 @@ int mlr_streams_step(float* x, int streams, int tokens, int width, const int* ro
 int mlr_head_norm_rope_write(const float* projected, int width, void* q_out, float* gate, const float* cos,
                              const float* sin, int rotary_dims, float eps, const int* slots, void* key_pages,
                              void* value_pages, float* v_keep, const float* v_first, const float* lambda,
-                             const void* q_weight, const void* k_weight, int weight_is_f32, int dtype, int tokens,
+                             const void* q_weight, const void* k_weight, int weight_is_f32, int values_are_keys,
+                             const int* positions, double temp_every, float temp_coef, int dtype, int tokens,
                              int heads, int kv_heads, int dim, int vdim, int kernel_dim, int block_size, int num_pages,
                              hipStream_t stream);
 int mlr_matrix_memory_scan(const float* projected, int width, int q_off, int k_off, int v_off, int i_off, int f_off,
@@ -333,7 +337,8 @@ int mlr_gate_group_norm(const float* y, const float* projected, int width, int g
                         hipStream_t stream);
 
 // Routed experts (moe.hip).  mlr_moe_route: per token, from the router's float32 logits [tokens,
-// experts]: s = sigmoid(z) (score_kind 0) or softmax(z) over all experts (1), choice scores c = s + correction (float32 [experts], or null); the
+// experts]: s = sigmoid(z) (score_kind 0), softmax(z) over all experts (1), or z itself for the choice and the softmax over
+// the chosen z as weights (2), choice scores c = s + correction (float32 [experts], or null); the
 // expert axis is cut into `groups` contiguous blocks of experts / groups; block score = top-2 sum of
 // c; eligible are the experts of the `keep` highest blocks; ids [tokens, top] = arg-top-`top` of c over
 // the eligible (ties to the lower index), weights [tokens, top] = s[id] * scale, with `normalise` divided by the
@@ -353,12 +358,14 @@ int mlr_moe_align(const int* ids, int pairs, int experts, int big, int max_tiles
                   int* tiles, hipStream_t stream);
 // One grouped product over those tiles; w is [experts, n, k] in `dtype` (0 float32, 1 bfloat16).
 // up 1: a = h [tokens, k]; out [pairs, n] in `dtype`, row r = act(h[sorted[r] / top] w[e]^T), act 0
-// none, 2 squared ReLU, 3 sigmoid.  up 0: a = the rows of the first product [pairs, k]; out float32
+// none, 2 squared ReLU, 3 sigmoid, 5 the clamped gating of rows woven in pairs (n gate and up rows give n / 2
+// activations a row: out [pairs, n / 2]; n a multiple of 4; glu_limit, glu_alpha as for the products' epilogue).
+// up 0: a = the rows of the first product [pairs, k]; out float32
 // [top, tokens, n], out[choice, token] = pair_weights[p] * (a[r] w[e]^T).  mfma 1 and 2: on the matrix
 // cores (bfloat16, k % 8 == 0; 1 streams tiles of 16 rows, 2 runs tiles of 64 rows through LDS and
 // needs n % 8 == 0), 0: plain 32-bit FMA arithmetic (tiles of 16 rows).
 int mlr_moe_gemm(const void* a, const void* w, const int* sorted, const int* offsets, const int* tiles,
                  const float* pair_weights, void* out, int up, int dtype, int mfma, int max_tiles, int tokens, int top,
-                 int n, int k, int act, hipStream_t stream);
+                 int n, int k, int act, float glu_limit, float glu_alpha, hipStream_t stream);
 
 }  // extern "C"

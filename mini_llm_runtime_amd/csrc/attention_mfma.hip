@@ -177,6 +177,28 @@ __device__ __forceinline__ DecodeTile load_decode_tile(const bf16* __restrict__ 
   return t;
 }
 
+// The keys an entry's single query sees, as a line of places that tiles of 32 cut: first the positions kept from the
+// request's start, rounded up to whole tiles, then the positions from `base` (a multiple of 16 at or before the
+// first key of the window or chunk) to the query's own.  Without kept tokens place x is position base + x.
+struct DecodeLine {
+  int kept, kept_places, first, base;
+  struct Span {  // of one tile: its first position, and the positions first .. ke - 1 that are seen
+    int ts, first, ke;
+  };
+  __device__ __forceinline__ DecodeLine(int p, int window, int chunk, int keep) {
+    const VisibleKeys sees = visible_keys(p, window, chunk, keep);
+    kept = sees.kept;
+    kept_places = (sees.kept + 31) / 32 * 32;
+    first = sees.first;
+    base = (first / 16) * 16;
+  }
+  __device__ __forceinline__ int places(int ctx) const { return kept_places + ctx - base; }
+  __device__ __forceinline__ Span tile(int ts, int ke) const {
+    const int jump = base - kept_places;
+    return ts < kept_places ? Span{ts, 0, kept} : Span{ts + jump, first, ke + jump};
+  }
+};
+
 template <int kDecodeDepth>
 __global__ __launch_bounds__(kDecodeWaves* kWave) void attn_decode_kernel(
     const bf16* __restrict__ q, int64_t q_stride, const bf16* __restrict__ key_pages,
@@ -184,7 +206,7 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void attn_decode_kernel(
     const int* __restrict__ cu_q, const int* __restrict__ context_lens, bf16* __restrict__ out,
     float* __restrict__ partial, int heads, int kv_heads, int head_tiles, int block_size, int num_pages,
     float scale, int window, int chunk, int part, int splits, const float* __restrict__ sinks, int keep_partial,
-    const float* __restrict__ score_bias, float softcap) {
+    const float* __restrict__ score_bias, float softcap, int keep_first) {
   __shared__ float sm_acc[kDecodeWaves][16][D];
   __shared__ float sm_m[kDecodeWaves][16];
   __shared__ float sm_l[kDecodeWaves][16];
@@ -209,10 +231,11 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void attn_decode_kernel(
 
   const int ctx = context_lens[entry];
   const int p = ctx - 1;
-  const int first = first_visible_key(p, window, chunk);
-  const int base = (first / 16) * 16;
-  const int kb = base + split * part;
-  const int ke = min(kb + part, ctx);
+  // The partitions cut a line of places: the tokens kept from the request's start (in whole tiles of 32), then the
+  // tokens from `base` on.  Place ts of a tile is position ts - jump behind the kept ones, ts itself among them.
+  const DecodeLine line(p, window, chunk, keep_first);
+  const int kb = split * part;
+  const int ke = min(kb + part, line.places(ctx));
   if (kb >= ke) return;  // a partition past this entry's keys: the merge does not look at it
   const int* table = block_table + static_cast<int64_t>(entry) * table_width;
   if (tid == 0) sm_bad = 0;
@@ -244,17 +267,21 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void attn_decode_kernel(
   for (int ts0 = kb + wave * 32; ts0 < ke; ts0 += kDecodeDepth * kStride) {
     DecodeTilePages pages[kDecodeDepth];
 #pragma unroll
-    for (int j = 0; j < kDecodeDepth; ++j)
-      pages[j] = find_decode_tile(table, ts0 + j * kStride, ke, block_size, col, quarter);
+    for (int j = 0; j < kDecodeDepth; ++j) {
+      const DecodeLine::Span at = line.tile(ts0 + j * kStride, ke);
+      pages[j] = find_decode_tile(table, at.ts, at.ke, block_size, col, quarter);
+    }
     DecodeTile tile[kDecodeDepth];
 #pragma unroll
-    for (int j = 0; j < kDecodeDepth; ++j)
-      tile[j] = load_decode_tile(key_pages, value_pages, pages[j], ts0 + j * kStride, ke, first, kvh, kv_heads,
-                                 block_size, num_pages, col, quarter);
+    for (int j = 0; j < kDecodeDepth; ++j) {
+      const DecodeLine::Span at = line.tile(ts0 + j * kStride, ke);
+      tile[j] = load_decode_tile(key_pages, value_pages, pages[j], at.ts, at.ke, at.first, kvh, kv_heads, block_size,
+                                 num_pages, col, quarter);
+    }
 #pragma unroll
     for (int j = 0; j < kDecodeDepth; ++j) {
-      const int ts = ts0 + j * kStride;
-      if (ts >= ke) break;
+      if (ts0 + j * kStride >= ke) break;
+      const DecodeLine::Span at = line.tile(ts0 + j * kStride, ke);
       DecodeTile& cur = tile[j];
       bad = bad || cur.bad;
       f32x4_t sc[2];
@@ -265,8 +292,8 @@ __global__ __launch_bounds__(kDecodeWaves* kWave) void attn_decode_kernel(
         if (softcap > 0.f) cap_scores(sc[half], cap1, cap2);
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int key = ts + half * 16 + quarter * 4 + i;
-          if (!(key >= first && key < ke)) {
+          const int key = at.ts + half * 16 + quarter * 4 + i;
+          if (!(key >= at.first && key < at.ke)) {
             sc[half][i] = -INFINITY;
             // unwritten slots may hold NaN, and 0 * NaN would reach the output
             const uint32_t keep = (i & 1) ? 0x0000ffffu : 0xffff0000u;
@@ -377,7 +404,8 @@ __global__ __launch_bounds__(kWave) void attn_decode_merge_kernel(const float* _
                                                                   bf16* __restrict__ out, int heads, int window,
                                                                   int chunk, int part, int all_splits,
                                                                   const float* __restrict__ sinks,
-                                                                  const float* __restrict__ extra, int gated) {
+                                                                  const float* __restrict__ extra, int gated,
+                                                                  int keep_first) {
   const int entry = blockIdx.x;
   const int h = blockIdx.y;
   const int lane = threadIdx.x;
@@ -386,8 +414,7 @@ __global__ __launch_bounds__(kWave) void attn_decode_merge_kernel(const float* _
   const float* src = partial + (static_cast<int64_t>(entry) * heads + h) * all_splits * kPartialStride;
   // the partitions that hold keys of this entry (the others wrote nothing), as attn_decode cuts them
   const int ctx = context_lens[entry];
-  const int first = first_visible_key(ctx - 1, window, chunk);
-  const int splits = min(all_splits, (ctx - (first / 16) * 16 + part - 1) / part);
+  const int splits = min(all_splits, (DecodeLine(ctx - 1, window, chunk, keep_first).places(ctx) + part - 1) / part);
   // The numerators are read kMergeBatch partitions at a time, all loads of a batch issued
   // before the first is used, and the first batch before the reductions below: this kernel's
   // time is the latency of its loads, so they must not wait for one another.
@@ -516,7 +543,7 @@ __global__ __launch_bounds__(256 * kKeyGroups) void attn_prefill_kernel(
     const int* __restrict__ tiles, const int* __restrict__ cu_q, const int* __restrict__ context_lens,
     bf16* __restrict__ out, int num_tiles, int heads, int kv_heads, int bs_shift, int num_pages, float scale,
     int window, int chunk, float* __restrict__ partial, const float* __restrict__ sinks, int keep_partial,
-    const float* __restrict__ score_bias, float softcap) {
+    const float* __restrict__ score_bias, float softcap, int keep_first) {
   // gridDim.y > 1: the keys of every tile are cut into that many runs, one workgroup each, which
   // leave their unnormalised results in `partial` for attn_prefill_merge (few tiles behind a long
   // context would otherwise be as many long chains on a few compute units).
@@ -584,14 +611,21 @@ __global__ __launch_bounds__(256 * kKeyGroups) void attn_prefill_kernel(
   const int last_q = min(q0 + kWgQ, q_len) - 1;
   const int k_end = pos0 + last_q + 1;
   const int k_begin_raw = first_visible_key(pos0 + q0, window, chunk);
-  const int k_begin_all = (k_begin_raw / kTileK) * kTileK;
+  // The key tiles form a line: first those of the tokens kept from the request's start, then, `jump` positions on,
+  // those from the first query's window on (where the two meet they are one run: no jump).  Place x of the line
+  // is position x + (x < kept_places ? 0 : jump).
+  const int window_tile = (k_begin_raw / kTileK) * kTileK;
+  const int kept_places = min((keep_first + kTileK - 1) / kTileK * kTileK, window_tile);
+  const int jump = window_tile - kept_places;
+  auto position_of = [&](int place) { return place < kept_places ? place : place + jump; };
   // this workgroup's run of the keys: whole turns of the loop below (all key groups together)
   constexpr int kTurn = kKeyGroups * kTileK;
   const int splits = gridDim.y;
-  const int turns = (k_end - k_begin_all + kTurn - 1) / kTurn;
+  const int places = k_end - jump;
+  const int turns = (places + kTurn - 1) / kTurn;
   const int turns_each = (turns + splits - 1) / splits;
-  const int k_begin = k_begin_all + static_cast<int>(blockIdx.y) * turns_each * kTurn;
-  const int k_stop = min(k_end, k_begin + turns_each * kTurn);  // keys from here on belong to the next run
+  const int k_begin = static_cast<int>(blockIdx.y) * turns_each * kTurn;
+  const int k_stop = min(places, k_begin + turns_each * kTurn);  // places from here on belong to the next run
   // the wavefront's own range (uniform within the wavefront)
   const int w_last = pos0 + min(q0 + wave * kWaveQ + kWaveQ - 1, q_len - 1);
   const int w_first = first_visible_key(pos0 + q0 + wave * kWaveQ, window, chunk);
@@ -675,7 +709,7 @@ __global__ __launch_bounds__(256 * kKeyGroups) void attn_prefill_kernel(
     for (int i = 0; i < kPieces; ++i) {
       const int page = k_ids[i];
       const bool in = static_cast<unsigned>(page) < static_cast<unsigned>(num_pages);
-      if (!in) bad = bad || (k_row[i] < lim && kt0 + k_row[i] >= k_begin_raw);
+      if (!in) bad = bad || (k_row[i] < lim && (kt0 + k_row[i] >= k_begin_raw || kt0 + k_row[i] < keep_first));
       t.k[i] = load_bf16x8(key_pages + (static_cast<uint64_t>(in ? static_cast<uint32_t>(page) : 0u) * page_elems + k_in_page[i]));
     }
     const bool guard = lim < kTileK || window > 0 || (chunk > 0 && kt0 < k_begin_raw);  // uniform
@@ -715,31 +749,32 @@ __global__ __launch_bounds__(256 * kKeyGroups) void attn_prefill_kernel(
   constexpr int kStep = kKeyGroups * kTileK;  // keys per turn of the loop, all groups together
   const int k_mine = k_begin + group * kTileK;  // this group's first tile
   if (k_mine < k_stop) {
-    lookup(k_mine);
-    fetch(k_mine, flight);
-    lookup(k_mine + kStep);
+    lookup(position_of(k_mine));
+    fetch(position_of(k_mine), flight);
+    lookup(position_of(k_mine + kStep));
     stash(flight, 0);
   }
   __syncthreads();
   int buf = 0;
-  for (int kt0 = k_mine; kt0 - group * kTileK < k_stop; kt0 += kStep, buf ^= 1) {  // as many turns for every group
-    const bool mine = kt0 < k_stop;
-    const bool more = kt0 + kStep < k_stop;
+  for (int place = k_mine; place - group * kTileK < k_stop; place += kStep, buf ^= 1) {  // as many turns for every group
+    const bool mine = place < k_stop;
+    const bool more = place + kStep < k_stop;
+    const int kt0 = position_of(place);
     if (more) {
-      fetch(kt0 + kStep, flight);  // in flight while this tile is computed
-      lookup(kt0 + 2 * kStep);
+      fetch(position_of(place + kStep), flight);  // in flight while this tile is computed
+      lookup(position_of(place + 2 * kStep));
     }
     const bf16* ks = lds + (buf * kKeyGroups + group) * kBuffer;
     const bf16* vs = ks + kTileK * kKLd;
 
-    if (mine && wave_has_queries && kt0 <= w_last && kt0 + kTileK - 1 >= w_first) {
+    if (mine && wave_has_queries && kt0 <= w_last && (kt0 + kTileK - 1 >= w_first || kt0 < keep_first)) {
       // Scores of the whole tile, then ONE softmax update for its kTileK positions.  The
       // vector ALU, not the matrix core, bounds this loop (a wavefront instruction takes four
       // cycles, an exponential sixteen), so every per-score operation counts: the scale is
       // folded into the exponent's multiply-add, hidden scores are -inf and become 0 in the
       // exponential by themselves, and only tiles that cross a query's limits build masks.
       f32x4_t s[QB][kSubTiles];
-      const bool full = kt0 + kTileK - 1 <= w_min_pos && kt0 >= w_max_first;  // uniform in the wavefront
+      const bool full = kt0 + kTileK - 1 <= w_min_pos && (kt0 >= w_max_first || kt0 + kTileK <= keep_first);  // uniform in the wavefront
 #pragma unroll
       for (int sub = 0; sub < kSubTiles; ++sub) {
         const RowOperand keys = load_row(ks + (sub * 16 + col) * kKLd, true, quarter);
@@ -776,7 +811,7 @@ __global__ __launch_bounds__(256 * kKeyGroups) void attn_prefill_kernel(
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
               const int key = kt0 + (sub / 2) * 32 + quarter * 8 + (sub % 2) * 4 + i;  // see key_row_in_lds
-              if (!(q_ok[b] && key <= pq[b] && key >= pq_first[b])) s[b][sub][i] = -INFINITY;
+              if (!(q_ok[b] && key <= pq[b] && (key >= pq_first[b] || key < keep_first))) s[b][sub][i] = -INFINITY;
             }
       }
       uint32_t pw[QB][kSubTiles][2];
@@ -1005,6 +1040,7 @@ int64_t mlr_attention_decode_scratch(int entries, int heads, int splits) {
 // mlr_attention_decode_scratch floats, laid out [entry, head, split, head size + 2]
 // (numerator, maximum in base 2, denominator).  `merge` 0 leaves the partitions unmerged in
 // `partial` for a consumer that merges them itself (or for mlr_attention_decode_merge).
+// `keep_first`: with a window, how many of the request's first tokens every query sees beside it.
 // `extra` (or null): float32 [tokens, heads, head size + 2], for every token and head one more share of the same
 // softmax in the partitions' form (numerator, maximum of score * scale * log2(e), denominator; a maximum of
 // -infinity: nothing), made by another kernel over other keys; the merge takes it in before the sink.
@@ -1012,7 +1048,7 @@ int mlr_attention_decode(const void* q, int64_t q_stride, const void* key_pages,
                          const int* block_table, int table_width, const int* cu_q, const int* context_lens,
                          void* out, float* partial, int entries, int heads, int kv_heads, int block_size,
                          int num_pages, float scale, int window, int chunk, int part, int splits, int merge,
-                         const float* sinks, const float* extra, const float* score_bias, float softcap,
+                         const float* sinks, const float* extra, const float* score_bias, float softcap, int keep_first,
                          hipStream_t stream) {
   MLR_REQUIRE(q && key_pages && value_pages && block_table && cu_q && context_lens && out, "null pointer");
   MLR_REQUIRE(score_bias == nullptr || (sinks == nullptr && extra == nullptr && merge),
@@ -1033,6 +1069,7 @@ int mlr_attention_decode(const void* q, int64_t q_stride, const void* key_pages,
   MLR_REQUIRE(softcap >= 0.f && softcap < INFINITY && (softcap == 0.f || (score_bias == nullptr && extra == nullptr)),
               "capped scores go with a softmax over the tokens' own keys");
   const int keep_partial = extra != nullptr;
+  MLR_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "first tokens are kept beside a window");
   const int group = heads / kv_heads;
   const int head_tiles = (group + 15) / 16;
   MLR_REQUIRE(kv_heads * head_tiles <= 65535, "too many heads for one launch");
@@ -1046,7 +1083,7 @@ int mlr_attention_decode(const void* q, int64_t q_stride, const void* key_pages,
   attn_decode_kernel<depth><<<grid, kDecodeWaves * kWave, 0, stream>>>(                                         \
       qp, q_stride, kp, vp, block_table, table_width, cu_q, context_lens, op, partial, heads, kv_heads,         \
       head_tiles, block_size, num_pages, scale, window, chunk, part, splits, sinks, keep_partial, score_bias,   \
-      softcap)
+      softcap, keep_first)
   bool launched = false;
   if constexpr (kMaxDecodeDepth >= 4) {
     if (tiles_per_wave >= 4) {
@@ -1067,7 +1104,7 @@ int mlr_attention_decode(const void* q, int64_t q_stride, const void* key_pages,
   if ((splits > 1 || keep_partial) && merge) {
     attn_decode_merge_kernel<<<dim3(entries, heads), kWave, 0, stream>>>(
         partial, cu_q, context_lens, static_cast<bf16*>(out), heads, window, chunk, part, splits, sinks, extra,
-        score_bias != nullptr);
+        score_bias != nullptr, keep_first);
     MLR_LAUNCH_CHECK();
   }
   return 0;
@@ -1082,7 +1119,7 @@ int mlr_attention_decode_merge(const float* partial, const int* cu_q, const int*
   MLR_REQUIRE(entries > 0 && heads > 0 && heads <= 65535, "bad sizes");
   MLR_REQUIRE(part > 0 && part % 64 == 0 && splits > 1 && window >= 0 && chunk >= 0, "bad partitions");
   attn_decode_merge_kernel<<<dim3(entries, heads), kWave, 0, stream>>>(partial, cu_q, context_lens,
-                                                                      static_cast<bf16*>(out), heads, window, chunk, part, splits, sinks, nullptr, 0);
+                                                                      static_cast<bf16*>(out), heads, window, chunk, part, splits, sinks, nullptr, 0, 0);
   MLR_LAUNCH_CHECK();
   return 0;
 }
@@ -1109,12 +1146,13 @@ int mlr_attention_prefill(const void* q, int64_t q_stride, const void* key_pages
                           const int* cu_q, const int* context_lens, void* out, int heads, int kv_heads,
                           int block_size, int num_pages, float scale, int window, int chunk, int splits,
                           float* partial, const float* sinks, const float* extra, const float* score_bias,
-                          float softcap, hipStream_t stream) {
+                          float softcap, int keep_first, hipStream_t stream) {
   MLR_REQUIRE(splits >= 1 && splits <= 64, "splits must lie within 1..64");
   MLR_REQUIRE(score_bias == nullptr || (sinks == nullptr && extra == nullptr),
               "keys weighed one by one have no sink and no share made elsewhere");
   MLR_REQUIRE((splits == 1 && extra == nullptr) || partial != nullptr, "several key runs, or a share made elsewhere, need scratch memory");
   const int keep_partial = extra != nullptr;
+  MLR_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "first tokens are kept beside a window");
   MLR_REQUIRE(q && key_pages && value_pages && block_table && tiles && cu_q && context_lens && out, "null pointer");
   MLR_REQUIRE(num_tiles > 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "bad sizes");
   MLR_REQUIRE(kv_heads <= 65535, "too many key/value heads");  // a page's elements fit 32 bits
@@ -1159,13 +1197,13 @@ int mlr_attention_prefill(const void* q, int64_t q_stride, const void* key_pages
           static_cast<const bf16*>(q), q_stride, static_cast<const bf16*>(key_pages),                         \
           static_cast<const bf16*>(value_pages), block_table, table_width, tiles, cu_q, context_lens,         \
           static_cast<bf16*>(out), num_tiles, heads, kv_heads, bs_shift, num_pages, scale, window, chunk, partial,  \
-          (splits > 1 || keep_partial) ? nullptr : sinks, keep_partial, score_bias, softcap);  \
+          (splits > 1 || keep_partial) ? nullptr : sinks, keep_partial, score_bias, softcap, keep_first);  \
     else                                                                                                      \
       attn_prefill_kernel<qb, false><<<grid, 256 * kKeyGroups, kPrefillLds, stream>>>(                        \
           static_cast<const bf16*>(q), q_stride, static_cast<const bf16*>(key_pages),                         \
           static_cast<const bf16*>(value_pages), block_table, table_width, tiles, cu_q, context_lens,         \
           static_cast<bf16*>(out), num_tiles, heads, kv_heads, bs_shift, num_pages, scale, window, chunk, partial,  \
-          (splits > 1 || keep_partial) ? nullptr : sinks, keep_partial, score_bias, softcap);  \
+          (splits > 1 || keep_partial) ? nullptr : sinks, keep_partial, score_bias, softcap, keep_first);  \
   } while (0)
   if constexpr (D <= 128) {
     if (wide)

@@ -24,7 +24,7 @@ __global__ __launch_bounds__(64) void paged_attention_simple_kernel(
     int heads, int kv_heads, int head_dim, int block_size, int num_pages, float scale, int window, int chunk,
     const float* __restrict__ sinks, const T* __restrict__ pooled_keys, const T* __restrict__ pooled_values,
     const int* __restrict__ pooled_table, int pooled_width, int pooled_pages, int pool,
-    const float* __restrict__ score_bias, float softcap) {
+    const float* __restrict__ score_bias, float softcap, int keep_first) {
   __shared__ float qs[MAXD];
   __shared__ float ps[kWave];
   __shared__ int64_t offs[kWave];
@@ -46,7 +46,7 @@ __global__ __launch_bounds__(64) void paged_attention_simple_kernel(
   for (int i = lane; i < head_dim; i += kWave) qs[i] = to_f32(qrow[i]) * scale;
   __syncthreads();
 
-  const int first = first_visible_key(p, window, chunk);
+  const VisibleKeys sees = visible_keys(p, window, chunk, keep_first);
   // score_bias: no softmax at all.  A visible key weighs sigmoid(score + score_bias[head]) whatever the other
   // keys are, and nothing is normalised.
   const bool gated_keys = score_bias != nullptr;
@@ -58,18 +58,19 @@ __global__ __launch_bounds__(64) void paged_attention_simple_kernel(
   for (int j = 0; j < MAXD / kWave; ++j) acc[j] = 0.f;
   bool bad = false;
 
-  // Two sources share the one softmax: pooled entries (one key and value per run of `pool`
+  // Three sources share the one softmax: pooled entries (one key and value per run of `pool`
   // positions that lies wholly before the window: entry b covers b * pool .. b * pool + pool - 1 and is
-  // seen when its last position is <= p - window), then the tokens first..p themselves.
+  // seen when its last position is <= p - window), the request's first tokens where they are kept beside a window,
+  // then the tokens first..p themselves.
   const int pooled_seen = (pool > 0 && window > 0 && p - window >= 0) ? (p - window + 1) / pool : 0;
-  for (int source = 0; source < 2; ++source) {
+  for (int source = 0; source < 3; ++source) {
     const T* kpages = source == 0 ? pooled_keys : key_pages;
     const T* vpages = source == 0 ? pooled_values : value_pages;
     const int* table = (source == 0 ? pooled_table : block_table) + static_cast<int64_t>(entry) * (source == 0 ? pooled_width : table_width);
     const int tw = source == 0 ? pooled_width : table_width;
     const int np = source == 0 ? pooled_pages : num_pages;
-    const int begin = source == 0 ? 0 : first;
-    const int last = source == 0 ? pooled_seen - 1 : p;
+    const int begin = source == 2 ? sees.first : 0;
+    const int last = source == 0 ? pooled_seen - 1 : (source == 1 ? sees.kept - 1 : p);
     for (int k0 = begin; k0 <= last; k0 += kWave) {
       const int kpos = k0 + lane;
       float s = -INFINITY;
@@ -152,7 +153,7 @@ extern "C" int mlr_paged_attention_simple(const void* q, int64_t q_stride, const
                                           int block_size, int num_pages, float scale, int window, int chunk,
                                           const float* sinks, const void* pooled_keys, const void* pooled_values,
                                           const int* pooled_table, int pooled_width, int pooled_pages, int pool,
-                                          const float* score_bias, float softcap, hipStream_t stream) {
+                                          const float* score_bias, float softcap, int keep_first, hipStream_t stream) {
   MLR_REQUIRE(q && key_pages && value_pages && block_table && token_entry && positions && out, "null pointer");
   MLR_REQUIRE(tokens > 0 && entries > 0 && heads > 0 && kv_heads > 0, "sizes must be > 0");
   MLR_REQUIRE(heads % kv_heads == 0, "query heads must be a multiple of KV heads");
@@ -161,6 +162,7 @@ extern "C" int mlr_paged_attention_simple(const void* q, int64_t q_stride, const
   MLR_REQUIRE(q_stride >= static_cast<int64_t>(heads) * head_dim, "q_stride is smaller than a row of queries");
   MLR_REQUIRE(scale > 0.f && scale < INFINITY, "scale must be positive and finite");
   MLR_REQUIRE(window >= 0 && chunk >= 0 && !(window > 0 && chunk > 0), "a window or a chunked mask, each >= 0");
+  MLR_REQUIRE(keep_first >= 0 && (keep_first == 0 || window > 0), "first tokens are kept beside a window");
   MLR_REQUIRE(heads < 65536, "too many heads for one launch");
   MLR_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pooled_keys && pooled_values && pooled_table && pooled_width > 0 &&
                                           pooled_pages > 0)),
@@ -175,7 +177,8 @@ extern "C" int mlr_paged_attention_simple(const void* q, int64_t q_stride, const
       static_cast<const T*>(q), q_stride, static_cast<const T*>(key_pages), static_cast<const T*>(value_pages),   \
       block_table, table_width, token_entry, positions, static_cast<T*>(out), entries, heads, kv_heads, head_dim, \
       block_size, num_pages, scale, window, chunk, sinks, static_cast<const T*>(pooled_keys),                    \
-      static_cast<const T*>(pooled_values), pooled_table, pooled_width, pooled_pages, pool, score_bias, softcap)
+      static_cast<const T*>(pooled_values), pooled_table, pooled_width, pooled_pages, pool, score_bias, softcap,  \
+      keep_first)
   if (head_dim > 256) {
     if (dtype == kF32)
       MLR_SIMPLE(float, kMaxHeadDim);
@@ -190,14 +193,14 @@ extern "C" int mlr_paged_attention_simple(const void* q, int64_t q_stride, const
         static_cast<const float*>(value_pages), block_table, table_width, token_entry, positions,
         static_cast<float*>(out), entries, heads, kv_heads, head_dim, block_size, num_pages, scale, window, chunk,
         sinks, static_cast<const float*>(pooled_keys), static_cast<const float*>(pooled_values), pooled_table,
-        pooled_width, pooled_pages, pool, score_bias, softcap);
+        pooled_width, pooled_pages, pool, score_bias, softcap, keep_first);
   else
     paged_attention_simple_kernel<bf16, 256><<<grid, kWave, 0, stream>>>(
         static_cast<const bf16*>(q), q_stride, static_cast<const bf16*>(key_pages),
         static_cast<const bf16*>(value_pages), block_table, table_width, token_entry, positions,
         static_cast<bf16*>(out), entries, heads, kv_heads, head_dim, block_size, num_pages, scale, window, chunk,
         sinks, static_cast<const bf16*>(pooled_keys), static_cast<const bf16*>(pooled_values), pooled_table,
-        pooled_width, pooled_pages, pool, score_bias, softcap);
+        pooled_width, pooled_pages, pool, score_bias, softcap, keep_first);
   MLR_LAUNCH_CHECK();
   return 0;
 }

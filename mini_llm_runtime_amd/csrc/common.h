@@ -89,6 +89,22 @@ __host__ __device__ inline int first_visible_key(int p, int window, int chunk) {
   return window > 0 ? (p - window + 1 > 0 ? p - window + 1 : 0) : 0;
 }
 
+// With a window whose queries also see the first `keep` positions of their request, what a query at position p sees
+// is two ranges: 0 .. kept - 1 and first .. p, disjoint.  Where they meet they are one (kept = 0, first = 0).
+struct VisibleKeys {
+  int kept;
+  int first;
+};
+
+__host__ __device__ inline VisibleKeys visible_keys(int p, int window, int chunk, int keep) {
+  VisibleKeys v{0, first_visible_key(p, window, chunk)};
+  if (keep >= v.first)
+    v.first = keep > 0 ? 0 : v.first;
+  else
+    v.kept = keep;
+  return v;
+}
+
 __device__ inline float wave_sum(float v) {
   v += dpp_move<0x121>(v);  // row_ror:1
   v += dpp_move<0x122>(v);  // row_ror:2

@@ -13,36 +13,52 @@ typedef float f32x4v __attribute__((ext_vector_type(4)));
 
 // ---- x += weight * y * rsqrt(mean(y^2) + eps), then what reads the stream next -----------------
 // y is one tensor (float32 or the engine's dtype) or `slices` float32 partial sums added in slice
-// order.  mode 1: out = next_weight * x * rsqrt(mean(x^2) + next_eps); mode 2: out = x rounded to the
+// order.  TWO: a second y, normed by its own size with a weight of its own, is added to the first, each times a
+// constant.  mode 1: out = next_weight * x * rsqrt(mean(x^2) + next_eps); mode 2: out = x rounded to the
 // engine's dtype; mode 0: nothing more.  One workgroup per row; the row stays in LDS between the
 // passes, and a thread only ever reads the elements it wrote itself.
-template <typename T>
-__global__ __launch_bounds__(256) void add_normed_kernel(float* __restrict__ x, const void* __restrict__ y,
-                                                         int y_is_f32, int slices, int rows,
-                                                         const void* __restrict__ weight, int weight_is_f32, float eps,
-                                                         const void* __restrict__ next_weight, int next_is_f32,
-                                                         float next_eps, int mode, T* __restrict__ out, int hidden) {
-  extern __shared__ float row_lds[];
+struct NormedOutput {
+  const void* y;
+  int is_f32, slices;
+  const void* weight;
+  int weight_is_f32;
+  float scale;
+};
+
+template <typename T, bool TWO>
+__global__ __launch_bounds__(256) void add_normed_kernel(float* __restrict__ x, NormedOutput first, NormedOutput second,
+                                                         int rows, float eps, const void* __restrict__ next_weight,
+                                                         int next_is_f32, float next_eps, int mode, T* __restrict__ out,
+                                                         int hidden) {
+  extern __shared__ float row_lds[];  // [hidden], twice with TWO
   __shared__ float scratch[16];
   const int64_t row = blockIdx.x;
-  float ss = 0.f;
-  for (int i = threadIdx.x; i < hidden; i += 256) {
-    float v;
-    if (slices > 0) {
-      v = 0.f;
-      const float* p = static_cast<const float*>(y);
-      for (int s = 0; s < slices; ++s) v += p[(static_cast<int64_t>(s) * rows + row) * hidden + i];
-    } else {
-      v = y_is_f32 ? static_cast<const float*>(y)[row * hidden + i] : to_f32(static_cast<const T*>(y)[row * hidden + i]);
+  float inv[2] = {1.f, 1.f};
+#pragma unroll
+  for (int which = 0; which < (TWO ? 2 : 1); ++which) {
+    const NormedOutput& a = which == 0 ? first : second;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < hidden; i += 256) {
+      float v;
+      if (a.slices > 0) {
+        v = 0.f;
+        const float* p = static_cast<const float*>(a.y);
+        for (int s = 0; s < a.slices; ++s) v += p[(static_cast<int64_t>(s) * rows + row) * hidden + i];
+      } else {
+        v = a.is_f32 ? static_cast<const float*>(a.y)[row * hidden + i] : to_f32(static_cast<const T*>(a.y)[row * hidden + i]);
+      }
+      row_lds[which * hidden + i] = v;
+      ss += v * v;
     }
-    row_lds[i] = v;
-    ss += v * v;
+    inv[which] = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(hidden) + eps);
   }
-  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(hidden) + eps);
   float* xr = x + row * hidden;
   float ss2 = 0.f;
   for (int i = threadIdx.x; i < hidden; i += 256) {
-    const float v = xr[i] + (row_lds[i] * inv) * load_as_f32(weight, i, weight_is_f32);
+    float add = (row_lds[i] * inv[0]) * load_as_f32(first.weight, i, first.weight_is_f32);
+    if constexpr (TWO)
+      add = first.scale * add + second.scale * ((row_lds[hidden + i] * inv[1]) * load_as_f32(second.weight, i, second.weight_is_f32));
+    const float v = xr[i] + add;
     xr[i] = v;
     row_lds[i] = v;
     ss2 += v * v;
@@ -61,64 +77,77 @@ __global__ __launch_bounds__(256) void add_normed_kernel(float* __restrict__ x, 
 // The same for rows whose width is a multiple of 4 and fits the registers of a workgroup: a thread keeps
 // VPT groups of 4 elements between the passes, and all loads of a pass (every slice of partial sums
 // included) are issued before the first is used: the kernel's time is the latency of its loads.
-template <typename T, int VPT, int THREADS>
-__global__ __launch_bounds__(THREADS) void add_normed_rows_kernel(
-    float* __restrict__ x, const void* __restrict__ y, int y_is_f32, int slices, int rows,
-    const void* __restrict__ weight, int weight_is_f32, float eps, const void* __restrict__ next_weight,
-    int next_is_f32, float next_eps, int mode, T* __restrict__ out, int hidden) {
+template <typename T, int VPT, int THREADS, bool TWO>
+__global__ __launch_bounds__(THREADS) void add_normed_rows_kernel(float* __restrict__ x, NormedOutput first,
+                                                                  NormedOutput second, int rows, float eps,
+                                                                  const void* __restrict__ next_weight, int next_is_f32,
+                                                                  float next_eps, int mode, T* __restrict__ out,
+                                                                  int hidden) {
   __shared__ float scratch[16];
+  constexpr int kCount = TWO ? 2 : 1;
   const int64_t row = blockIdx.x;
   const int quads = hidden / 4;
   constexpr int kSliceBatch = 8;
-  f32x4v v[VPT], xv[VPT], wv[VPT], nv[VPT];
+  f32x4v v[kCount][VPT], xv[VPT], wv[kCount][VPT], nv[VPT];
 #pragma unroll
   for (int j = 0; j < VPT; ++j) {
     const int i = min(static_cast<int>(threadIdx.x) + j * THREADS, quads - 1);
     const int64_t at = row * hidden + 4 * i;
     xv[j] = *reinterpret_cast<const f32x4v*>(x + at);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      wv[j][e] = load_as_f32(weight, 4 * i + e, weight_is_f32);
-      nv[j][e] = mode == 1 ? load_as_f32(next_weight, 4 * i + e, next_is_f32) : 0.f;
-    }
-    if (slices > 0) {
-      v[j] = f32x4v{0.f, 0.f, 0.f, 0.f};
-    } else if (y_is_f32) {
-      v[j] = *reinterpret_cast<const f32x4v*>(static_cast<const float*>(y) + at);
-    } else {
+    for (int e = 0; e < 4; ++e) nv[j][e] = mode == 1 ? load_as_f32(next_weight, 4 * i + e, next_is_f32) : 0.f;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[j][e] = to_f32(static_cast<const T*>(y)[at + e]);
-    }
-  }
-  for (int s0 = 0; s0 < slices; s0 += kSliceBatch) {
-    f32x4v part[VPT][kSliceBatch];
+    for (int which = 0; which < kCount; ++which) {
+      const NormedOutput& a = which == 0 ? first : second;
 #pragma unroll
-    for (int j = 0; j < VPT; ++j) {
-      const int i = min(static_cast<int>(threadIdx.x) + j * THREADS, quads - 1);
+      for (int e = 0; e < 4; ++e) wv[which][j][e] = load_as_f32(a.weight, 4 * i + e, a.weight_is_f32);
+      if (a.slices > 0) {
+        v[which][j] = f32x4v{0.f, 0.f, 0.f, 0.f};
+      } else if (a.is_f32) {
+        v[which][j] = *reinterpret_cast<const f32x4v*>(static_cast<const float*>(a.y) + at);
+      } else {
 #pragma unroll
-      for (int u = 0; u < kSliceBatch; ++u) {
-        const int sl = min(s0 + u, slices - 1);
-        part[j][u] = *reinterpret_cast<const f32x4v*>(static_cast<const float*>(y) +
-                                                      (static_cast<int64_t>(sl) * rows + row) * hidden + 4 * i);
+        for (int e = 0; e < 4; ++e) v[which][j][e] = to_f32(static_cast<const T*>(a.y)[at + e]);
       }
     }
+  }
 #pragma unroll
-    for (int u = 0; u < kSliceBatch; ++u) {
-      const bool live = s0 + u < slices;
+  for (int which = 0; which < kCount; ++which) {
+    const NormedOutput& a = which == 0 ? first : second;
+    for (int s0 = 0; s0 < a.slices; s0 += kSliceBatch) {
+      f32x4v part[VPT][kSliceBatch];
 #pragma unroll
-      for (int j = 0; j < VPT; ++j)
+      for (int j = 0; j < VPT; ++j) {
+        const int i = min(static_cast<int>(threadIdx.x) + j * THREADS, quads - 1);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[j][e] = live ? v[j][e] + part[j][u][e] : v[j][e];
+        for (int u = 0; u < kSliceBatch; ++u) {
+          const int sl = min(s0 + u, a.slices - 1);
+          part[j][u] = *reinterpret_cast<const f32x4v*>(static_cast<const float*>(a.y) +
+                                                        (static_cast<int64_t>(sl) * rows + row) * hidden + 4 * i);
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < kSliceBatch; ++u) {
+        const bool live = s0 + u < a.slices;
+#pragma unroll
+        for (int j = 0; j < VPT; ++j)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[which][j][e] = live ? v[which][j][e] + part[j][u][e] : v[which][j][e];
+      }
     }
   }
-  float ss = 0.f;
+  float inv[kCount];
 #pragma unroll
-  for (int j = 0; j < VPT; ++j) {
-    if (static_cast<int>(threadIdx.x) + j * THREADS >= quads) v[j] = f32x4v{0.f, 0.f, 0.f, 0.f};
+  for (int which = 0; which < kCount; ++which) {
+    float ss = 0.f;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) ss += v[j][e] * v[j][e];
+    for (int j = 0; j < VPT; ++j) {
+      if (static_cast<int>(threadIdx.x) + j * THREADS >= quads) v[which][j] = f32x4v{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss += v[which][j][e] * v[which][j][e];
+    }
+    inv[which] = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(hidden) + eps);
   }
-  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(hidden) + eps);
   float ss2 = 0.f;
 #pragma unroll
   for (int j = 0; j < VPT; ++j) {
@@ -129,7 +158,9 @@ __global__ __launch_bounds__(THREADS) void add_normed_rows_kernel(
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      xv[j][e] += (v[j][e] * inv) * wv[j][e];
+      float add = (v[0][j][e] * inv[0]) * wv[0][j][e];
+      if constexpr (TWO) add = first.scale * add + second.scale * ((v[1][j][e] * inv[1]) * wv[1][j][e]);
+      xv[j][e] += add;
       ss2 += xv[j][e] * xv[j][e];
     }
     *reinterpret_cast<f32x4v*>(x + row * hidden + 4 * i) = xv[j];
@@ -147,19 +178,18 @@ __global__ __launch_bounds__(THREADS) void add_normed_rows_kernel(
   }
 }
 
-template <typename T>
-static void launch_add_normed(float* x, const void* y, int y_is_f32, int slices, const void* weight, int weight_is_f32,
-                              float eps, const void* next_weight, int next_is_f32, float next_eps, int mode, void* out,
-                              int rows, int hidden, hipStream_t stream) {
+template <typename T, bool TWO>
+static void launch_add_normed(float* x, const NormedOutput& first, const NormedOutput& second, float eps,
+                              const void* next_weight, int next_is_f32, float next_eps, int mode, void* out, int rows,
+                              int hidden, hipStream_t stream) {
   T* o = static_cast<T*>(out);
   const int quads = hidden / 4;
-#define MLR_ROWS(VPT, THREADS)                                                                                     \
-  add_normed_rows_kernel<T, VPT, THREADS><<<rows, THREADS, 0, stream>>>(x, y, y_is_f32, slices, rows, weight,     \
-                                                                        weight_is_f32, eps, next_weight, next_is_f32, \
-                                                                        next_eps, mode, o, hidden)
+#define MLR_ROWS(VPT, THREADS)                                                                                   \
+  add_normed_rows_kernel<T, VPT, THREADS, TWO><<<rows, THREADS, 0, stream>>>(x, first, second, rows, eps, next_weight, \
+                                                                             next_is_f32, next_eps, mode, o, hidden)
   if (hidden % 4 != 0 || quads > 2048)
-    add_normed_kernel<T><<<rows, 256, static_cast<size_t>(hidden) * sizeof(float), stream>>>(
-        x, y, y_is_f32, slices, rows, weight, weight_is_f32, eps, next_weight, next_is_f32, next_eps, mode, o, hidden);
+    add_normed_kernel<T, TWO><<<rows, 256, static_cast<size_t>(hidden) * sizeof(float) * (TWO ? 2 : 1), stream>>>(
+        x, first, second, rows, eps, next_weight, next_is_f32, next_eps, mode, o, hidden);
   else if (rows <= 64 && quads > 512)
     MLR_ROWS(2, 1024);
   else if (rows <= 64 && quads > 256)
@@ -793,20 +823,32 @@ using namespace mlr;
 extern "C" {
 
 int mlr_add_normed(float* x, const void* y, int y_is_f32, int slices, const void* weight, int weight_is_f32, float eps,
-                   const void* next_weight, int next_is_f32, float next_eps, int mode, void* out, int dtype, int rows,
-                   int hidden, hipStream_t stream) {
-  MLR_REQUIRE(x && y && weight, "null pointer");
-  MLR_REQUIRE(rows > 0 && hidden > 0 && hidden <= 16384, "rows must be > 0 and hidden within 1..16384");
-  MLR_REQUIRE(slices >= 0 && (slices == 0 || y_is_f32), "partial sums are float32");
+                   const void* y2, int y2_is_f32, int slices2, const void* weight2, int weight2_is_f32, float scale,
+                   float scale2, const void* next_weight, int next_is_f32, float next_eps, int mode, void* out, int dtype,
+                   int rows, int hidden, hipStream_t stream) {
+  MLR_REQUIRE(x && y && weight && (y2 == nullptr || weight2), "null pointer");
+  MLR_REQUIRE(rows > 0 && hidden > 0 && hidden <= (y2 ? 8192 : 16384), "rows must be > 0 and hidden within 1..16384 (8192 with two outputs)");
+  MLR_REQUIRE(slices >= 0 && (slices == 0 || y_is_f32) && slices2 >= 0 && (slices2 == 0 || y2_is_f32), "partial sums are float32");
   MLR_REQUIRE(mode >= 0 && mode <= 2 && (mode == 0 || out) && (mode != 1 || next_weight), "bad mode or missing output");
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
-  MLR_REQUIRE(dtype == kBF16 || y_is_f32, "a float32 engine has float32 activations");
-  if (dtype == kF32)
-    launch_add_normed<float>(x, y, y_is_f32, slices, weight, weight_is_f32, eps, next_weight, next_is_f32, next_eps, mode,
-                             out, rows, hidden, stream);
-  else
-    launch_add_normed<bf16>(x, y, y_is_f32, slices, weight, weight_is_f32, eps, next_weight, next_is_f32, next_eps, mode,
-                            out, rows, hidden, stream);
+  MLR_REQUIRE(dtype == kBF16 || (y_is_f32 && (y2 == nullptr || y2_is_f32)), "a float32 engine has float32 activations");
+  MLR_REQUIRE(y2 || scale == 1.f, "one output alone enters as it is");
+  const NormedOutput first{y, y_is_f32, slices, weight, weight_is_f32, scale};
+  const NormedOutput second{y2, y2_is_f32, slices2, weight2, weight2_is_f32, scale2};
+#define MLR_ADD_NORMED(T, TWO) \
+  launch_add_normed<T, TWO>(x, first, second, eps, next_weight, next_is_f32, next_eps, mode, out, rows, hidden, stream)
+  if (dtype == kF32) {
+    if (y2)
+      MLR_ADD_NORMED(float, true);
+    else
+      MLR_ADD_NORMED(float, false);
+  } else {
+    if (y2)
+      MLR_ADD_NORMED(bf16, true);
+    else
+      MLR_ADD_NORMED(bf16, false);
+  }
+#undef MLR_ADD_NORMED
   MLR_LAUNCH_CHECK();
   return 0;
 }

@@ -29,7 +29,8 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
   }
 }
 
-// One wavefront per token.  s = sigmoid(z) (score_kind 0) or softmax(z) over all experts (1), c = s + correction;
+// One wavefront per token.  s = sigmoid(z) (score_kind 0), softmax(z) over all experts (1) or z itself (2: the weights
+// are then the softmax over the chosen z, times the scale), c = s + correction;
 // with `normalise` the chosen weights are divided by their sum (+ 1e-20) before the scale.  Block g of experts / groups
 // consecutive experts scores top-2 sum of its c; c := -inf outside the `keep` highest blocks; then
 // `top` rounds of arg-max over c (ties to the lower index), each winner e leaving ids = e and
@@ -57,7 +58,7 @@ __global__ __launch_bounds__(kWave) void moe_route_kernel(const float* __restric
     z_inv = 1.0f / wave_sum(sum);
   }
   for (int e = lane; e < experts; e += kWave) {
-    const float sv = score_kind == 1 ? expf(z[e] - z_max) * z_inv : 1.0f / (1.0f + expf(-z[e]));
+    const float sv = score_kind == 2 ? z[e] : (score_kind == 1 ? expf(z[e] - z_max) * z_inv : 1.0f / (1.0f + expf(-z[e])));
     s[e] = sv;
     c[e] = sv + (correction != nullptr ? correction[e] : 0.f);
   }
@@ -97,6 +98,7 @@ __global__ __launch_bounds__(kWave) void moe_route_kernel(const float* __restric
     __syncthreads();
   }
   float chosen_sum = 0.f;
+  float z_top = 0.f;  // the first chosen logit: the largest
   for (int k = 0; k < top; ++k) {
     float v = -INFINITY;
     int i = 0x7fffffff;
@@ -109,10 +111,12 @@ __global__ __launch_bounds__(kWave) void moe_route_kernel(const float* __restric
     }
     wave_argmax(v, i);
     if (i >= experts) i = 0;  // only if every score left is NaN or -inf: keep the id in range
-    chosen_sum += s[i];
+    if (k == 0) z_top = s[i];
+    const float w = score_kind == 2 ? expf(s[i] - z_top) : s[i];
+    chosen_sum += w;
     if (lane == 0) {
       ids[static_cast<int64_t>(t) * top + k] = i;
-      weights[static_cast<int64_t>(t) * top + k] = s[i] * scale;
+      weights[static_cast<int64_t>(t) * top + k] = w * scale;
       c[i] = -INFINITY;
     }
     __syncthreads();
@@ -186,9 +190,26 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__
   }
 }
 
+// ---- the clamped gating in a grouped product's epilogue ------------------------------------------------
+// v: the sums of rows gate 2j, gate 2j + 1, up 2j, up 2j + 1 of an expert's first matrix, woven in pairs.  g * sigmoid(alpha
+// g) * (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit).  PRECISE: the float32 engine's exponential.
+template <bool PRECISE>
+__device__ __forceinline__ float clamped_gate(float gate, float up, float limit, float alpha) {
+  const float g = fminf(gate, limit);
+  const float u = fminf(fmaxf(up, -limit), limit);
+  const float e = PRECISE ? expf(-alpha * g) : __expf(-alpha * g);
+  return g / (1.0f + e) * (u + 1.0f);
+}
+
+__device__ __forceinline__ void store_clamped_glu(bf16* dst, const float (&v)[4], float limit, float alpha) {
+  *reinterpret_cast<uint32_t*>(dst) = pack_bf16x2(clamped_gate<false>(v[0], v[2], limit, alpha),
+                                                  clamped_gate<false>(v[1], v[3], limit, alpha));
+}
+
 // ---- grouped products, plain 32-bit FMA arithmetic -----------------------------------------------
 //
-// UP:   act[row, n]  = f(sum_k h[token(row), k] * w[e, n, k])                  (rows in sorted order)
+// UP:   act[row, n]  = f(sum_k h[token(row), k] * w[e, n, k])                  (rows in sorted order; with the
+//       clamped gating (act 5) N woven rows make N / 2 activations)
 // DOWN: out[choice(row), token(row), n] = weight[pair(row)] * sum_k act[row, k] * w[e, n, k]
 // A workgroup owns 16 rows of one tile and 64 features; K in slices of 16 through LDS.
 
@@ -203,7 +224,7 @@ __global__ __launch_bounds__(256) void moe_gemm_simple_kernel(const T* __restric
                                                               const int* __restrict__ tiles,
                                                               const float* __restrict__ pair_weights,
                                                               void* __restrict__ out, int tokens, int top, int N,
-                                                              int K, int act) {
+                                                              int K, int act, float glu_limit, float glu_alpha) {
   const int expert = tiles[2 * blockIdx.x];
   if (expert < 0) return;
   const int row0 = tiles[2 * blockIdx.x + 1];
@@ -248,6 +269,14 @@ __global__ __launch_bounds__(256) void moe_gemm_simple_kernel(const T* __restric
   if (pair < 0) return;
   const int token = pair / top;
   const int choice = pair - token * top;
+  if (UP && act == 5) {
+    const int gn = n0 + tn * 4;
+    if (gn >= N) return;  // N is a multiple of 4 here
+    T* dst = static_cast<T*>(out) + static_cast<int64_t>(row0 + tm) * (N / 2) + gn / 2;
+    dst[0] = from_f32<T>(clamped_gate<true>(acc[0], acc[2], glu_limit, glu_alpha));
+    dst[1] = from_f32<T>(clamped_gate<true>(acc[1], acc[3], glu_limit, glu_alpha));
+    return;
+  }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int gn = n0 + tn * 4 + j;
@@ -287,7 +316,7 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(const bf16* __restri
                                                             const int* __restrict__ tiles,
                                                             const float* __restrict__ pair_weights,
                                                             void* __restrict__ out, int tokens, int top, int N, int K,
-                                                            int act, int a_rows) {
+                                                            int act, int a_rows, float glu_limit, float glu_alpha) {
   const int expert = tiles[2 * blockIdx.x];
   if (expert < 0) return;
   const int row0 = tiles[2 * blockIdx.x + 1];
@@ -328,7 +357,10 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(const bf16* __restri
   const int token = in_pair / top;
   const int choice = in_pair - token * top;
   const int n = n_base + quad * 4;
-  if (UP) {
+  if (UP && act == 5) {
+    const float v[4] = {acc[0], acc[1], acc[2], acc[3]};
+    if (n < N) store_clamped_glu(static_cast<bf16*>(out) + static_cast<int64_t>(in_row) * (N / 2) + n / 2, v, glu_limit, glu_alpha);
+  } else if (UP) {
     bf16* dst = static_cast<bf16*>(out) + static_cast<int64_t>(in_row) * N + n;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -368,7 +400,7 @@ __global__ __launch_bounds__(256) void moe_gemm_stream_kernel(const bf16* __rest
                                                               const int* __restrict__ tiles,
                                                               const float* __restrict__ pair_weights,
                                                               void* __restrict__ out, int tokens, int top, int N, int K,
-                                                              int act, int a_rows) {
+                                                              int act, int a_rows, float glu_limit, float glu_alpha) {
   const int expert = tiles[2 * blockIdx.x];
   if (expert < 0) return;
   const int row0 = tiles[2 * blockIdx.x + 1];
@@ -449,7 +481,10 @@ __global__ __launch_bounds__(256) void moe_gemm_stream_kernel(const bf16* __rest
   const int token = pair / top;
   const int choice = pair - token * top;
   const int n = n0 + wave * 16 + quad * 4;
-  if (UP) {
+  if (UP && act == 5) {
+    const float v[4] = {acc[0], acc[1], acc[2], acc[3]};
+    if (n < N) store_clamped_glu(static_cast<bf16*>(out) + static_cast<int64_t>(row0 + col) * (N / 2) + n / 2, v, glu_limit, glu_alpha);
+  } else if (UP) {
     bf16* dst = static_cast<bf16*>(out) + static_cast<int64_t>(row0 + col) * N + n;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -490,7 +525,7 @@ __global__ __launch_bounds__(256) void moe_gemm_tiled_kernel(const bf16* __restr
                                                              const int* __restrict__ tiles,
                                                              const float* __restrict__ pair_weights,
                                                              void* __restrict__ out, int tokens, int top, int N, int K,
-                                                             int act, int a_rows) {
+                                                             int act, int a_rows, float glu_limit, float glu_alpha) {
   constexpr int kRows = big_rows(RB);
   const int expert = tiles[2 * blockIdx.x];
   if (expert < 0) return;
@@ -602,7 +637,9 @@ __global__ __launch_bounds__(256) void moe_gemm_tiled_kernel(const bf16* __restr
         float v[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) v[i] = acc[r][b][g * 4 + i];
-        if (UP) {
+        if (UP && act == 5) {
+          store_clamped_glu(static_cast<bf16*>(out) + static_cast<int64_t>(row0 + row) * (N / 2) + n / 2, v, glu_limit, glu_alpha);
+        } else if (UP) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             if (act == 2) {
@@ -626,7 +663,7 @@ __global__ __launch_bounds__(256) void moe_gemm_tiled_kernel(const bf16* __restr
 template <bool UP, int RB>
 static int launch_moe_tiled(const bf16* a, const bf16* w, const int* sorted, const int* offsets, const int* tiles,
                             const float* pair_weights, void* out, int max_tiles, int tokens, int top, int n, int k,
-                            int act, int a_rows, hipStream_t stream) {
+                            int act, int a_rows, float glu_limit, float glu_alpha, hipStream_t stream) {
   static bool configured = false;
   if (!configured) {
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(moe_gemm_tiled_kernel<UP, RB>),
@@ -639,7 +676,8 @@ static int launch_moe_tiled(const bf16* a, const bf16* w, const int* sorted, con
   }
   const dim3 grid(max_tiles, (n + kBigCols - 1) / kBigCols);
   moe_gemm_tiled_kernel<UP, RB><<<grid, 256, big_lds_bytes(RB), stream>>>(a, w, sorted, offsets, tiles, pair_weights, out,
-                                                                        tokens, top, n, k, act, a_rows);
+                                                                        tokens, top, n, k, act, a_rows, glu_limit,
+                                                                        glu_alpha);
   return 0;
 }
 
@@ -652,14 +690,15 @@ extern "C" {
 int mlr_moe_route(const float* logits, const float* correction, int* ids, float* weights, int tokens, int experts,
                   int top, int groups, int keep, float scale, int score_kind, int normalise, hipStream_t stream) {
   MLR_REQUIRE(logits && ids && weights, "null pointer");
-  MLR_REQUIRE(score_kind == 0 || score_kind == 1, "scores are sigmoids (0) or a softmax (1)");
+  MLR_REQUIRE(score_kind >= 0 && score_kind <= 2, "scores are sigmoids (0), a softmax (1) or the logits themselves (2)");
+  MLR_REQUIRE(score_kind != 2 || correction == nullptr, "a softmax over the chosen logits has no correction");
   MLR_REQUIRE(tokens > 0 && experts > 0 && top > 0 && top <= experts, "sizes must be > 0 and top <= experts");
   MLR_REQUIRE(groups > 0 && experts % groups == 0 && keep > 0 && keep <= groups, "bad groups");
   MLR_REQUIRE(top <= keep * (experts / groups), "the kept groups hold fewer experts than a token uses");
   MLR_REQUIRE(experts <= 4096, "at most 4096 experts");
   const size_t lds = (2 * static_cast<size_t>(experts) + groups) * sizeof(float);
   moe_route_kernel<<<tokens, kWave, lds, stream>>>(logits, correction, ids, weights, experts, top, groups, keep, scale,
-                                                   score_kind, normalise);
+                                                   score_kind, normalise || score_kind == 2);
   MLR_LAUNCH_CHECK();
   return 0;
 }
@@ -701,18 +740,19 @@ int mlr_moe_align(const int* ids, int pairs, int experts, int big, int max_tiles
 }
 
 // One of the two grouped products (`up` 1: act = f(h w_up^T) for the sorted rows, `act` 0 none, 2
-// squared ReLU, 3 sigmoid; `up` 0: out[choice, token] = weight * (act w_down^T), float32).  a and w
+// squared ReLU, 3 sigmoid, 5 the clamped gating over rows woven in pairs, whose rows of `act` are n / 2 wide; `up` 0: out[choice, token] = weight * (act w_down^T), float32).  a and w
 // in `dtype`; w is [experts, n, k].  `mfma` 1: the streaming matrix-core kernel (bfloat16, k % 8 == 0;
 // tiles of 16 rows), 2 and 3: the tiled one (tiles of 64 and of 128 rows, as mlr_moe_align made them
 // with `big` 1 and 2; n % 8 == 0 too); 0: plain arithmetic (tiles of 16 rows).
 int mlr_moe_gemm(const void* a, const void* w, const int* sorted, const int* offsets, const int* tiles,
                  const float* pair_weights, void* out, int up, int dtype, int mfma, int max_tiles, int tokens, int top,
-                 int n, int k, int act, hipStream_t stream) {
+                 int n, int k, int act, float glu_limit, float glu_alpha, hipStream_t stream) {
   MLR_REQUIRE(a && w && sorted && offsets && tiles && out, "null pointer");
   MLR_REQUIRE(up || pair_weights, "the down product needs the pairs' weights");
   MLR_REQUIRE(max_tiles > 0 && tokens > 0 && top > 0 && n > 0 && k > 0, "sizes must be > 0");
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
-  MLR_REQUIRE(act == 0 || act == 2 || act == 3, "unknown activation");
+  MLR_REQUIRE(act == 0 || act == 2 || act == 3 || act == 5, "unknown activation");
+  MLR_REQUIRE(act != 5 || (up && n % 4 == 0 && glu_limit > 0.f), "the clamped gating takes a first matrix of rows woven in pairs and a limit > 0");
   MLR_REQUIRE((n + kMoeCols - 1) / kMoeCols <= 65535, "too many features for one launch");
   const dim3 grid(max_tiles, (n + kMoeCols - 1) / kMoeCols);
   if (mfma) {
@@ -732,35 +772,36 @@ int mlr_moe_gemm(const void* a, const void* w, const int* sorted, const int* off
     if (mfma >= 2) {
       int status;
       if (mfma == 2)
-        status = up ? launch_moe_tiled<true, 1>(ab, wb, sorted, offsets, tiles, pair_weights, out, max_tiles, tokens, top, n, k, act, rows, stream)
-                    : launch_moe_tiled<false, 1>(ab, wb, sorted, offsets, tiles, pair_weights, out, max_tiles, tokens, top, n, k, act, rows, stream);
+        status = up ? launch_moe_tiled<true, 1>(ab, wb, sorted, offsets, tiles, pair_weights, out, max_tiles, tokens, top, n, k, act, rows, glu_limit, glu_alpha, stream)
+                    : launch_moe_tiled<false, 1>(ab, wb, sorted, offsets, tiles, pair_weights, out, max_tiles, tokens, top, n, k, act, rows, glu_limit, glu_alpha, stream);
       else
-        status = up ? launch_moe_tiled<true, 2>(ab, wb, sorted, offsets, tiles, pair_weights, out, max_tiles, tokens, top, n, k, act, rows, stream)
-                    : launch_moe_tiled<false, 2>(ab, wb, sorted, offsets, tiles, pair_weights, out, max_tiles, tokens, top, n, k, act, rows, stream);
+        status = up ? launch_moe_tiled<true, 2>(ab, wb, sorted, offsets, tiles, pair_weights, out, max_tiles, tokens, top, n, k, act, rows, glu_limit, glu_alpha, stream)
+                    : launch_moe_tiled<false, 2>(ab, wb, sorted, offsets, tiles, pair_weights, out, max_tiles, tokens, top, n, k, act, rows, glu_limit, glu_alpha, stream);
       if (status != 0) return -1;
     } else if (static_cast<int64_t>(n) * k * 2 >= (1ll << 20)) {
       // an expert's matrix of a megabyte or more: whole lines through LDS
       const dim3 stream_grid(max_tiles, (n + kStCols - 1) / kStCols);
       if (up)
-        moe_gemm_stream_kernel<true><<<stream_grid, 256, 0, stream>>>(ab, wb, sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, rows);
+        moe_gemm_stream_kernel<true><<<stream_grid, 256, 0, stream>>>(ab, wb, sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, rows, glu_limit, glu_alpha);
       else
-        moe_gemm_stream_kernel<false><<<stream_grid, 256, 0, stream>>>(ab, wb, sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, rows);
+        moe_gemm_stream_kernel<false><<<stream_grid, 256, 0, stream>>>(ab, wb, sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, rows, glu_limit, glu_alpha);
     } else {
       // four wavefronts (64 features) a workgroup, or two where that leaves the compute units with too
       // few workgroups to keep their loads in flight
       const int waves = static_cast<int64_t>(max_tiles) * ((n + 63) / 64) < 2048 ? 2 : 4;
       const dim3 small_grid(max_tiles, (n + waves * 16 - 1) / (waves * 16));
       if (up)
-        moe_gemm_mfma_kernel<true><<<small_grid, waves * kWave, 0, stream>>>(ab, wb, sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, rows);
+        moe_gemm_mfma_kernel<true><<<small_grid, waves * kWave, 0, stream>>>(ab, wb, sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, rows, glu_limit, glu_alpha);
       else
-        moe_gemm_mfma_kernel<false><<<small_grid, waves * kWave, 0, stream>>>(ab, wb, sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, rows);
+        moe_gemm_mfma_kernel<false><<<small_grid, waves * kWave, 0, stream>>>(ab, wb, sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, rows, glu_limit, glu_alpha);
     }
     MLR_LAUNCH_CHECK();
     return 0;
   }
 #define MLR_MOE_SIMPLE(T, UP)                                                                                  \
   moe_gemm_simple_kernel<T, UP><<<grid, 256, 0, stream>>>(static_cast<const T*>(a), static_cast<const T*>(w), \
-                                                          sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act)
+                                                          sorted, offsets, tiles, pair_weights, out, tokens, top, n, k, act, \
+                                                          glu_limit, glu_alpha)
   if (dtype == kF32) {
     if (up)
       MLR_MOE_SIMPLE(float, true);

@@ -200,14 +200,16 @@ __global__ __launch_bounds__(256) void streams_fill_kernel(const float* __restri
 // negative slot stores nothing.
 // q_weight given (and k_weight [dim], with keys): a head is divided by its root mean square and multiplied by that
 // weight BEFORE it turns, and the values are stored as they are.  kv_heads 0: the rows hold queries only.
+// values_are_keys (weighted norms, vdim = dim): the rows hold no values, the keys' sums before their norm are stored as
+// values too.  positions given: queries are multiplied by 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1).
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
     const float* __restrict__ p, int width, T* __restrict__ q_out, float* __restrict__ gate,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rdims, float eps,
     const int* __restrict__ slots, T* __restrict__ key_pages, T* __restrict__ value_pages, float* __restrict__ v_keep,
     const float* __restrict__ v_first, const float* __restrict__ lambda_p, const void* __restrict__ q_weight,
-    const void* __restrict__ k_weight, int weight_is_f32, int heads, int kv_heads, int dim, int vdim, int D, int block_size,
-    int num_pages) {
+    const void* __restrict__ k_weight, int weight_is_f32, int values_are_keys, const int* __restrict__ positions,
+    double temp_every, float temp_coef, int heads, int kv_heads, int dim, int vdim, int D, int block_size, int num_pages) {
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x % kWave;
   const int wave = threadIdx.x / kWave;
@@ -226,7 +228,8 @@ __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
     const bool is_k = !is_q && job < heads + kv_heads;
     const int h = is_q ? job : (is_k ? job - heads : job - heads - kv_heads);
     const int n = (is_q || is_k) ? dim : vdim;
-    const float* src = row + (is_q ? h * dim : (is_k ? heads * dim + h * dim : (heads + kv_heads) * dim + h * vdim));
+    const float* src =
+        row + (is_q ? h * dim : (is_k || values_are_keys ? heads * dim + h * dim : (heads + kv_heads) * dim + h * vdim));
     if (q_weight != nullptr) {
       float inv = 1.0f;
       if (is_q || is_k) {
@@ -243,7 +246,10 @@ __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
       };
       if (is_q) {
         T* dst = q_out + (t * heads + h) * D;
-        for (int j = lane; j < D; j += kWave) dst[j] = from_f32<T>(j < n ? turned(j) : 0.f);
+        float grown = 1.0f;  // 1 + coef * ln(floor((position + 1) / every) + 1)
+        if (positions != nullptr)
+          grown += temp_coef * logf(static_cast<float>(floor((static_cast<double>(positions[t]) + 1.0) / temp_every)) + 1.0f);
+        for (int j = lane; j < D; j += kWave) dst[j] = from_f32<T>(j < n ? turned(j) * grown : 0.f);
       } else if (store && is_k) {
         T* dst = key_pages + ((static_cast<int64_t>(page) * kv_heads + h) * block_size + off) * D;
         for (int j = lane; j < D; j += kWave) dst[j] = from_f32<T>(j < n ? turned(j) : 0.f);
@@ -603,8 +609,9 @@ int mlr_streams_step(float* x, int streams, int tokens, int width, const int* ro
 int mlr_head_norm_rope_write(const float* projected, int width, void* q_out, float* gate, const float* cos,
                              const float* sin, int rotary_dims, float eps, const int* slots, void* key_pages,
                              void* value_pages, float* v_keep, const float* v_first, const float* lambda, const void* q_weight,
-                             const void* k_weight, int weight_is_f32, int dtype, int tokens, int heads, int kv_heads, int dim, int vdim, int kernel_dim, int block_size,
-                             int num_pages, hipStream_t stream) {
+                             const void* k_weight, int weight_is_f32, int values_are_keys, const int* positions,
+                             double temp_every, float temp_coef, int dtype, int tokens, int heads, int kv_heads, int dim,
+                             int vdim, int kernel_dim, int block_size, int num_pages, hipStream_t stream) {
   MLR_REQUIRE(projected && q_out && (kv_heads == 0 || (slots && key_pages && value_pages)), "null pointer");
   MLR_REQUIRE(tokens > 0 && heads > 0 && kv_heads >= 0 && dim > 0 && vdim > 0, "sizes must be > 0");
   MLR_REQUIRE(q_weight == nullptr || ((kv_heads == 0 || k_weight) && !v_keep && !v_first),
@@ -612,7 +619,9 @@ int mlr_head_norm_rope_write(const float* projected, int width, void* q_out, flo
   MLR_REQUIRE(kernel_dim >= dim && kernel_dim >= vdim, "the kernels' head size must hold keys and values");
   MLR_REQUIRE(rotary_dims >= 0 && rotary_dims % 2 == 0 && rotary_dims <= dim, "rotary_dims must be even and within dim");
   MLR_REQUIRE(rotary_dims == 0 || (cos && sin), "a rotation needs cos and sin tables");
-  MLR_REQUIRE(width >= (heads + kv_heads) * dim + kv_heads * vdim + (gate ? heads : 0), "the projected rows are too narrow");
+  MLR_REQUIRE(!values_are_keys || (q_weight && kv_heads > 0 && vdim == dim && !gate), "keys that are values have one size and weighted norms, and no gate behind them");
+  MLR_REQUIRE(positions == nullptr || (q_weight && temp_every > 0.0), "queries that grow have weighted norms and a length > 0 per step");
+  MLR_REQUIRE(width >= (heads + kv_heads) * dim + (values_are_keys ? 0 : kv_heads * vdim) + (gate ? heads : 0), "the projected rows are too narrow");
   MLR_REQUIRE(v_first == nullptr || lambda, "mixing values in needs its weight");
   MLR_REQUIRE(kv_heads == 0 || (block_size > 0 && num_pages > 0), "page sizes must be > 0");
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
@@ -623,12 +632,14 @@ int mlr_head_norm_rope_write(const float* projected, int width, void* q_out, flo
     head_norm_rope_write_kernel<float><<<grid, 256, 0, stream>>>(
         projected, width, static_cast<float*>(q_out), gate, cos, sin, rotary_dims, eps, slots,
         static_cast<float*>(key_pages), static_cast<float*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight,
-        weight_is_f32, heads, kv_heads, dim, vdim, kernel_dim, block_size, num_pages);
+        weight_is_f32, values_are_keys, positions, temp_every, temp_coef, heads, kv_heads, dim, vdim, kernel_dim, block_size,
+        num_pages);
   else
     head_norm_rope_write_kernel<bf16><<<grid, 256, 0, stream>>>(
         projected, width, static_cast<bf16*>(q_out), gate, cos, sin, rotary_dims, eps, slots,
         static_cast<bf16*>(key_pages), static_cast<bf16*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight,
-        weight_is_f32, heads, kv_heads, dim, vdim, kernel_dim, block_size, num_pages);
+        weight_is_f32, values_are_keys, positions, temp_every, temp_coef, heads, kv_heads, dim, vdim, kernel_dim, block_size,
+        num_pages);
   MLR_LAUNCH_CHECK();
   return 0;
 }

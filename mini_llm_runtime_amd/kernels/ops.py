@@ -25,11 +25,14 @@ _VP = ctypes.c_void_p
 _I = ctypes.c_int
 _I64 = ctypes.c_int64
 _F = ctypes.c_float
+_D = ctypes.c_double
 
 _SIGNATURES = {
     "mlr_version": ([], _I),
     "mlr_embedding": ([_VP, _I, _VP, _VP, _I, _I, _I, _I, _VP], _I),
-    "mlr_add_normed": ([_VP, _VP, _I, _I, _VP, _I, _F, _VP, _I, _F, _I, _VP, _I, _I, _I, _VP], _I),
+    "mlr_add_normed": (
+        [_VP, _VP, _I, _I, _VP, _I, _F, _VP, _I, _I, _VP, _I, _F, _F, _VP, _I, _F, _I, _VP, _I, _I, _I, _VP], _I,
+    ),
     "mlr_round": ([_VP, _VP, _I64, _VP], _I),
     "mlr_glu_gelu": ([_VP, _VP, _I, _I, _I, _VP], _I),
     "mlr_conv_gates": (
@@ -56,8 +59,8 @@ _SIGNATURES = {
     "mlr_streams_fill": ([_VP, _VP, _I, _I, _I, _VP], _I),
     "mlr_streams_step": ([_VP, _I, _I, _I, _VP, _I, _VP, _I, _I, _VP, _VP, _VP, _VP, _I, _F, _VP, _VP, _I, _VP], _I),
     "mlr_head_norm_rope_write": (
-        [_VP, _I, _VP, _VP, _VP, _VP, _I, _F, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I,
-         _VP],
+        [_VP, _I, _VP, _VP, _VP, _VP, _I, _F, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _VP, _D, _F, _I, _I, _I, _I, _I,
+         _I, _I, _I, _I, _VP],
         _I,
     ),
     "mlr_matrix_memory_scan": (
@@ -98,7 +101,7 @@ _SIGNATURES = {
     "mlr_moe_tile_rows": ([_I], _I),
     "mlr_moe_max_tiles": ([_I, _I, _I], _I),
     "mlr_moe_align": ([_VP, _I, _I, _I, _I, _VP, _VP, _VP, _VP], _I),
-    "mlr_moe_gemm": ([_VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _I, _VP], _I),
+    "mlr_moe_gemm": ([_VP, _VP, _VP, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _VP], _I),
     "mlr_gemm_residual_parts": ([_I, _I], _I),
     "mlr_gemm_residual_bf16": ([_VP, _VP, _VP, _I, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _VP], _I),
     "mlr_gemm_bf16_slices": ([_I, _I, _I, _I], _I),
@@ -118,7 +121,7 @@ _SIGNATURES = {
     "mlr_gemm_merge_fused_bf16": ([_VP, _VP, _I, _I, _I, _I, _I, _VP, _VP, _I, _VP, _I, _I, _I, _I, _VP], _I),
     "mlr_paged_attention_simple": (
         [_VP, _I64, _VP, _VP, _VP, _I, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _VP, _VP, _VP, _VP,
-         _I, _I, _I, _VP, _F, _VP],
+         _I, _I, _I, _VP, _F, _I, _VP],
         _I,
     ),
     "mlr_sample": ([_VP, _VP, _VP, _VP, _VP, _I, _I, _VP], _I),
@@ -129,14 +132,14 @@ _SIGNATURES = {
     "mlr_attention_decode_scratch": ([_I, _I, _I], _I64),
     "mlr_attention_decode": (
         [_VP, _I64, _VP, _VP, _VP, _I, _VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _I, _VP, _VP, _VP, _F,
-         _VP],
+         _I, _VP],
         _I,
     ),
     "mlr_attention_decode_merge": ([_VP, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _VP, _VP], _I),
     "mlr_attention_prefill_scratch": ([_I, _I, _I, _I], _I64),
     "mlr_attention_prefill": (
         [_VP, _I64, _VP, _VP, _VP, _I, _VP, _I, _I, _VP, _VP, _VP, _I, _I, _I, _I, _F, _I, _I, _I, _VP, _VP, _VP, _VP, _F,
-         _VP],
+         _I, _VP],
         _I,
     ),
 }
@@ -296,7 +299,7 @@ class HipOps:
         in the engine's dtype.  delta: [rows, hidden] in the engine's dtype, or a float32 stack
         [S, rows, hidden] of partial sums (see `linear`), or None."""
         if isinstance(delta, NormedDelta):  # one kernel: the normed addition and this norm
-            return self.add_normed(x, delta.y, delta.weight, delta.eps, next_weight=weight, next_eps=eps)
+            return self.add_normed(x, delta.y, delta.weight, delta.eps, next_weight=weight, next_eps=eps, **delta.options())
         self._check(x, "residual stream", torch.float32, (None, None))
         rows, hidden = x.shape
         self._check(weight, "norm weight", (torch.float32, self.dtype), (hidden,))
@@ -324,22 +327,28 @@ class HipOps:
         next_weight: Optional[torch.Tensor] = None,
         next_eps: float = 0.0,
         cast: bool = False,
+        second: Optional[tuple] = None,
+        scales: tuple[float, float] = (1.0, 1.0),
     ) -> Optional[torch.Tensor]:
         """x (float32 residual stream [rows, hidden], in place) += weight * y * rsqrt(mean(y^2) + eps): a part's
         output that enters the stream through a norm of its own.  y: [rows, hidden] in the engine's dtype or
         float32, a float32 stack [S, rows, hidden] whose sum it is, or a product that has not run.  The same
         kernel then makes what reads the stream next: with `next_weight` the RMSNorm of the new x (weight,
-        `next_eps`), with `cast` x itself, both in the engine's dtype; else nothing is returned."""
+        `next_eps`), with `cast` x itself, both in the engine's dtype; else nothing is returned.
+        second: (y, weight) of another output, normed by its own size: what x receives then is scales[0] * the first +
+        scales[1] * the second."""
         self._check(x, "residual stream", torch.float32, (None, None))
         rows, hidden = x.shape
-        y = self.settle(y)
-        slices = 0
-        if y.dim() == 3:
-            self._check(y, "partial sums", torch.float32, (None, rows, hidden))
-            slices = y.shape[0]
-        else:
-            self._check(y, "sublayer output", (torch.float32, self.dtype), (rows, hidden))
+        y, slices = self._output_sums(y, rows, hidden)
         self._check(weight, "norm weight", (torch.float32, self.dtype), (hidden,))
+        other = other_weight = None
+        other_slices = 0
+        if second is not None:
+            other, other_weight = second
+            other, other_slices = self._output_sums(other, rows, hidden)
+            self._check(other_weight, "second norm weight", (torch.float32, self.dtype), (hidden,))
+        elif scales[0] != 1.0:
+            weight, scales = weight.to(torch.float32) * float(scales[0]), (1.0, 1.0)
         mode = 0
         out = None
         if next_weight is not None:
@@ -351,11 +360,23 @@ class HipOps:
             out = self._empty((rows, hidden), self.dtype)
         self._call(
             "mlr_add_normed", self._ptr(x), self._ptr(y), int(y.dtype == torch.float32), slices, self._ptr(weight),
-            int(weight.dtype == torch.float32), float(eps), self._ptr(next_weight),
+            int(weight.dtype == torch.float32), float(eps), self._ptr(other),
+            int(other is not None and other.dtype == torch.float32), other_slices, self._ptr(other_weight),
+            int(other_weight is not None and other_weight.dtype == torch.float32), float(scales[0]), float(scales[1]),
+            self._ptr(next_weight),
             int(next_weight is not None and next_weight.dtype == torch.float32), float(next_eps), mode, self._ptr(out),
             self.code, rows, hidden, self._stream(),
         )
         return out
+
+    def _output_sums(self, y, rows: int, hidden: int):
+        """(tensor, number of partial sums; 0: it is whole) of a part's output."""
+        y = self.settle(y)
+        if y.dim() == 3:
+            self._check(y, "partial sums", torch.float32, (None, rows, hidden))
+            return y, y.shape[0]
+        self._check(y, "sublayer output", (torch.float32, self.dtype), (rows, hidden))
+        return y, 0
 
     def add_(self, x: torch.Tensor, delta: torch.Tensor) -> None:
         """x (float32) += delta (the engine's dtype, or float32; or a float32 stack [S, ...] of partial sums, or a
@@ -383,7 +404,7 @@ class HipOps:
         if isinstance(x, PendingLinear):
             return PendingLinear(self.gather_rows(self.settle(x.x), rows), x.weight, x.bias)
         if isinstance(x, NormedDelta):  # the norm is per row: it commutes with the choice of rows
-            return NormedDelta(self.gather_rows(x.y, rows), x.weight, x.eps)
+            return x.with_outputs(lambda y: self.gather_rows(y, rows))
         x = self.settle(x)
         self._check(x, "rows source", (torch.float32, torch.bfloat16))
         if x.dim() not in (2, 3):
@@ -441,7 +462,7 @@ class HipOps:
         if isinstance(h, NormedDelta):  # what it adds to the stream, float32
             y = self.settle(h.y)
             added = torch.zeros(y.shape[-2:], dtype=torch.float32, device=self.device)
-            self.add_normed(added, y, h.weight, h.eps)
+            self.add_normed(added, y, h.weight, h.eps, **h.options())
             return added
         if isinstance(h, PendingMerge):
             out = self._empty((h.tokens, h.heads * h.head_dim), self.dtype)
@@ -531,6 +552,7 @@ class HipOps:
         clamped_glu: Optional[tuple[float, float]] = None,
         multiply_rows: Optional[torch.Tensor] = None,
         geglu: bool = False,
+        out: Optional[torch.Tensor] = None,
     ) -> torch.Tensor:
         """x [M, K] times weight [N, K] transposed, plus bias [N]; F.linear semantics.
 
@@ -559,6 +581,7 @@ class HipOps:
         accepts, instead of [M, N], a float32 stack [S, M, N] of partial sums over slices
         of k (bias in slice 0).  Narrow products of a few tokens are cut that way so that
         all compute units stream the weight; the norm kernel adds the slices in order.
+        out: a tensor of the result's shape and dtype to write it into (a stack [S, M, N] with `slices` = S > 1).
         mfma_kernel, slices: force one of the matrix-core kernels (16, 14, 11, 22, 23, 44 to 48, 62 to 68) and a number
         of k slices instead of letting the shape choose; for tests and tuning.
         """
@@ -597,7 +620,7 @@ class HipOps:
                 return PendingLinear(x, weight, bias)
         if isinstance(x, (PendingNorm, PendingMerge)):
             fused = None
-            if multiply is None:
+            if multiply is None and out is None:
                 fused = self._linear_fused(x, weight, bias, out_dtype, kernel, epilogue, partial_sums, mfma_kernel, slices)
             if fused is not None:
                 return fused
@@ -635,10 +658,10 @@ class HipOps:
             elif slices < 1 or (slices > 1 and not (partial_sums and not swiglu)):
                 raise KernelError("k slices need partial_sums and no SwiGLU")
             if slices > 1:
-                y = self._empty((slices, m, n), torch.float32)
+                y = self._into(out, (slices, m, n), torch.float32)
                 out_f32 = 1
             else:
-                y = self._empty((m, n // 2 if swiglu else n), out_dtype)
+                y = self._into(out, (m, n // 2 if swiglu else n), out_dtype)
                 out_f32 = int(out_dtype == torch.float32)
             self._call(
                 "mlr_gemm_bf16", self._ptr(x), self._ptr(weight), self._ptr(bias), bias_f32, self._ptr(y), out_f32,
@@ -646,13 +669,16 @@ class HipOps:
                 glu_limit, glu_alpha, self._stream(),
             )
             return y
-        y = self._empty((m, n // 2 if swiglu else n), out_dtype)
+        y = self._into(out, (m, n // 2 if swiglu else n), out_dtype)
         self._call(
             "mlr_gemm_simple", self._ptr(x), self._ptr(weight), self._ptr(bias), bias_f32, self._ptr(y),
             int(out_dtype == torch.float32), epilogue, self.code, m, n, k, self._ptr(multiply),
             self._ptr(multiply_rows), glu_limit, glu_alpha, self._stream(),
         )
         return y
+
+    def _into(self, out: Optional[torch.Tensor], shape: Sequence[int], dtype: torch.dtype) -> torch.Tensor:
+        return self._empty(shape, dtype) if out is None else self._check(out, "linear output", dtype, shape)
 
     def _linear_fused(self, x, weight, bias, out_dtype, kernel, epilogue, partial_sums, mfma_kernel, slices):
         """`linear` on a pending activation in one kernel, or None when that cannot be.  `epilogue`:
@@ -960,8 +986,11 @@ class HipOps:
         pooled: Optional[tuple] = None,
         score_bias: Optional[torch.Tensor] = None,
         softcap: Optional[float] = None,
+        keep_first: int = 0,
     ):
         """Causal attention of the step's tokens over their requests' pages.
+
+        keep_first: with a window, every query also sees the first `keep_first` positions of its request.
 
         softcap: the scaled score s becomes softcap * tanh(s / softcap) before the softmax.
 
@@ -1023,6 +1052,9 @@ class HipOps:
                 raise KernelError("a soft cap must be > 0")
             if score_bias is not None or pooled is not None:
                 raise KernelError("capped scores go with a softmax over the tokens' own keys")
+        keep_first = int(keep_first)
+        if keep_first < 0 or (keep_first and (not window or pooled is not None)):
+            raise KernelError("first tokens are kept beside a window without pooled entries")
         out = self._empty((tokens, num_heads * head_dim), self.dtype)
         width = block_table.shape[1]
         pooled_keys = pooled_values = pooled_table = None
@@ -1061,7 +1093,7 @@ class HipOps:
                 self._ptr(out), self.code, tokens, entries, num_heads, num_kv_heads, head_dim, block_size,
                 num_pages, float(scale), int(window or 0), chunk, self._ptr(sinks), self._ptr(pooled_keys),
                 self._ptr(pooled_values), self._ptr(pooled_table), pooled_width, pooled_pages, pool,
-                self._ptr(score_bias), cap, self._stream(),
+                self._ptr(score_bias), cap, keep_first, self._stream(),
             )
             return out
         self._check(ctx.cu_q, "cu_q", torch.int32, (entries + 1,))
@@ -1079,7 +1111,10 @@ class HipOps:
             )
         if num_decode:
             span = int(plan.max_decode_context)
-            if window:
+            if window and keep_first:
+                # the kept positions in whole tiles of 32, then the window from a multiple of 16 on
+                span = min(span + 48, int(window) + 15 + -(-keep_first // 32) * 32)
+            elif window:
                 span = min(span, int(window) + 15)
             if chunk:
                 span = min(span, chunk + 15)  # a partition starts at a multiple of 16 at or before the first key
@@ -1097,14 +1132,14 @@ class HipOps:
             leave_unmerged = (
                 defer_merge and self.tuning.fuse_merge and not num_tiles and num_decode == entries == tokens
                 and 1 < splits <= 64 and tokens <= self.FUSED_TOKENS and not chunk and sinks is None and share is None
-                and score_bias is None
+                and score_bias is None and not keep_first
             )
             self._call(
                 "mlr_attention_decode", self._ptr(qkv), stride, self._ptr(key_pages), self._ptr(value_pages),
                 self._ptr(block_table), width, self._ptr(ctx.cu_q), self._ptr(ctx.context_lens), self._ptr(out),
                 self._ptr(partial), entries, num_heads, num_kv_heads, block_size, num_pages, float(scale),
                 int(window or 0), chunk, part, splits, int(not leave_unmerged), self._ptr(sinks), self._ptr(share),
-                self._ptr(score_bias), cap, self._stream(), lib=lib,
+                self._ptr(score_bias), cap, keep_first, self._stream(), lib=lib,
             )
             if leave_unmerged:
                 return PendingMerge(
@@ -1142,7 +1177,7 @@ class HipOps:
                 self._ptr(block_table), width, self._ptr(tiles), num_tiles, wide, self._ptr(ctx.cu_q),
                 self._ptr(ctx.context_lens), self._ptr(out), num_heads, num_kv_heads, block_size, num_pages,
                 float(scale), int(window or 0), chunk, key_runs, self._ptr(partial), self._ptr(sinks), self._ptr(share),
-                self._ptr(score_bias), cap, self._stream(), lib=lib,
+                self._ptr(score_bias), cap, keep_first, self._stream(), lib=lib,
             )
         return out
 
@@ -1665,6 +1700,9 @@ class HipOps:
         first_values: Optional[torch.Tensor] = None,
         mix_weight: Optional[torch.Tensor] = None,
         weights: Optional[tuple] = None,
+        values_are_keys: bool = False,
+        temperature: Optional[tuple] = None,
+        projected_column: int = 0,
     ):
         """From the float32 sums of an attention layer's input product ([T, heads * head_dim + kv_heads * head_dim +
         kv_heads * value_dim (+ heads)]: queries, keys, values, gate logits) to what the attention kernels take.
@@ -1675,6 +1713,9 @@ class HipOps:
         the pages at `slot_mapping`, all zero beyond their own widths.  weights: (query norm weight, key norm weight),
         [head_dim] each; a head is then normed and multiplied by its weight BEFORE the rotation, and values are stored as
         they are.  kv_heads 0: the rows hold queries only (keys and values are another layer's), nothing is stored.
+        values_are_keys: the rows hold no values; a key's sums before its norm are its value too.  temperature: (positions
+        int32 [T], every, coef); queries are multiplied by 1 + coef * ln(floor((position + 1) / every) + 1).  Both go with
+        `weights`.  projected_column: where the rows start within wider ones that also hold other parts' sums.
         Returns (queries, sigmoid of the gate
         logits as float32 [T, heads] or None, the normed values before mixing as float32 if `keep_values`)."""
         self._check(projected, "projected input", torch.float32, (None, None))
@@ -1703,7 +1744,18 @@ class HipOps:
                 k_weight = None
             if keep_values or first_values is not None:
                 raise KernelError("weighted head norms leave the values as they are")
-        if width < (heads + kv_heads) * head_dim + kv_heads * value_dim + (heads if gated else 0):
+        if (values_are_keys or temperature is not None) and weights is None:
+            raise KernelError("keys that are values and queries that grow go with weighted head norms")
+        if values_are_keys and (not kv_heads or value_dim != head_dim or gated):
+            raise KernelError("keys that are values have one size, and no gate behind them")
+        positions, every, coef = None, 1.0, 0.0
+        if temperature is not None:
+            positions, every, coef = temperature
+            self._check(positions, "positions", torch.int32, (tokens,))
+            if not float(every) > 0:
+                raise KernelError("queries grow once in a length > 0")
+        own = (heads + kv_heads) * head_dim + (0 if values_are_keys else kv_heads * value_dim) + (heads if gated else 0)
+        if projected_column < 0 or width - projected_column < own:
             raise KernelError("the projected rows are too narrow")
         if first_values is not None:
             self._check(first_values, "first values", torch.float32, (tokens, kv_heads * value_dim))
@@ -1712,12 +1764,13 @@ class HipOps:
         gate = self._empty((tokens, heads), torch.float32) if gated else None
         kept = self._empty((tokens, kv_heads * value_dim), torch.float32) if keep_values else None
         self._call(
-            "mlr_head_norm_rope_write", self._ptr(projected), width, self._ptr(q), self._ptr(gate), self._ptr(cos),
+            "mlr_head_norm_rope_write", _VP(projected.data_ptr() + 4 * int(projected_column)), width, self._ptr(q), self._ptr(gate), self._ptr(cos),
             self._ptr(sin), int(rotary), float(eps), self._ptr(slot_mapping), self._ptr(key_pages),
             self._ptr(value_pages), self._ptr(kept), self._ptr(first_values),
             self._ptr(mix_weight if first_values is not None else None), self._ptr(q_weight), self._ptr(k_weight),
-            int(q_weight is not None and q_weight.dtype == torch.float32), self.code, tokens, heads, kv_heads, head_dim,
-            value_dim, kernel_dim, block_size, num_pages, self._stream(),
+            int(q_weight is not None and q_weight.dtype == torch.float32), int(bool(values_are_keys)), self._ptr(positions),
+            float(every), float(coef), self.code, tokens, heads, kv_heads, head_dim, value_dim, kernel_dim, block_size,
+            num_pages, self._stream(),
         )
         return q, gate, kept
 
@@ -2015,9 +2068,13 @@ class HipOps:
         axis is cut into `groups` contiguous blocks, a block scores the top-2 sum of its c, and ids are
         the arg-top-`top` of c over the experts of the `keep_groups` highest blocks; weights = s[ids] *
         `scale` (c only decides).  scores="softmax": s = softmax(z) over all experts instead.  normalise: the
-        chosen weights are divided by their sum (+ 1e-20) before the scale."""
-        if scores not in ("sigmoid", "softmax"):
-            raise KernelError("router scores are 'sigmoid' or 'softmax'")
+        chosen weights are divided by their sum (+ 1e-20) before the scale.  scores="chosen_softmax": the choice goes by z itself
+        (no correction) and the weights are the softmax over the chosen z."""
+        kinds = ("sigmoid", "softmax", "chosen_softmax")
+        if scores not in kinds:
+            raise KernelError(f"router scores are one of {', '.join(kinds)}")
+        if scores == "chosen_softmax" and correction is not None:
+            raise KernelError("a softmax over the chosen logits has no correction")
         self._check(logits, "router logits", torch.float32, (None, None))
         tokens, experts = logits.shape
         if correction is not None:
@@ -2026,7 +2083,7 @@ class HipOps:
         weights = self._empty((tokens, top), torch.float32)
         self._call(
             "mlr_moe_route", self._ptr(logits), self._ptr(correction), self._ptr(ids), self._ptr(weights), tokens,
-            experts, int(top), int(groups), int(keep_groups), float(scale), int(scores == "softmax"), int(bool(normalise)),
+            experts, int(top), int(groups), int(keep_groups), float(scale), kinds.index(scores), int(bool(normalise)),
             self._stream(),
         )
         return ids, weights
@@ -2043,6 +2100,9 @@ class HipOps:
         activation: str,
         kernel: str = "auto",
         pass_through: int = 0,
+        glu: Optional[tuple[float, float]] = None,
+        woven: bool = False,
+        beside: Optional[tuple[torch.Tensor, torch.Tensor]] = None,
     ) -> torch.Tensor:
         """The chosen experts' outputs, weighted: float32 [top, T, hidden] with [j, t] = weights[t, j]
         * down_e(act(up_e(h[t]))), e = ids[t, j]; the sum over j is the mixture's output, which a norm
@@ -2052,12 +2112,24 @@ class HipOps:
         - 1 name experts without matrices whose output is their input: [j, t] = weights[t, j] * h[t].  up_weight [experts * inner, hidden], down_weight [experts *
         hidden, inner].  Three launches: the pairs sorted by expert into tiles of rows, and a grouped
         product over the tiles for each of the two matrices (bfloat16 with hidden and inner multiples
-        of 8 on the matrix cores, everything else, and kernel="fma", as plain 32-bit arithmetic)."""
+        of 8 on the matrix cores, everything else, and kernel="fma", as plain 32-bit arithmetic).
+        activation "clamped_glu" with glu = (limit, alpha): a gated expert whose activation is that of `linear`'s `clamped_glu`.
+        `woven`: its gate and up rows lie in pairs as for `linear`, and the gating is the first product's epilogue; else
+        they lie as for "swiglu" and it is a kernel of its own.
+        beside: (x [T, k], weight [hidden, k]) of a product whose sums join the mixture (a shared expert's second matrix):
+        one more slice of the stack, or a few of partial sums over k."""
         if kernel not in ("auto", "fma"):
             raise KernelError("kernel must be 'auto' or 'fma'")
-        if activation not in ("relu2", "sigmoid", "swiglu"):
+        if activation not in ("relu2", "sigmoid", "swiglu", "clamped_glu"):
             raise KernelError(f"unknown activation {activation!r}")
-        gated = activation == "swiglu"
+        gated = activation in ("swiglu", "clamped_glu")
+        limit = alpha = 0.0
+        if activation == "clamped_glu":
+            if glu is None or not glu[0] > 0:
+                raise KernelError("the clamped gating needs a limit > 0")
+            limit, alpha = float(glu[0]), float(glu[1])
+        if woven and activation != "clamped_glu":
+            raise KernelError("rows woven in pairs go with the clamped gating")
         self._check(h, "expert input", self.dtype, (None, None))
         tokens, hidden = h.shape
         self._check(ids, "expert ids", torch.int32, (tokens, None))
@@ -2066,8 +2138,8 @@ class HipOps:
         if experts <= 0 or up_weight.shape[0] % experts:
             raise KernelError("the stacked expert matrices do not divide by the number of experts")
         wide = up_weight.shape[0] // experts  # rows of an expert's first matrix
-        if gated and wide % 2:
-            raise KernelError("a gated expert's first matrix holds gate rows and as many up rows")
+        if gated and (wide % 2 or (woven and wide % 4)):
+            raise KernelError("a gated expert's first matrix holds gate rows and as many up rows (an even number if woven)")
         inner = wide // 2 if gated else wide
         self._check(up_weight, "expert up weights", self.dtype, (experts * wide, hidden))
         self._check(down_weight, "expert down weights", self.dtype, (experts * hidden, inner))
@@ -2087,15 +2159,27 @@ class HipOps:
             "mlr_moe_align", self._ptr(ids), pairs, experts, big, max_tiles, self._ptr(order), self._ptr(offsets),
             self._ptr(tiles), self._stream(),
         )
-        act = self._empty((pairs, wide), self.dtype)
-        out = self._empty((top, tokens, hidden), torch.float32)
+        act = self._empty((pairs, inner if woven else wide), self.dtype)
+        more = 0
+        if beside is not None:
+            x, weight = beside
+            self._check(weight, "weight of the product beside the experts", self.dtype, (hidden, None))
+            more = 1
+            if self.dtype == torch.bfloat16 and kernel == "auto" and weight.shape[1] % 8 == 0:
+                more = self.lib.mlr_gemm_bf16_slices(tokens, hidden, weight.shape[1], self.max_k_slices)
+        out = self._empty((top + more, tokens, hidden), torch.float32)
+        if more == 1:
+            self.linear(x, weight, None, out_dtype=torch.float32, kernel=kernel, slices=None, out=out[top])
+        elif more:
+            self.linear(x, weight, None, partial_sums=True, slices=more, out=out[top:])
         common = (self._ptr(order), self._ptr(offsets), self._ptr(tiles))
         self._call(
             "mlr_moe_gemm", self._ptr(h), self._ptr(up_weight), *common, _VP(None), self._ptr(act), 1, self.code, mfma,
-            max_tiles, tokens, top, wide, hidden, 0 if gated else _EPILOGUES[activation], self._stream(),
+            max_tiles, tokens, top, wide, hidden, 0 if gated and not woven else _EPILOGUES[activation], limit, alpha,
+            self._stream(),
         )
-        if gated:
-            act = self.silu_mul(act)  # rows that no pair owns hold whatever memory held: nothing reads them
+        if gated and not woven:  # rows that no pair owns hold whatever memory held: nothing reads them
+            act = self.silu_mul(act) if activation == "swiglu" else self.glu_clamped(act, limit, alpha)
         if pass_through:
             self._call(
                 "mlr_moe_identity", self._ptr(h), self._ptr(ids), self._ptr(weights), self._ptr(out), self.code, tokens,
@@ -2103,7 +2187,7 @@ class HipOps:
             )
         self._call(
             "mlr_moe_gemm", self._ptr(act), self._ptr(down_weight), *common, self._ptr(weights), self._ptr(out), 0,
-            self.code, mfma, max_tiles, tokens, top, hidden, inner, 0, self._stream(),
+            self.code, mfma, max_tiles, tokens, top, hidden, inner, 0, 0.0, 0.0, self._stream(),
         )
         return out
 

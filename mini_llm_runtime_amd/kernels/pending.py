@@ -100,11 +100,28 @@ class NormedDelta:
     x += weight * y * rsqrt(mean(y^2) + eps), for arrangements that norm a sublayer's output as well as
     its input.  Handed to the next norm as its delta, so that the normed addition and that norm are one
     kernel.  `y` is whatever a part may return: [T, H] in the engine's dtype or float32, a float32 stack
-    [S, T, H] whose sum it is, or a product that has not run."""
+    [S, T, H] whose sum it is, or a product that has not run.
+
+    `second` = (y, weight): another output, normed by its own size with a weight of its own, added to the first; both
+    are then multiplied by `scale` and `second_scale`."""
 
     y: object
     weight: torch.Tensor
     eps: float
+    second: Optional[tuple] = None
+    scale: float = 1.0
+    second_scale: float = 1.0
+
+    def options(self) -> dict:
+        """What the kernel library's `add_normed` takes beyond y, weight and eps (nothing where there is nothing)."""
+        if self.second is None and self.scale == 1.0:
+            return {}
+        return {"second": self.second, "scales": (self.scale, self.second_scale)}
+
+    def with_outputs(self, choose) -> "NormedDelta":
+        """The same with `choose` (of rows, say) applied to every output."""
+        second = None if self.second is None else (choose(self.second[0]), self.second[1])
+        return NormedDelta(choose(self.y), self.weight, self.eps, second, self.scale, self.second_scale)
 
 
 @dataclass

@@ -1,6 +1,6 @@
 """Architectures: each module registers one name with its configuration and builder."""
 
-from . import bubitar, fedolorn, pepulix, qwen2, rofetar, vobisun  # noqa: F401  (each registers its architecture)
+from . import bubitar, fedolorn, goguzen, pepulix, qwen2, rofetar, vobisun  # noqa: F401  (each registers its architecture)
 from .registry import (
     ARCHITECTURES,
     Architecture,

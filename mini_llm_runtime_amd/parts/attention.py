@@ -52,6 +52,11 @@ class GQAAttention(Mixer):
         kernel norms, rotates and stores, and heads whose size is no multiple of 16 are padded there to one that is.
     softcap: score <- softcap * tanh(score / softcap), after the scale.
     unit_sink: the softmax's denominator is one larger (a key of score 0 without a value).
+    sink: the denominator of head h is larger by exp(sinks[h]), a learned number per head.
+    values_are_keys: there is no value projection; a token's value is its key as projected, before norm and position
+        (both are stored).  Goes with `qk_norm_eps`.
+    query_temperature: (every, coef); queries at position p are multiplied by 1 + coef * ln(floor((p + 1) / every) + 1), in
+        32-bit, behind norm and rotation.  Goes with `qk_norm_eps`.
     reads_cache: the layer has no key and value projections; it reads the pages another site owns (an execution
         order entry with `reads_cache_of`).  Goes with `qk_norm_eps`.
     """
@@ -77,6 +82,9 @@ class GQAAttention(Mixer):
         softcap: Optional[float] = None,
         unit_sink: bool = False,
         reads_cache: bool = False,
+        sink: bool = False,
+        values_are_keys: bool = False,
+        query_temperature: Optional[tuple] = None,
     ) -> None:
         if num_heads <= 0 or num_kv_heads <= 0 or num_heads % num_kv_heads:
             raise ValueError("num_heads must be a positive multiple of num_kv_heads")
@@ -90,6 +98,14 @@ class GQAAttention(Mixer):
             raise ValueError("softcap must be > 0")
         if qk_norm_eps is None and reads_cache:
             raise ValueError("queries without keys of their own go with per-head norms")
+        if qk_norm_eps is None and (values_are_keys or query_temperature is not None):
+            raise ValueError("values that are keys and a query temperature go with per-head norms")
+        if values_are_keys and (reads_cache or value_dim not in (None, head_dim)):
+            raise ValueError("values that are keys are a layer's own and have the keys' size")
+        if sink and unit_sink:
+            raise ValueError("a mixer has learned sinks or one of score 0, not both")
+        if query_temperature is not None and not query_temperature[0] > 0:
+            raise ValueError("queries grow once in a length > 0")
         if qk_norm_eps is not None and (qkv_bias or not qk_norm_eps >= 0):
             raise ValueError("per-head norms have an eps >= 0 and go with projections without biases")
         self.hidden_size = int(hidden_size)
@@ -113,6 +129,13 @@ class GQAAttention(Mixer):
         self.qk_norm_eps = None if qk_norm_eps is None else float(qk_norm_eps)
         self.softcap = None if softcap is None else float(softcap)
         self.unit_sink = bool(unit_sink)
+        self.sink = bool(sink)
+        self.values_are_keys = bool(values_are_keys)
+        self.query_temperature = (
+            None if query_temperature is None else (float(query_temperature[0]), float(query_temperature[1]))
+        )
+        # `forward(projected=)` takes the input product's sums from whoever made them
+        self.open_input = self.qk_norm_eps is not None
         self.reads_cache = bool(reads_cache)
         self.position: Optional[PositionEncoding] = (
             build_part("position", position) if position is not None else None
@@ -138,7 +161,16 @@ class GQAAttention(Mixer):
 
     @property
     def v_size(self) -> int:
-        return self.num_kv_heads * self.value_dim
+        return 0 if self.values_are_keys else self.num_kv_heads * self.value_dim
+
+    # the input product under the names that a holder of several mixers looks for
+    @property
+    def in_weight(self) -> Optional[torch.Tensor]:
+        return self.qkv_weight
+
+    @in_weight.setter
+    def in_weight(self, weight: Optional[torch.Tensor]) -> None:
+        self.qkv_weight = weight
 
     @property
     def out_size(self) -> int:
@@ -157,6 +189,8 @@ class GQAAttention(Mixer):
             specs["o_bias_vec"] = ParamSpec((self.hidden_size,), keep_stored_precision=True)
         if self.output_gate:
             specs["gate_weight"] = ParamSpec((self.out_size, self.hidden_size))
+        if self.sink:
+            specs["sinks"] = ParamSpec((self.num_heads,), keep_stored_precision=True)
         if self.qk_norm_eps is not None:
             specs["q_norm_weight"] = ParamSpec((self.head_dim,), init="one_plus_normal", keep_stored_precision=True)
             if not self.reads_cache:
@@ -168,6 +202,8 @@ class GQAAttention(Mixer):
         D = self.kernel_dim
         if self.unit_sink:
             self.sinks = torch.zeros(self.num_heads, dtype=torch.float32, device=device)  # exp(0) = 1
+        elif self.sink:
+            self.sinks = self.sinks.to(torch.float32).contiguous()
         if D == self.head_dim == self.value_dim:
             return
         # heads of two widths: every head at the common size D, the added rows and columns zero
@@ -203,7 +239,9 @@ class GQAAttention(Mixer):
         make = getattr(ops, "attention_plan", None)  # the kernel library knows what its kernels want
         return make(shape) if make is not None else None
 
-    def forward(self, ctx: StepContext, h: torch.Tensor, site: int) -> torch.Tensor:
+    def forward(self, ctx: StepContext, h: torch.Tensor, site: int, projected=None) -> torch.Tensor:
+        """`projected`: (float32 sums [T, ...], first column) of h times `qkv_weight`, when the caller made them within a
+        larger product (with `open_input` only)."""
         ops = ctx.ops
         cache = ctx.kv(site)
         rotation = self.position.rotation(ctx) if self.position is not None else None
@@ -220,8 +258,18 @@ class GQAAttention(Mixer):
             if self.position is not None and rotation is None:
                 raise RuntimeError("per-head norms go with a rotation or no position encoding")
             own = self.num_kv_heads if cache.writable else 0
+            first = 0
+            if projected is None:
+                projected = ops.linear(h, self.qkv_weight, None, out_dtype=torch.float32)  # norms read it unrounded
+            else:
+                projected, first = projected
+            options = {"values_are_keys": True} if self.values_are_keys else {}
+            if self.query_temperature is not None:
+                options["temperature"] = (ctx.positions, *self.query_temperature)
+            if first:
+                options["projected_column"] = first
             qkv, _, _ = ops.head_norm_rope_write(
-                ops.linear(h, self.qkv_weight, None, out_dtype=torch.float32),  # norms read it unrounded
+                projected,
                 heads=self.num_heads,
                 kv_heads=own,
                 head_dim=self.head_dim,
@@ -234,6 +282,7 @@ class GQAAttention(Mixer):
                 value_pages=cache.value if own else None,
                 block_size=cache.block_size,
                 weights=(self.q_norm_weight, self.k_norm_weight),
+                **options,
             )
         elif self.position is not None and rotation is None:
             # a position encoding with a rule of its own: it sees the queries and keys between
@@ -267,7 +316,7 @@ class GQAAttention(Mixer):
             defer_merge=not self.output_gate,  # the output product is the only reader
             plan=ctx.plan(getattr(ops, "ATTENTION_PLAN", None)),
             **({"chunk": self.chunk} if self.chunk is not None else {}),
-            **({"sinks": self.sinks} if self.unit_sink else {}),
+            **({"sinks": self.sinks} if self.sinks is not None else {}),
             **({"softcap": self.softcap} if self.softcap is not None else {}),
         )
         if self.output_gate:

@@ -6,10 +6,10 @@ from typing import Optional
 
 import torch
 
-from .base import FeedForward
+from .base import FeedForward, Part
 from .context import StepContext
-from .registry import register_part
-from .spec import ParamSpec
+from .registry import build_part, register_part
+from .spec import ParamSpec, PartSpec
 
 
 @register_part("feed_forward", "swiglu")
@@ -61,7 +61,7 @@ class SwiGLU(FeedForward):
 
 @register_part("feed_forward", "clamped_glu")
 class ClampedGLU(FeedForward):
-    """Dense gated feed-forward with clamped halves and biases on all three products:
+    """Dense gated feed-forward with clamped halves and (unless `bias` is False) biases on all three products:
 
         g = min(Wgate x + bgate, limit),  u = clamp(Wup x + bup, -limit, limit),
         y = Wdown (g * sigmoid(alpha * g) * (u + 1)) + bdown.
@@ -74,13 +74,16 @@ class ClampedGLU(FeedForward):
 
     replayable = True
 
-    def __init__(self, hidden_size: int, intermediate_size: int, limit: float, alpha: float = 1.702) -> None:
+    def __init__(
+        self, hidden_size: int, intermediate_size: int, limit: float, alpha: float = 1.702, bias: bool = True
+    ) -> None:
         if hidden_size <= 0 or intermediate_size <= 0 or not limit > 0:
             raise ValueError("ClampedGLU sizes and limit must be > 0")
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
         self.limit = float(limit)
         self.alpha = float(alpha)
+        self.bias = bool(bias)
         self.woven = self.intermediate_size % 2 == 0
         self.gate_up_weight: Optional[torch.Tensor] = None
         self.gate_up_bias: Optional[torch.Tensor] = None
@@ -88,21 +91,25 @@ class ClampedGLU(FeedForward):
         self.down_bias: Optional[torch.Tensor] = None
 
     def param_specs(self) -> dict[str, ParamSpec]:
-        return {
+        specs = {
             "gate_up_weight": ParamSpec((2 * self.intermediate_size, self.hidden_size)),
-            "gate_up_bias": ParamSpec((2 * self.intermediate_size,), keep_stored_precision=True),
             "down_weight": ParamSpec((self.hidden_size, self.intermediate_size)),
-            "down_bias": ParamSpec((self.hidden_size,), keep_stored_precision=True),
         }
+        if self.bias:
+            specs["gate_up_bias"] = ParamSpec((2 * self.intermediate_size,), keep_stored_precision=True)
+            specs["down_bias"] = ParamSpec((self.hidden_size,), keep_stored_precision=True)
+        return specs
 
-    def forward(self, ctx: StepContext, h: torch.Tensor) -> torch.Tensor:
+    def inner(self, ctx: StepContext, h: torch.Tensor) -> torch.Tensor:
+        """What the last product reads."""
         ops = ctx.ops
         if self.woven:
-            hidden = ops.linear(h, self.gate_up_weight, self.gate_up_bias, clamped_glu=(self.limit, self.alpha))
-        else:
-            sums = ops.linear(h, self.gate_up_weight, self.gate_up_bias, out_dtype=torch.float32)
-            hidden = ops.glu_clamped(sums, self.limit, self.alpha)
-        return ops.linear(hidden, self.down_weight, self.down_bias, for_stream=True)
+            return ops.linear(h, self.gate_up_weight, self.gate_up_bias, clamped_glu=(self.limit, self.alpha))
+        sums = ops.linear(h, self.gate_up_weight, self.gate_up_bias, out_dtype=torch.float32)
+        return ops.glu_clamped(sums, self.limit, self.alpha)
+
+    def forward(self, ctx: StepContext, h: torch.Tensor) -> torch.Tensor:
+        return ctx.ops.linear(self.inner(ctx, h), self.down_weight, self.down_bias, for_stream=True)
 
 
 @register_part("feed_forward", "geglu")
@@ -146,7 +153,8 @@ class GeGLU(FeedForward):
 
 
 ACTIVATIONS = ("relu2", "sigmoid")  # what `ops.linear(..., activation=)` applies to its sums
-EXPERT_ACTIVATIONS = ACTIVATIONS + ("swiglu",)  # an expert may also be gated: down(silu(gate(x)) * up(x))
+# an expert may also be gated: down(silu(gate(x)) * up(x)), or with clamped halves as in `ClampedGLU`
+EXPERT_ACTIVATIONS = ACTIVATIONS + ("swiglu", "clamped_glu")
 
 
 @register_part("feed_forward", "mlp")
@@ -207,6 +215,12 @@ class RoutedExperts(FeedForward):
         matrices whose output is their input itself (times the weight).
     activation "swiglu": every expert is gated, down_e(silu(gate_e(x)) * up_e(x)); `up_weight` then holds, per
         expert, its gate rows and then its up rows ([experts * 2 * inner, hidden]).
+    activation "clamped_glu" (with `limit`, `alpha`): every expert is a `ClampedGLU` without biases; its gate and up rows lie
+        woven in pairs, expert by expert, and the gating is the first grouped product's epilogue (an odd inner size: gate
+        rows, then up rows, gated by a kernel of its own).
+    scores "chosen_softmax": the choice goes by z, the weights are the softmax over the chosen z only.
+    correction False: there is no stored correction.  router_bias: z = Wr h + b.
+    shared: a `ClampedGLU` without biases that every token runs; its output is added (one more slice of the stack).
     """
 
     replayable = True
@@ -224,6 +238,11 @@ class RoutedExperts(FeedForward):
         scores: str = "sigmoid",
         normalise: bool = False,
         identity: int = 0,
+        limit: Optional[float] = None,
+        alpha: float = 1.702,
+        correction: bool = True,
+        router_bias: bool = False,
+        shared: Optional[PartSpec] = None,
     ) -> None:
         if hidden_size <= 0 or intermediate_size <= 0 or experts <= 0 or top <= 0 or identity < 0:
             raise ValueError("RoutedExperts sizes must be > 0")
@@ -232,8 +251,12 @@ class RoutedExperts(FeedForward):
             raise ValueError("the experts must divide into equal groups, of which 1..groups are kept")
         if top > keep_groups * (routed // groups):
             raise ValueError("the kept groups hold fewer experts than a token uses")
-        if scores not in ("sigmoid", "softmax"):
-            raise ValueError("scores are 'sigmoid' or 'softmax'")
+        if scores not in ("sigmoid", "softmax", "chosen_softmax"):
+            raise ValueError("scores are 'sigmoid', 'softmax' or 'chosen_softmax'")
+        if scores == "chosen_softmax" and (correction or normalise):
+            raise ValueError("a softmax over the chosen logits has no correction and is normalised by itself")
+        if (activation == "clamped_glu") != (limit is not None) or (limit is not None and not limit > 0):
+            raise ValueError("a limit > 0 goes with the clamped gating")
         if activation not in EXPERT_ACTIVATIONS:
             raise ValueError(f"unknown activation {activation!r}; known: {', '.join(ACTIVATIONS)}")
         self.hidden_size = int(hidden_size)
@@ -248,28 +271,45 @@ class RoutedExperts(FeedForward):
         self.normalise = bool(normalise)
         self.identity = int(identity)
         self.routed = routed
+        self.limit = None if limit is None else float(limit)
+        self.alpha = float(alpha)
+        self.has_correction = bool(correction)
+        self.has_router_bias = bool(router_bias)
+        self.gated = activation in ("swiglu", "clamped_glu")
+        self.woven = activation == "clamped_glu" and self.intermediate_size % 2 == 0
+        self.shared = build_part("feed_forward", shared) if shared is not None else None
+        if self.shared is not None and (not hasattr(self.shared, "inner") or getattr(self.shared, "bias", True)):
+            raise ValueError("a shared expert ends in a product without a bias (a clamped_glu part with bias=False)")
+        self.router_bias: Optional[torch.Tensor] = None
         self.router_weight: Optional[torch.Tensor] = None
         self.correction: Optional[torch.Tensor] = None
         self.up_weight: Optional[torch.Tensor] = None
         self.down_weight: Optional[torch.Tensor] = None
 
+    def children(self) -> dict[str, Part]:
+        return {"shared": self.shared} if self.shared is not None else {}
+
     def param_specs(self) -> dict[str, ParamSpec]:
-        return {
-            "router_weight": ParamSpec((self.routed, self.hidden_size)),
-            "correction": ParamSpec((self.routed,), keep_stored_precision=True),
-            "up_weight": ParamSpec(
-                (self.experts * self.intermediate_size * (2 if self.activation == "swiglu" else 1), self.hidden_size)
-            ),
-            "down_weight": ParamSpec((self.experts * self.hidden_size, self.intermediate_size)),
-        }
+        specs = {"router_weight": ParamSpec((self.routed, self.hidden_size))}
+        if self.has_correction:
+            specs["correction"] = ParamSpec((self.routed,), keep_stored_precision=True)
+        if self.has_router_bias:
+            specs["router_bias"] = ParamSpec((self.routed,), keep_stored_precision=True)
+        specs["up_weight"] = ParamSpec((self.experts * self.intermediate_size * (2 if self.gated else 1), self.hidden_size))
+        specs["down_weight"] = ParamSpec((self.experts * self.hidden_size, self.intermediate_size))
+        return specs
 
     def bind(self, params, *, dtype: torch.dtype, device: torch.device) -> None:
         super().bind(params, dtype=dtype, device=device)
-        self.correction = self.correction.to(torch.float32)  # the routing is 32-bit throughout
+        # the routing is 32-bit throughout
+        if self.correction is not None:
+            self.correction = self.correction.to(torch.float32)
+        if self.router_bias is not None:
+            self.router_bias = self.router_bias.to(torch.float32)
 
     def forward(self, ctx: StepContext, h: torch.Tensor):
         ops = ctx.ops
-        logits = ops.linear(h, self.router_weight, None, out_dtype=torch.float32)
+        logits = ops.linear(h, self.router_weight, self.router_bias, out_dtype=torch.float32)
         ids, weights = ops.route_experts(
             logits, self.correction, top=self.top, groups=self.groups, keep_groups=self.keep_groups,
             scale=self.router_scale,
@@ -278,4 +318,6 @@ class RoutedExperts(FeedForward):
         return ops.expert_products(
             h, self.up_weight, self.down_weight, ids, weights, experts=self.experts, activation=self.activation,
             **({"pass_through": self.identity} if self.identity else {}),
+            **({"glu": (self.limit, self.alpha), "woven": self.woven} if self.activation == "clamped_glu" else {}),
+            **({"beside": (self.shared.inner(ctx, h), self.shared.down_weight)} if self.shared is not None else {}),
         )

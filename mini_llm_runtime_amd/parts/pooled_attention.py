@@ -1,4 +1,4 @@
-"""Windowed attention that also sees pooled blocks of what left the window."""
+"""Windowed attention that also sees pooled blocks of what left the window, or the first tokens."""
 
 from __future__ import annotations
 
@@ -27,6 +27,8 @@ class PooledWindowAttention(Mixer):
     A query at position p sees the tokens j with 0 <= p - j < window and, if `pool` = P is given, block b
     (positions bP .. bP + P - 1) once bP + P - 1 <= p - window, through the means of the block's cached keys
     and of its values; tokens that have left the window and whose block is not complete yet are not seen.
+    keep_first: the first `keep_first` tokens of a request are seen by all its later queries beside the window, at
+    their true positions (not with `pool`); their pages are not given back.  window None: all earlier tokens are seen.
     Tokens and blocks share one softmax, score = q . k * scale, whose denominator also holds exp(sink_i)
     (a learned number per head, if `sink`).  `head_gate`: head i's output times sigmoid(Wg h)_i, one number
     per head.  Output: Wo on the heads side by side.
@@ -48,7 +50,7 @@ class PooledWindowAttention(Mixer):
         num_heads: int,
         num_kv_heads: int,
         head_dim: int,
-        window: int,
+        window: Optional[int],
         scale: float,
         value_dim: Optional[int] = None,
         pool: Optional[int] = None,
@@ -59,11 +61,16 @@ class PooledWindowAttention(Mixer):
         temperature: bool = False,
         sink: bool = False,
         head_gate: bool = False,
+        keep_first: int = 0,
     ) -> None:
         if num_heads <= 0 or num_kv_heads <= 0 or num_heads % num_kv_heads:
             raise ValueError("num_heads must be a positive multiple of num_kv_heads")
-        if head_dim <= 0 or window <= 0 or (pool is not None and pool <= 0) or not scale > 0:
+        if head_dim <= 0 or (window is not None and window <= 0) or (pool is not None and pool <= 0) or not scale > 0:
             raise ValueError("head_dim, window, pool and scale must be > 0")
+        if window is None and pool is not None:
+            raise ValueError("pooled blocks lie before a window")
+        if keep_first < 0 or (keep_first and pool is not None):
+            raise ValueError("keep_first must be >= 0 and goes without pooled blocks")
         self.hidden_size = int(hidden_size)
         self.num_heads = int(num_heads)
         self.num_kv_heads = int(num_kv_heads)
@@ -74,7 +81,8 @@ class PooledWindowAttention(Mixer):
         # the one head size that kernels and pages see
         self.kernel_dim = -(-max(self.head_dim, self.value_dim) // 16) * 16
         check_attention_sizes(num_heads, num_kv_heads, self.kernel_dim)
-        self.window = int(window)
+        self.window = None if window is None else int(window)
+        self.keep_first = int(keep_first) if window is not None else 0
         self.pool = None if pool is None else int(pool)
         self.scale = float(scale)
         self.qkv_bias = bool(qkv_bias)
@@ -161,7 +169,7 @@ class PooledWindowAttention(Mixer):
     def cache_spec(self) -> Any:
         # a block is pooled from its tokens' pages when its last token comes in: they stay that long
         keep = self.window if self.pool is None else max(self.window, self.pool)
-        tokens = PagedKVSpec(self.num_kv_heads, self.kernel_dim, keep)
+        tokens = PagedKVSpec(self.num_kv_heads, self.kernel_dim, keep, keep_first=self.keep_first)
         if self.pool is None:
             return tokens
         return CompositeSpec({"tokens": tokens, "pooled": PagedKVSpec(self.num_kv_heads, self.kernel_dim, tokens_per_entry=self.pool)})
@@ -170,11 +178,8 @@ class PooledWindowAttention(Mixer):
         make = getattr(ops, "attention_plan", None)
         return make(shape) if make is not None else None
 
-    def activations(
-        self, ctx: StepContext, h, site: Any, *, out: torch.Tensor, column: int, scale: float = 1.0, projected=None
-    ) -> None:
-        """`projected`: (float32 sums [T, ...], first column) of h times `in_weight` (+ `in_bias`), when the
-        caller made them within a larger product."""
+    def _attended(self, ctx: StepContext, h, site: Any, projected=None):
+        """(heads side by side at the kernels' head size, gates per head or None)."""
         ops = ctx.ops
         if self.pool is None:
             cache, pooled = ctx.kv(site), None
@@ -212,13 +217,25 @@ class PooledWindowAttention(Mixer):
             block_size=cache.block_size, scale=self.scale, window=self.window, sinks=self.sinks,
             plan=ctx.plan(getattr(ops, "ATTENTION_PLAN", None)),
             **({"pooled": seen} if seen is not None else {}),
+            **({"keep_first": self.keep_first} if self.keep_first else {}),
         )
-        ops.scale_heads(
+        return attended, gate
+
+    def activations(
+        self, ctx: StepContext, h, site: Any, *, out: torch.Tensor, column: int, scale: float = 1.0, projected=None
+    ) -> None:
+        """`projected`: (float32 sums [T, ...], first column) of h times `in_weight` (+ `in_bias`), when the
+        caller made them within a larger product."""
+        attended, gate = self._attended(ctx, h, site, projected)
+        ctx.ops.scale_heads(
             attended, gate, heads=self.num_heads, head_dim=self.kernel_dim, out_dim=self.value_dim, scale=scale,
             out=out, column=column,
         )
 
     def forward(self, ctx: StepContext, h: torch.Tensor, site: Any) -> torch.Tensor:
-        out = torch.empty((h.shape[0], self.out_width), dtype=ctx.dtype, device=ctx.device)
-        self.activations(ctx, h, site, out=out, column=0)
-        return ctx.ops.linear(out, self.o_weight, None, for_stream=True)
+        attended, gate = self._attended(ctx, h, site)
+        if gate is not None or self.kernel_dim != self.value_dim:
+            attended = ctx.ops.scale_heads(
+                attended, gate, heads=self.num_heads, head_dim=self.kernel_dim, out_dim=self.value_dim
+            )
+        return ctx.ops.linear(attended, self.o_weight, None, for_stream=True)

@@ -31,7 +31,9 @@ class RotaryEmbedding(PositionEncoding):
     lo, 0.001), 0, 1), pair j turns at f_j / factor * ramp_j + f_j * (1 - ramp_j): fast pairs keep
     their frequency, slow ones are stretched by `factor`.  Cosines and sines are then multiplied by
     0.1 ln(factor) + 1.  A scaling that gives `factor` alone is the linear one: every pair turns at f_j /
-    factor, amplitudes stay 1.
+    factor, amplitudes stay 1.  One of (factor, original, low, high) goes by the turn's length l_j = 2 pi / f_j: pairs with
+    l_j < original / high keep f_j, those with l_j > original / low turn at f_j / factor, and between the two, with s =
+    (original / l_j - low) / (high - low), a pair turns at (1 - s) f_j / factor + s f_j; amplitudes stay 1.
 
     interleaved: the checkpoint pairs dim 2j with dim 2j + 1 (instead of j with j + r/2).  The kernels
     rotate halves; a dot product of a query and a key does not care in which order both list their
@@ -69,6 +71,17 @@ class RotaryEmbedding(PositionEncoding):
                 raise ValueError("the factor of a rotary scaling must be > 0")
             self.scaling = (factor,)
             self._inv_freq_host = self._inv_freq_host / factor
+        elif scaling is not None and "low" in scaling:
+            factor, original = float(scaling["factor"]), float(scaling["original"])
+            low, high = float(scaling["low"]), float(scaling["high"])
+            if not (factor > 0 and original > 0 and 0 < low <= high):
+                raise ValueError("the numbers of a rotary scaling must be > 0, and 'high' at least 'low'")
+            self.scaling = ("bands", factor, original, low, high)
+            f = self._inv_freq_host
+            turn = 2.0 * math.pi / f
+            keep = np.clip((original / turn - low) / (high - low), 0.0, 1.0) if high > low else np.zeros_like(f)
+            blended = (1.0 - keep) * f / factor + keep * f
+            self._inv_freq_host = np.where(turn < original / high, f, np.where(turn > original / low, f / factor, blended))
         elif scaling is not None:
             factor, original = float(scaling["factor"]), float(scaling["original"])
             fast, slow = float(scaling["fast"]), float(scaling["slow"])

@@ -47,6 +47,7 @@ class StateSpace(Mixer):
     """
 
     replayable = True
+    open_input = True  # `forward(projected=)` takes the input product's sums from whoever made them
 
     def __init__(
         self, hidden_size: int, num_heads: int, value_dim: int, state_dim: int, groups: int, taps: int, norm_groups: int,
@@ -105,18 +106,24 @@ class StateSpace(Mixer):
         state = SlotStateSpec((self.num_heads, self.state_dim, self.value_dim), "float32")
         return conv_state_spec(state, self.taps, self.channels)
 
-    def forward(self, ctx: StepContext, h: torch.Tensor, site: Any) -> torch.Tensor:
+    def forward(self, ctx: StepContext, h: torch.Tensor, site: Any, projected=None) -> torch.Tensor:
+        """`projected`: (float32 sums [T, ...], first column) of h times `in_weight`, when the caller made them within a
+        larger product."""
         ops = ctx.ops
         state, carried = conv_state_views(ctx, site, self.taps)
-        projected = ops.linear(h, self.in_weight, None, out_dtype=torch.float32)  # what enters the recurrence stays 32-bit
+        first = 0
+        if projected is None:
+            projected = ops.linear(h, self.in_weight, None, out_dtype=torch.float32)  # what enters the recurrence stays 32-bit
+        else:
+            projected, first = projected
         b_at = self.inner  # the channels: x, B, C
         y = ops.conv_decay_scan(
-            projected, self.conv_taps, self.conv_bias, carried, state, ctx, column=self.inner, heads=self.num_heads,
+            projected, self.conv_taps, self.conv_bias, carried, state, ctx, column=first + self.inner, heads=self.num_heads,
             key_heads=self.groups, head_dim=self.state_dim, value_dim=self.value_dim,
             offsets=(b_at + self.groups * self.state_dim, b_at, 0), rate=self.rate, dt_bias=self.dt_bias,
-            step_column=self.inner + self.channels, skip=self.skip,
+            step_column=first + self.inner + self.channels, skip=self.skip,
         )
         gated = ops.gate_group_norm(
-            y, projected, gate_column=0, groups=self.norm_groups, eps=self.norm_eps, norm_weight=self.norm_weight
+            y, projected, gate_column=first, groups=self.norm_groups, eps=self.norm_eps, norm_weight=self.norm_weight
         )
         return ops.linear(gated, self.o_weight, None, for_stream=True)

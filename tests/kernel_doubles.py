@@ -36,18 +36,23 @@ class TorchOps:
 
     def settle(self, h):
         if isinstance(h, NormedDelta):
-            y = self._sum(h.y)
-            return h.weight.float() * (y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + h.eps))
+
+            def normed(y, weight):
+                y = self._sum(self.settle(y))
+                return weight.float() * (y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + h.eps))
+
+            added = h.scale * normed(h.y, h.weight)
+            return added if h.second is None else added + h.second_scale * normed(*h.second)
         return h
 
     @staticmethod
     def _sum(y):
         return y.float().sum(0) if y.dim() == 3 else y.float()
 
-    def add_normed(self, x, y, weight, eps, next_weight=None, next_eps=0.0, cast=False):
+    def add_normed(self, x, y, weight, eps, next_weight=None, next_eps=0.0, cast=False, second=None, scales=(1.0, 1.0)):
         self._count("add_normed")
         assert x.dtype == torch.float32
-        x += self.settle(NormedDelta(y, weight, eps))
+        x += self.settle(NormedDelta(y, weight, eps, second, *scales))
         if next_weight is not None:
             return (next_weight.float() * (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + next_eps))).to(self.dtype)
         return x.to(self.dtype) if cast else None
@@ -56,7 +61,7 @@ class TorchOps:
         self._count("rmsnorm")
         assert x.dtype == torch.float32
         if isinstance(delta, NormedDelta):
-            return self.add_normed(x, delta.y, delta.weight, delta.eps, next_weight=weight, next_eps=eps)
+            return self.add_normed(x, delta.y, delta.weight, delta.eps, next_weight=weight, next_eps=eps, **delta.options())
         if delta is not None:
             x += delta.float().sum(0) if delta.dim() == 3 else delta.float()
         variance = x.pow(2).mean(-1, keepdim=True)
@@ -73,7 +78,7 @@ class TorchOps:
 
     def gather_rows(self, x, rows):
         if isinstance(x, NormedDelta):
-            return NormedDelta(self.gather_rows(x.y, rows), x.weight, x.eps)
+            return x.with_outputs(lambda y: self.gather_rows(y, rows))
         return (x[:, rows.long()] if x.dim() == 3 else x[rows.long()]).contiguous()
 
     # matrix products ---------------------------------------------------------------------
@@ -381,7 +386,7 @@ class TorchOps:
 
     def paged_attention(
         self, qkv, key_pages, value_pages, block_table, ctx, *, num_heads, num_kv_heads, head_dim, block_size, scale, window,
-        defer_merge=False, plan=None, chunk=None, sinks=None, pooled=None, score_bias=None, softcap=None,
+        defer_merge=False, plan=None, chunk=None, sinks=None, pooled=None, score_bias=None, softcap=None, keep_first=0,
     ):
         self._count("paged_attention")
         tokens = qkv.shape[0]
@@ -395,7 +400,7 @@ class TorchOps:
             first = 0 if window is None else max(0, p - window + 1)
             if chunk is not None:
                 first = p // chunk * chunk
-            idx = torch.arange(first, p + 1)
+            idx = torch.cat([torch.arange(min(keep_first, first)), torch.arange(first, p + 1)])
             page = table[r, idx // block_size]
             assert (page >= 0).all(), "attention would read a page that is not there"
             k = key_pages[page, :, idx % block_size, :].float()  # [n, Hkv, d]
@@ -449,10 +454,11 @@ class TorchOps:
     def head_norm_rope_write(
         self, projected, *, heads, kv_heads, head_dim, value_dim, kernel_dim, eps, rotation, slot_mapping, key_pages,
         value_pages, block_size, gated=False, keep_values=False, first_values=None, mix_weight=None, weights=None,
+        values_are_keys=False, temperature=None, projected_column=0,
     ):
         self._count("head_norm_rope_write")
         tokens = projected.shape[0]
-        p = projected.float()
+        p = projected.float()[:, projected_column:]
         a, b = heads * head_dim, (heads + kv_heads) * head_dim
         c = b + kv_heads * value_dim
 
@@ -461,12 +467,15 @@ class TorchOps:
 
         if weights is not None:  # norm and weight before the rotation, values as they are
             q = self._rotate(unit(p[:, :a].view(tokens, heads, head_dim)) * weights[0].float(), rotation)
+            if temperature is not None:
+                positions, every, coef = temperature
+                q = q * (1.0 + coef * torch.log(torch.floor((positions.double() + 1.0) / every) + 1.0)).float()[:, None, None]
             if kv_heads == 0:
                 q_out = torch.zeros(tokens, heads, kernel_dim)
                 q_out[..., :head_dim] = q
                 return q_out.view(tokens, heads * kernel_dim).to(self.dtype), None, None
             k = self._rotate(unit(p[:, a:b].view(tokens, kv_heads, head_dim)) * weights[1].float(), rotation)
-            v = p[:, b:c].view(tokens, kv_heads, value_dim)
+            v = (p[:, a:b] if values_are_keys else p[:, b:c]).view(tokens, kv_heads, value_dim)
         else:
             q = unit(self._rotate(p[:, :a].view(tokens, heads, head_dim), rotation))
             k = unit(self._rotate(p[:, a:b].view(tokens, kv_heads, head_dim), rotation))
@@ -605,8 +614,12 @@ class TorchOps:
     def route_experts(self, logits, correction, *, top, groups, keep_groups, scale, scores="sigmoid", normalise=False):
         self._count("route_experts")
         tokens, experts = logits.shape
-        s = torch.softmax(logits.float(), -1) if scores == "softmax" else torch.sigmoid(logits.float())
-        c = s + correction.float()
+        by_logits = scores == "chosen_softmax"
+        if by_logits:
+            s = logits.float()
+        else:
+            s = torch.softmax(logits.float(), -1) if scores == "softmax" else torch.sigmoid(logits.float())
+        c = s if correction is None else s + correction.float()
         per = experts // groups
         ids = torch.empty(tokens, top, dtype=torch.int32)
         weights = torch.empty(tokens, top, dtype=torch.float32)
@@ -616,18 +629,24 @@ class TorchOps:
             allowed = [e for e in range(experts) if e // per in kept]
             chosen = sorted(allowed, key=lambda e: (-float(c[t, e]), e))[:top]
             total = sum(float(s[t, e]) for e in chosen) + 1e-20 if normalise else 1.0
+            own = torch.softmax(s[t, chosen], -1) if by_logits else s[t, chosen] / total
             for j, e in enumerate(chosen):
                 ids[t, j] = e
-                weights[t, j] = s[t, e] / total * scale
+                weights[t, j] = own[j] * scale
         return ids.to(logits.device), weights.to(logits.device)
 
-    def expert_products(self, h, up_weight, down_weight, ids, weights, *, experts, activation, pass_through=0):
+    def expert_products(
+        self, h, up_weight, down_weight, ids, weights, *, experts, activation, pass_through=0, glu=None, woven=False,
+        beside=None,
+    ):
         self._count("expert_products")
         tokens, hidden = h.shape
         top = ids.shape[1]
         up = up_weight.float().view(experts, -1, hidden)
         down = down_weight.float().view(experts, hidden, -1)
-        out = torch.zeros(top, tokens, hidden, dtype=torch.float32, device=h.device)
+        out = torch.zeros(top + (beside is not None), tokens, hidden, dtype=torch.float32, device=h.device)
+        if beside is not None:
+            out[top] = beside[0].float() @ beside[1].float().t()
         for t in range(tokens):
             for j in range(top):
                 e = int(ids[t, j])
@@ -640,6 +659,15 @@ class TorchOps:
                     z = z.to(self.dtype).float()
                     half = z.shape[0] // 2
                     a = z[:half] * torch.sigmoid(z[:half]) * z[half:]
+                elif activation == "clamped_glu":
+                    limit, alpha = glu
+                    if woven:
+                        quads = z.view(-1, 4)
+                        g, u = quads[:, :2].reshape(-1), quads[:, 2:].reshape(-1)
+                    else:
+                        g, u = z.to(self.dtype).float().chunk(2)
+                    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+                    a = g * torch.sigmoid(alpha * g) * (u + 1.0)
                 else:
                     a = torch.clamp(z, min=0.0) ** 2 if activation == "relu2" else torch.sigmoid(z)
                 out[j, t] = weights[t, j] * (down[e] @ a.to(self.dtype).float())
