@@ -53,6 +53,9 @@ dense feed-forwards with biases and a mixture of gated experts) beside that Qwen
 The points named `delta-*` (`ROFETAR_POINTS`; not among the default points) run the Rofetar decoder (norms on the
 sublayers' outputs; layers of a gated delta rule, attention with capped scores, a state-space recurrence and attention
 that reads the other attention's keys in turn) beside that Qwen2 twin.
+The points named `pair-*` (`GOGUZEN_POINTS`; not among the default points) run the Goguzen decoder (windowed attention
+with kept first tokens, then layers of attention beside a state space; clamped gated experts and a shared one) beside
+the Fedolorn decoder of the same width, heads, layers and vocabulary whose experts hold as many weights a token.
 `reference`: the reference's own published measurements, run here at their parameters with the
 0.5B shape (random weights and token ids of the published lengths; its figures are of an RTX 3060
 laptop GPU in float16 and stand beside for scale): the burst of 8 short requests under continuous and
@@ -112,7 +115,7 @@ def parse_args() -> argparse.Namespace:
     p.add_argument("--no-prefill", action="store_true", help="skip the prefill measurement")
     p.add_argument("--seed", type=int, default=0)
     p.add_argument("--workload", default="decode", choices=("decode", "burst", "chunked", "library", "reference", "designs"))
-    p.add_argument("--design-only", default="", choices=("", "fedolorn", "qwen2", "bubitar", "vobisun", "pepulix", "rofetar"), help="run one of the two designs of the `designs` workload (for profiles)")
+    p.add_argument("--design-only", default="", choices=("", "fedolorn", "qwen2", "bubitar", "vobisun", "pepulix", "rofetar", "goguzen"), help="run one of the two designs of the `designs` workload (for profiles)")
     p.add_argument("--design-points", default="", help="names of the `designs` workload's points to run, comma separated (default: all)")
     p.add_argument("--no-large", action="store_true", help="leave out the 7B and 32B points of the default run")
     p.add_argument("--samples", action="store_true", help="print every raw sample, not only their summary")
@@ -809,6 +812,27 @@ class Bench:
                 pairs = sum(min(t + 1, a.window) + max(0, t - a.window + 1) // a.pool for t in range(tokens))
                 flops += 2 * tokens * per_token + 2 * a.heads * (a.dim + a.vdim) * pairs
             return flops
+        if getattr(config, "architecture", "") == "Goguzen":
+            # per layer: windowed attention (the window's keys and the kept ones), or attention without a value projection
+            # beside a state space (products, convolution, the state's update and read); the router, a token's chosen
+            # experts and the shared one (three matrices each)
+            for layer in config.layers:
+                a, m, per_pair, pairs = layer.mixer, layer.mlp, 0, 0
+                if a.kind == "attention":
+                    per_token = width * (a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)) + a.heads * a.vdim * width
+                    per_pair = a.heads * (a.dim + a.vdim)
+                    size = a.window or tokens
+                    pairs = sum(min(t + 1, size) + min(max(0, t + 1 - size), a.keep_first) for t in range(tokens))
+                else:
+                    left, b = a.left, a.right
+                    per_token = width * (2 * left.heads + left.kv_heads) * left.dim
+                    per_pair, pairs = 2 * left.heads * left.dim, tokens * (tokens + 1) // 2
+                    per_token += width * (2 * b.heads * b.vdim + 2 * b.groups * b.state + b.heads) + b.heads * b.vdim * width
+                    per_token += 2 * b.heads * b.state * b.vdim + b.conv * (b.heads * b.vdim + 2 * b.groups * b.state)
+                if m is not None:
+                    per_token += width * m.experts + 3 * width * (m.top * m.expert.ff + (m.shared.ff if m.shared else 0))
+                flops += 2 * tokens * per_token + 2 * per_pair * pairs
+            return flops
         if getattr(config, "architecture", "") == "Rofetar":
             # per layer: the mixer's products, its (query, visible key) pairs or its state's update and read (the delta
             # rule reads the state twice), and a gated feed-forward of three matrices
@@ -1104,7 +1128,53 @@ def rofetar_configs(name: str) -> dict:
     return {"rofetar": rofetar, "qwen2": qwen2}
 
 
+# The Goguzen decoder beside the Fedolorn decoder: the same width, query and key/value heads, head size, layers,
+# vocabulary and number of experts.  Every third layer is attention over a window of 1,024 tokens and the first 64, the
+# others attention beside a state space (as many heads, values of twice the head size, a state of 128 rows in two
+# groups).  A token uses `top` experts of `ff` and a shared one of 2 ff, three matrices each; its twin's token uses
+# top + 2 experts of two matrices of 1.5 ff: as many weights a token.
+GOGUZEN_POINTS = {
+    # name: (width, heads, kv heads, head size, experts, top, ff, layers run)
+    "pair-896x16e": (896, 14, 2, 64, 16, 4, 800, 12),
+    "pair-2048x64e": (2048, 16, 4, 128, 64, 4, 512, 9),
+    "pair-4096x128e": (4096, 32, 8, 128, 128, 6, 1024, 3),
+}
+
+
+def goguzen_configs(name: str) -> dict:
+    width, heads, kv_heads, dim, experts, top, ff, layers = GOGUZEN_POINTS[name]
+    sizes = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim**-0.5}
+    mlp = {
+        "kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff, "limit": 7.0},
+        "shared": {"ff": 2 * ff, "limit": 7.0},
+    }
+    listed = []
+    for i in range(layers):
+        if i % 3 == 0:
+            rot = {"base": 1000000.0, "dims": dim, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}
+            entry = {"type": "attention", "mixer": {**sizes, "mask": {"size": 1024, "keep_first": 64}, "rot": rot}}
+        else:
+            entry = {"type": "parallel", "mixer": {
+                "left": {**sizes, "q_temp": {"every": 1024, "coef": 0.1}},
+                "right": {"heads": heads, "vdim": 2 * dim, "state": 128, "groups": 2, "conv": 4, "norm_groups": 2},
+            }}
+        listed.append({**entry, "mlp": dict(mlp)})
+    goguzen = {
+        "architecture": "Goguzen", "vocab": DESIGN_VOCAB, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+        "layers": listed, "logit_scale": 0.5, "logit_softcap": 30.0,
+    }
+    twin = {"kind": "moe", "expert": {"ff": 3 * ff // 2},
+            "router": {"experts": experts, "top": top + 2, "scale": 2.0, "groups": {"count": 8, "keep": 4}}}
+    fedolorn = {
+        "architecture": "Fedolorn", "vocab": DESIGN_VOCAB, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+        "layers": [{"type": "attention", "mlp": twin, "mixer": {**sizes, "mask": {"size": 8192}}} for _ in range(layers)],
+    }
+    return {"goguzen": goguzen, "fedolorn": fedolorn}
+
+
 def design_configs(name: str) -> dict:
+    if name in GOGUZEN_POINTS:
+        return goguzen_configs(name)
     if name in ROFETAR_POINTS:
         return rofetar_configs(name)
     if name in PEPULIX_POINTS:
@@ -1157,9 +1227,9 @@ def design_comparison(args) -> dict:
             bench.close()
             print(f"# {name} {design}: {point[design]}", file=sys.stderr, flush=True)
         if len(point) == 2:
-            other = next(d for d in point if d != "qwen2")
-            point["decode_ratio"] = round(point[other]["decode_tokens_per_s"] / point["qwen2"]["decode_tokens_per_s"], 3)
-            point["prefill_ratio"] = round(point[other]["prefill_tokens_per_s"] / point["qwen2"]["prefill_tokens_per_s"], 3)
+            other, twin = list(point)  # the design and the model it is held against
+            point["decode_ratio"] = round(point[other]["decode_tokens_per_s"] / point[twin]["decode_tokens_per_s"], 3)
+            point["prefill_ratio"] = round(point[other]["prefill_tokens_per_s"] / point[twin]["prefill_tokens_per_s"], 3)
         points[name] = point
     return {
         "metric": "decode and prefill tokens/s of two designs at equal sizes",

@@ -184,9 +184,14 @@ def route(logits: torch.Tensor, top: int) -> torch.Tensor:
     return torch.zeros_like(logits).scatter(-1, index, torch.softmax(value, -1))
 
 
-def mixture(w, p: str, f: Mapping, h: torch.Tensor, round_to=None) -> torch.Tensor:
+def mixture(w, p: str, f: Mapping, h: torch.Tensor, round_to=None, margins: Optional[list] = None) -> torch.Tensor:
     hr = _r(h, round_to)
-    weight = route(hr @ w[p + "router"].T + w[p + "router.b"], int(f["router"]["top"]))
+    logits = hr @ w[p + "router"].T + w[p + "router.b"]
+    top = int(f["router"]["top"])
+    if margins is not None and top < logits.shape[1]:  # how far the last chosen expert is from the first that is not
+        ordered = logits.sort(-1, descending=True).values
+        margins.append(ordered[:, top - 1] - ordered[:, top])
+    weight = route(logits, top)
     out = torch.zeros_like(h)
     for e in range(int(f["router"]["experts"])):
         rows = weight[:, e].nonzero()[:, 0]
@@ -202,8 +207,12 @@ def mixture(w, p: str, f: Mapping, h: torch.Tensor, round_to=None) -> torch.Tens
 MIXERS = {"attention": window_attention, "parallel": two_mixers}
 
 
-def forward(config: Mapping, weights: Mapping[str, torch.Tensor], tokens, round_to: Optional[torch.dtype] = None):
-    """logits [T, vocab] and the stream after every layer [layers, T, width]."""
+def forward(
+    config: Mapping, weights: Mapping[str, torch.Tensor], tokens, round_to: Optional[torch.dtype] = None,
+    margins: Optional[list] = None,
+):
+    """logits [T, vocab] and the stream after every layer [layers, T, width].  `margins`: a list that receives, per
+    mixture, how close each token's choice of experts was ([T])."""
     w = weights
     eps = float(config["norm"]["eps"])
     x = w["embed"][torch.as_tensor(tokens, dtype=torch.long)] * float(config["embedding"]["scale"])
@@ -215,7 +224,7 @@ def forward(config: Mapping, weights: Mapping[str, torch.Tensor], tokens, round_
         p = f"l{owner}."
         x = x + MIXERS[layer["type"]](w, p + "mix.", layer["mixer"], rms_norm(x, w[p + "norm1"], eps), eps, round_to)
         if layer.get("mlp") is not None:
-            x = x + mixture(w, p + "mlp.", layer["mlp"], rms_norm(x, w[p + "norm2"], eps), round_to)
+            x = x + mixture(w, p + "mlp.", layer["mlp"], rms_norm(x, w[p + "norm2"], eps), round_to, margins)
         after.append(x)
     logits = (_r(rms_norm(x, w["final.norm"], eps), round_to) @ w["head"].T) * float(config.get("logit_scale", 1.0))
     cap = config.get("logit_softcap")
