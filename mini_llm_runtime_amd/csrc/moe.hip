@@ -145,7 +145,7 @@ __global__ __launch_bounds__(256) void moe_identity_kernel(const T* __restrict__
 
 // ---- pairs sorted by expert ------------------------------------------------------------------
 
-// One workgroup.  counts -> offsets and tiles (thread 0) -> placement.
+// One workgroup.  counts -> offsets and tiles (the first wavefront) -> placement.
 __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__ ids, int pairs, int experts,
                                                          int tile_rows, int max_tiles, int* __restrict__ sorted,
                                                          int* __restrict__ offsets, int* __restrict__ tiles) {
@@ -161,21 +161,38 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__
     if (e >= 0 && e < experts) atomicAdd(&counts[e], 1);
   }
   __syncthreads();
-  if (tid == 0) {
+  if (tid < kWave) {  // the first wavefront: where every expert's run and tiles start, 64 experts at a time
     int at = 0, nt = 0;
-    for (int e = 0; e < experts; ++e) {
-      const int n = counts[e];
-      offsets[e] = at;
-      start[e] = at;
-      for (int r = 0; r < n && nt < max_tiles; r += tile_rows) {
-        tiles[2 * nt] = e;
-        tiles[2 * nt + 1] = at + r;
-        ++nt;
+    for (int e0 = 0; e0 < experts; e0 += kWave) {
+      const int e = e0 + tid;
+      const int n = e < experts ? counts[e] : 0;
+      const int mine = (n + tile_rows - 1) / tile_rows;
+      int rows_upto = n, tiles_upto = mine;  // running sums over the lanes
+#pragma unroll
+      for (int off = 1; off < kWave; off *= 2) {
+        const int r = __shfl_up(rows_upto, off, kWave), t = __shfl_up(tiles_upto, off, kWave);
+        if (tid >= off) {
+          rows_upto += r;
+          tiles_upto += t;
+        }
       }
-      at += n;
+      const int row0 = at + rows_upto - n;
+      const int tile0 = nt + tiles_upto - mine;
+      if (e < experts) {
+        offsets[e] = row0;
+        start[e] = row0;
+        for (int i = 0; i < mine && tile0 + i < max_tiles; ++i) {
+          tiles[2 * (tile0 + i)] = e;
+          tiles[2 * (tile0 + i) + 1] = row0 + i * tile_rows;
+        }
+      }
+      at += __shfl(rows_upto, kWave - 1, kWave);
+      nt += __shfl(tiles_upto, kWave - 1, kWave);
     }
-    offsets[experts] = at;
-    used_tiles = nt;
+    if (tid == 0) {
+      offsets[experts] = at;
+      used_tiles = min(nt, max_tiles);
+    }
   }
   __syncthreads();
   for (int i = used_tiles + tid; i < max_tiles; i += blockDim.x) {

@@ -73,16 +73,17 @@ __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
   const float* cs = cos_t ? cos_t + t * half : nullptr;
   const float* sn = sin_t ? sin_t + t * half : nullptr;
   float q_inv = 1.f, k_inv = 1.f;
+  float q_ss = 0.f, k_ss = 0.f;
   if (q_norm != nullptr) {
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < heads * dim; i += 256) ss += q[i] * q[i];
-    q_inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(heads * dim) + eps);
+#pragma unroll 8
+    for (int i = threadIdx.x; i < heads * dim; i += 256) q_ss += q[i] * q[i];
   }
   if (k_norm != nullptr) {
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < kv_heads * dim; i += 256) ss += k[i] * k[i];
-    k_inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(kv_heads * dim) + eps);
+#pragma unroll 4
+    for (int i = threadIdx.x; i < kv_heads * dim; i += 256) k_ss += k[i] * k[i];
   }
+  if (q_norm != nullptr) q_inv = 1.0f / sqrtf(block_sum(q_ss, scratch) / static_cast<float>(heads * dim) + eps);
+  if (k_norm != nullptr) k_inv = 1.0f / sqrtf(block_sum(k_ss, scratch) / static_cast<float>(kv_heads * dim) + eps);
   // dim j of head `head` of a normed, rotated projection
   auto turned = [&](const float* part, const void* w, float inv, int head, int j) -> float {
     const int at = head * dim + j;
@@ -91,7 +92,10 @@ __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
     return j < half ? normed(at) * cs[j] - normed(at + half) * sn[j]
                     : normed(at) * cs[j - half] + normed(at - half) * sn[j - half];
   };
-  for (int i = threadIdx.x; i < heads * D; i += 256) {
+  // gridDim.y workgroups share a token's outputs (each has summed the squares for itself)
+  const int step = 256 * gridDim.y;
+  const int mine = blockIdx.y * 256 + threadIdx.x;
+  for (int i = mine; i < heads * D; i += step) {
     const int hd = i / D;
     const int j = i - hd * D;
     float val = 0.f;
@@ -106,7 +110,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
     const int page = slot / block_size;
     const int off = slot - page * block_size;
     if (page < num_pages) {
-      for (int i = threadIdx.x; i < kv_heads * D; i += 256) {
+      for (int i = mine; i < kv_heads * D; i += step) {
         const int g = i / D;
         const int j = i - g * D;
         const int64_t head_base = (static_cast<int64_t>(page) * kv_heads + g) * block_size * D;
@@ -115,7 +119,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
       }
     }
   }
-  if (gated) {
+  if (gated && blockIdx.y == 0) {
     const float* logits = v + kv_heads * vdim;
     for (int hd = threadIdx.x; hd < heads; hd += 256) gate[t * heads + hd] = 1.0f / (1.0f + expf(-logits[hd]));
   }
@@ -578,13 +582,15 @@ int mlr_qk_norm_rope_write(const float* projected, int width, const void* q_norm
   MLR_REQUIRE(width >= heads * dim + kv_heads * (dim + vdim) + (gated ? heads : 0), "the projected rows are too narrow");
   MLR_REQUIRE(block_size > 0 && num_pages > 0, "pages must exist");
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
+  // few tokens: a token's heads spread over workgroups; many: a workgroup takes a token
+  const dim3 grid(tokens, tokens <= 256 ? min((heads * head_dim + 255) / 256, 16) : 1);
   if (dtype == kF32)
-    qk_norm_rope_write_kernel<float><<<tokens, 256, 0, stream>>>(
+    qk_norm_rope_write_kernel<float><<<grid, 256, 0, stream>>>(
         projected, width, q_norm, k_norm, weight_is_f32, eps, head_scale, rotary_dim ? cos_t : nullptr,
         rotary_dim ? sin_t : nullptr, rotary_dim, slots, static_cast<float*>(key_pages), static_cast<float*>(value_pages),
         static_cast<float*>(q_out), gate, heads, kv_heads, dim, vdim, head_dim, block_size, num_pages, gated);
   else
-    qk_norm_rope_write_kernel<bf16><<<tokens, 256, 0, stream>>>(
+    qk_norm_rope_write_kernel<bf16><<<grid, 256, 0, stream>>>(
         projected, width, q_norm, k_norm, weight_is_f32, eps, head_scale, rotary_dim ? cos_t : nullptr,
         rotary_dim ? sin_t : nullptr, rotary_dim, slots, static_cast<bf16*>(key_pages), static_cast<bf16*>(value_pages),
         static_cast<bf16*>(q_out), gate, heads, kv_heads, dim, vdim, head_dim, block_size, num_pages, gated);
