@@ -89,6 +89,31 @@ __host__ __device__ inline int first_visible_key(int p, int window, int chunk) {
   return window > 0 ? (p - window + 1 > 0 ? p - window + 1 : 0) : 0;
 }
 
+// A workgroup of THREADS threads copies `count` floats into LDS, eight loads a thread on their way at once; the caller
+// synchronises.
+template <int THREADS>
+__device__ __forceinline__ void stage_floats(const float* __restrict__ src, float* lds, int count) {
+  for (int i0 = threadIdx.x; i0 < count; i0 += 8 * THREADS) {
+    float v[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) v[u] = src[min(i0 + u * THREADS, count - 1)];
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+      if (i0 + u * THREADS < count) lds[i0 + u * THREADS] = v[u];
+  }
+}
+
+constexpr int kStagedRowFloats = 12288;  // the longest row a workgroup stages (48 KB: three workgroups fit a compute unit)
+
+// Which token a workgroup of a long token list takes.  Workgroups go to the 8 dies in turn; taken in order, the
+// tokens of one cache page, whose values lie side by side in the page's rows, would be written through 8 separate
+// L2 caches, a few bytes of every line each.  So each die gets 16 consecutive tokens of every 128.
+__device__ inline int64_t token_of_workgroup(int block, int count) {
+  const int whole = count / 128 * 128;
+  if (block >= whole) return block;
+  return block / 128 * 128 + block % 8 * 16 + block / 8 % 16;
+}
+
 // With a window whose queries also see the first `keep` positions of their request, what a query at position p sees
 // is two ranges: 0 .. kept - 1 and first .. p, disjoint.  Where they meet they are one (kept = 0, first = 0).
 struct VisibleKeys {

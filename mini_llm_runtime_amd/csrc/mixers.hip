@@ -74,8 +74,18 @@ __global__ __launch_bounds__(256) void add_normed_kernel(float* __restrict__ x, 
     orow[i] = from_f32<T>(load_as_f32(next_weight, i, next_is_f32) * (row_lds[i] * inv2));
 }
 
-// The same for rows whose width is a multiple of 4 and fits the registers of a workgroup: a thread keeps
-// VPT groups of 4 elements between the passes, and all loads of a pass (every slice of partial sums
+// Four neighbouring numbers, float32 or bfloat16, with one load (i is a multiple of 4, p aligned to 16 bytes).
+__device__ __forceinline__ f32x4v load4_as_f32(const void* p, int64_t i, int is_f32) {
+  if (is_f32) return *reinterpret_cast<const f32x4v*>(static_cast<const float*>(p) + i);
+  const u16x4_t bits = *reinterpret_cast<const u16x4_t*>(static_cast<const bf16*>(p) + i);
+  f32x4v v;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[e] = __builtin_bit_cast(float, static_cast<uint32_t>(bits[e]) << 16);
+  return v;
+}
+
+// The same for rows whose width is a multiple of 4 and fits the registers of a workgroup (operands aligned to 16
+// bytes): a thread keeps VPT groups of 4 elements between the passes, and all loads of a pass (every slice of partial sums
 // included) are issued before the first is used: the kernel's time is the latency of its loads.
 template <typename T, int VPT, int THREADS, bool TWO>
 __global__ __launch_bounds__(THREADS) void add_normed_rows_kernel(float* __restrict__ x, NormedOutput first,
@@ -94,21 +104,12 @@ __global__ __launch_bounds__(THREADS) void add_normed_rows_kernel(float* __restr
     const int i = min(static_cast<int>(threadIdx.x) + j * THREADS, quads - 1);
     const int64_t at = row * hidden + 4 * i;
     xv[j] = *reinterpret_cast<const f32x4v*>(x + at);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) nv[j][e] = mode == 1 ? load_as_f32(next_weight, 4 * i + e, next_is_f32) : 0.f;
+    nv[j] = mode == 1 ? load4_as_f32(next_weight, 4 * i, next_is_f32) : f32x4v{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int which = 0; which < kCount; ++which) {
       const NormedOutput& a = which == 0 ? first : second;
-#pragma unroll
-      for (int e = 0; e < 4; ++e) wv[which][j][e] = load_as_f32(a.weight, 4 * i + e, a.weight_is_f32);
-      if (a.slices > 0) {
-        v[which][j] = f32x4v{0.f, 0.f, 0.f, 0.f};
-      } else if (a.is_f32) {
-        v[which][j] = *reinterpret_cast<const f32x4v*>(static_cast<const float*>(a.y) + at);
-      } else {
-#pragma unroll
-        for (int e = 0; e < 4; ++e) v[which][j][e] = to_f32(static_cast<const T*>(a.y)[at + e]);
-      }
+      wv[which][j] = load4_as_f32(a.weight, 4 * i, a.weight_is_f32);
+      v[which][j] = a.slices > 0 ? f32x4v{0.f, 0.f, 0.f, 0.f} : load4_as_f32(a.y, at, a.is_f32);
     }
   }
 #pragma unroll
@@ -173,8 +174,15 @@ __global__ __launch_bounds__(THREADS) void add_normed_rows_kernel(float* __restr
     const int i = threadIdx.x + j * THREADS;
     if (i >= quads) continue;
     const int64_t at = row * hidden + 4 * i;
+    f32x4v r;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) out[at + e] = from_f32<T>(mode == 1 ? nv[j][e] * (xv[j][e] * inv2) : xv[j][e]);
+    for (int e = 0; e < 4; ++e) r[e] = mode == 1 ? nv[j][e] * (xv[j][e] * inv2) : xv[j][e];
+    if constexpr (sizeof(T) == 4) {
+      *reinterpret_cast<f32x4v*>(out + at) = r;
+    } else {
+      const u16x4_t bits = {f32_to_bf16(r[0]).bits, f32_to_bf16(r[1]).bits, f32_to_bf16(r[2]).bits, f32_to_bf16(r[3]).bits};
+      *reinterpret_cast<u16x4_t*>(out + at) = bits;
+    }
   }
 }
 
@@ -187,7 +195,11 @@ static void launch_add_normed(float* x, const NormedOutput& first, const NormedO
 #define MLR_ROWS(VPT, THREADS)                                                                                   \
   add_normed_rows_kernel<T, VPT, THREADS, TWO><<<rows, THREADS, 0, stream>>>(x, first, second, rows, eps, next_weight, \
                                                                              next_is_f32, next_eps, mode, o, hidden)
-  if (hidden % 4 != 0 || quads > 2048)
+  const uintptr_t places = reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(first.y) |
+                           reinterpret_cast<uintptr_t>(first.weight) | reinterpret_cast<uintptr_t>(second.y) |
+                           reinterpret_cast<uintptr_t>(second.weight) | reinterpret_cast<uintptr_t>(next_weight) |
+                           reinterpret_cast<uintptr_t>(out);
+  if (hidden % 4 != 0 || quads > 2048 || places % 16 != 0)
     add_normed_kernel<T, TWO><<<rows, 256, static_cast<size_t>(hidden) * sizeof(float) * (TWO ? 2 : 1), stream>>>(
         x, first, second, rows, eps, next_weight, next_is_f32, next_eps, mode, o, hidden);
   else if (rows <= 64 && quads > 512)

@@ -56,8 +56,9 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ h
 //    [page, kv_head, offset, D] and the value pages [page, kv_head, D, offset]; dims beyond dim / vdim are
 //    zeros; a negative slot stores nothing,
 //  * gate[t, head] = sigmoid(logit), float32.
-// Everything in float32, one rounding.
-template <typename T>
+// Everything in float32, one rounding.  STAGED: the row is copied into LDS first (steps of many tokens, where a workgroup
+// takes a whole token: its passes over the row would be as many trips to memory one after the other).
+template <typename T, bool STAGED>
 __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
     const float* __restrict__ p, int width, const void* __restrict__ q_norm, const void* __restrict__ k_norm,
     int weight_is_f32, float eps, const float* __restrict__ head_scale, const float* __restrict__ cos_t,
@@ -65,8 +66,14 @@ __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
     T* __restrict__ value_pages, T* __restrict__ q_out, float* __restrict__ gate, int heads, int kv_heads, int dim,
     int vdim, int D, int block_size, int num_pages, int gated) {
   __shared__ float scratch[16];
-  const int64_t t = blockIdx.x;
+  const int64_t t = token_of_workgroup(blockIdx.x, gridDim.x);
+  extern __shared__ float qk_row[];
   const float* q = p + t * width;
+  if constexpr (STAGED) {
+    stage_floats<256>(q, qk_row, heads * dim + kv_heads * (dim + vdim) + (gated ? heads : 0));
+    __syncthreads();
+    q = qk_row;
+  }
   const float* k = q + heads * dim;
   const float* v = k + kv_heads * dim;
   const int half = rdims / 2;
@@ -584,16 +591,25 @@ int mlr_qk_norm_rope_write(const float* projected, int width, const void* q_norm
   MLR_REQUIRE(dtype == kF32 || dtype == kBF16, "dtype must be 0 (float32) or 1 (bfloat16)");
   // few tokens: a token's heads spread over workgroups; many: a workgroup takes a token
   const dim3 grid(tokens, tokens <= 256 ? min((heads * head_dim + 255) / 256, 16) : 1);
-  if (dtype == kF32)
-    qk_norm_rope_write_kernel<float><<<grid, 256, 0, stream>>>(
-        projected, width, q_norm, k_norm, weight_is_f32, eps, head_scale, rotary_dim ? cos_t : nullptr,
-        rotary_dim ? sin_t : nullptr, rotary_dim, slots, static_cast<float*>(key_pages), static_cast<float*>(value_pages),
-        static_cast<float*>(q_out), gate, heads, kv_heads, dim, vdim, head_dim, block_size, num_pages, gated);
-  else
-    qk_norm_rope_write_kernel<bf16><<<grid, 256, 0, stream>>>(
-        projected, width, q_norm, k_norm, weight_is_f32, eps, head_scale, rotary_dim ? cos_t : nullptr,
-        rotary_dim ? sin_t : nullptr, rotary_dim, slots, static_cast<bf16*>(key_pages), static_cast<bf16*>(value_pages),
-        static_cast<bf16*>(q_out), gate, heads, kv_heads, dim, vdim, head_dim, block_size, num_pages, gated);
+  const int own = heads * dim + kv_heads * (dim + vdim) + (gated ? heads : 0);
+  const bool staged = tokens > 256 && own <= kStagedRowFloats;
+#define MLR_QK_NORM(T, STAGED)                                                                                          \
+  qk_norm_rope_write_kernel<T, STAGED><<<grid, 256, STAGED ? own * sizeof(float) : 0, stream>>>(                        \
+      projected, width, q_norm, k_norm, weight_is_f32, eps, head_scale, rotary_dim ? cos_t : nullptr,                   \
+      rotary_dim ? sin_t : nullptr, rotary_dim, slots, static_cast<T*>(key_pages), static_cast<T*>(value_pages),        \
+      static_cast<T*>(q_out), gate, heads, kv_heads, dim, vdim, head_dim, block_size, num_pages, gated)
+  if (dtype == kF32) {
+    if (staged)
+      MLR_QK_NORM(float, true);
+    else
+      MLR_QK_NORM(float, false);
+  } else {
+    if (staged)
+      MLR_QK_NORM(bf16, true);
+    else
+      MLR_QK_NORM(bf16, false);
+  }
+#undef MLR_QK_NORM
   MLR_LAUNCH_CHECK();
   return 0;
 }

@@ -202,7 +202,8 @@ __global__ __launch_bounds__(256) void streams_fill_kernel(const float* __restri
 // weight BEFORE it turns, and the values are stored as they are.  kv_heads 0: the rows hold queries only.
 // values_are_keys (weighted norms, vdim = dim): the rows hold no values, the keys' sums before their norm are stored as
 // values too.  positions given: queries are multiplied by 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1).
-template <typename T>
+// STAGED: as in qk_norm_rope_write_kernel.
+template <typename T, bool STAGED>
 __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
     const float* __restrict__ p, int width, T* __restrict__ q_out, float* __restrict__ gate,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rdims, float eps,
@@ -210,10 +211,16 @@ __global__ __launch_bounds__(256) void head_norm_rope_write_kernel(
     const float* __restrict__ v_first, const float* __restrict__ lambda_p, const void* __restrict__ q_weight,
     const void* __restrict__ k_weight, int weight_is_f32, int values_are_keys, const int* __restrict__ positions,
     double temp_every, float temp_coef, int heads, int kv_heads, int dim, int vdim, int D, int block_size, int num_pages) {
-  const int64_t t = blockIdx.x;
+  const int64_t t = token_of_workgroup(blockIdx.x, gridDim.x);
   const int lane = threadIdx.x % kWave;
   const int wave = threadIdx.x / kWave;
+  extern __shared__ float head_row[];
   const float* row = p + t * width;
+  if constexpr (STAGED) {
+    stage_floats<256>(row, head_row, (heads + kv_heads) * dim + (values_are_keys ? 0 : kv_heads * vdim) + (gate != nullptr ? heads : 0));
+    __syncthreads();
+    row = head_row;
+  }
   const int half = rdims / 2;
   const float* cs = cos_t != nullptr ? cos_t + t * half : nullptr;
   const float* sn = sin_t != nullptr ? sin_t + t * half : nullptr;
@@ -628,18 +635,25 @@ int mlr_head_norm_rope_write(const float* projected, int width, void* q_out, flo
   // few tokens: every wavefront one head; many: a workgroup takes a token's heads in turn
   const dim3 grid(tokens, tokens <= 256 ? (heads + 2 * kv_heads + 3) / 4 : 1);
   MLR_REQUIRE(grid.y < 65536u, "too many heads for one launch");
-  if (dtype == kF32)
-    head_norm_rope_write_kernel<float><<<grid, 256, 0, stream>>>(
-        projected, width, static_cast<float*>(q_out), gate, cos, sin, rotary_dims, eps, slots,
-        static_cast<float*>(key_pages), static_cast<float*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight,
-        weight_is_f32, values_are_keys, positions, temp_every, temp_coef, heads, kv_heads, dim, vdim, kernel_dim, block_size,
-        num_pages);
-  else
-    head_norm_rope_write_kernel<bf16><<<grid, 256, 0, stream>>>(
-        projected, width, static_cast<bf16*>(q_out), gate, cos, sin, rotary_dims, eps, slots,
-        static_cast<bf16*>(key_pages), static_cast<bf16*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight,
-        weight_is_f32, values_are_keys, positions, temp_every, temp_coef, heads, kv_heads, dim, vdim, kernel_dim, block_size,
-        num_pages);
+  const int own = (heads + kv_heads) * dim + (values_are_keys ? 0 : kv_heads * vdim) + (gate ? heads : 0);
+  const bool staged = tokens > 256 && own <= kStagedRowFloats;
+#define MLR_HEAD_NORM(T, STAGED)                                                                                       \
+  head_norm_rope_write_kernel<T, STAGED><<<grid, 256, STAGED ? own * sizeof(float) : 0, stream>>>(                     \
+      projected, width, static_cast<T*>(q_out), gate, cos, sin, rotary_dims, eps, slots, static_cast<T*>(key_pages),   \
+      static_cast<T*>(value_pages), v_keep, v_first, lambda, q_weight, k_weight, weight_is_f32, values_are_keys,       \
+      positions, temp_every, temp_coef, heads, kv_heads, dim, vdim, kernel_dim, block_size, num_pages)
+  if (dtype == kF32) {
+    if (staged)
+      MLR_HEAD_NORM(float, true);
+    else
+      MLR_HEAD_NORM(float, false);
+  } else {
+    if (staged)
+      MLR_HEAD_NORM(bf16, true);
+    else
+      MLR_HEAD_NORM(bf16, false);
+  }
+#undef MLR_HEAD_NORM
   MLR_LAUNCH_CHECK();
   return 0;
 }
