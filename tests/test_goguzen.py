@@ -447,7 +447,7 @@ def _step_context(lengths, starts, ops):
     )
 
 
-MASKS = [(10, 3), (72, 6), (64, 64), (100, 33), (5, 90), (1, 1), (300, 17), (40, 200), (16, 16)]
+MASKS = [(10, 3), (75, 7), (64, 64), (100, 33), (5, 90), (1, 1), (300, 17), (40, 200), (16, 16)]
 
 
 @pytest.mark.parametrize("dtype", GPU_CASES)
@@ -572,7 +572,7 @@ def test_two_outputs_normed_before_they_are_added(dtype, rows, hidden, slices):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("experts,top", [(1, 1), (12, 4), (7, 7), (64, 6), (200, 8)])
+@pytest.mark.parametrize("experts,top", [(1, 1), (13, 4), (7, 7), (64, 6), (200, 8)])
 def test_softmax_over_the_chosen_logits(experts, top):
     hip, double = _ops("hip", torch.float32), TorchOps(torch.float32, "cpu")
     g = torch.Generator().manual_seed(experts)
